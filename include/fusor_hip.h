@@ -51,7 +51,7 @@ enum {
 /* GgmlType ids, fusor-ml/gguf/src/lib.rs:35-50.  Q4_0, Q8_0, Q4_K and Q6_K weights are re-laid-out for the
  * matrix-core kernels; Q5_0, Q5_K and dense F32 (0) / F16 (1) weights keep the file's layout and run through
  * the per-element kernels (every fh_qmatrix_* call, fh_embed_rows, fh_qmatmul, fh_qmatmul_add2 / _swiglu). */
-enum { FH_Q4_0 = 2, FH_Q5_0 = 6, FH_Q8_0 = 8, FH_Q4_K = 12, FH_Q5_K = 13, FH_Q6_K = 14 };
+enum { FH_Q4_0 = 2, FH_Q5_0 = 6, FH_Q8_0 = 8, FH_Q4_K = 12, FH_Q5_K = 13, FH_Q6_K = 14, FH_BF16 = 30 };
 
 /* MaskKind, fusor-ml/fusor/src/composite/flash_attention.rs:12-24 */
 enum { FH_MASK_NONE = 0, FH_MASK_CAUSAL = 1, FH_MASK_ADDITIVE = 2 /* QKMask [sq, skv] */,
@@ -64,6 +64,7 @@ typedef struct fh_device fh_device;
 typedef struct fh_qmatrix fh_qmatrix;
 typedef struct fh_kvcache fh_kvcache;
 typedef struct fh_llama fh_llama;
+typedef struct fh_decoder fh_decoder;
 typedef struct fh_graph fh_graph;
 typedef struct fh_gguf fh_gguf;
 
@@ -199,6 +200,15 @@ typedef struct {
     float factor, high_freq_factor, low_freq_factor;
     int32_t original_max_position_embeddings;
 } fh_rope_scaling;
+/* YaRN scaling of `dims` rotated dimensions: rotations that turn at least `fast` times within `original` positions keep
+ * their frequency, those that turn at most `slow` times are slowed down by `factor`, a ramp over the pair index joins
+ * them, and cos and sin carry the factor 0.1 ln(factor) + 1.  scaling NULL: plain frequencies base^(-2i/dims).  The
+ * tables are [ctx, dims/2].  No counterpart in the reference. */
+typedef struct {
+    float factor, original, fast, slow;
+} fh_yarn_scaling;
+fh_status fh_rope_tables_yarn(fh_device *dev, int32_t dims, int32_t ctx, double base, const fh_yarn_scaling *scaling,
+                              float *cos_dev, float *sin_dev);
 fh_status fh_rope_tables_scaled(fh_device *dev, int32_t head_dim, int32_t ctx, float theta,
                                 const fh_rope_scaling *scaling, const float *freq_weight_host,
                                 float *cos_dev, float *sin_dev);
@@ -472,6 +482,42 @@ fh_status fh_llama_config_from_gguf(const fh_gguf *g, fh_llama_config *cfg);
 /* Load every decoder tensor of the file (raw/mod.rs:418-604: token_embd, output_norm, output,
  * rope_freqs, blk.N.*); f16 vectors are widened to f32.  Call fh_llama_finalize afterwards. */
 fh_status fh_llama_load_gguf(fh_llama *m, const fh_gguf *g);
+
+/* ---------------------------------------------------------------- any decoder
+ * The handle all decoder families share.  fh_llama_decoder gives that of a Llama decoder (owned by the fh_llama);
+ * fh_decoder_create / _open make one for a model that comes as a configuration text and a safetensors file, by the
+ * configuration's "architecture" (registered: "Fidasun", whose configuration lists its layers).  dtype: FH_F32
+ * (everything in 32 bits) or FH_DECODER_BF16 (operands of the matrix products in bf16; sums, scores, norms, routers,
+ * recurrent states and the residual stream in 32 bits). */
+enum { FH_DECODER_BF16 = 2 };
+fh_status fh_llama_decoder(fh_llama *m, fh_decoder **out);
+fh_status fh_decoder_create(fh_device *dev, const char *config_json, int32_t dtype, int32_t ctx, fh_decoder **out);
+/* A folder with config.json and model.safetensors, loaded and finalized. */
+fh_status fh_decoder_open(fh_device *dev, const char *dir, int32_t dtype, int32_t ctx, fh_decoder **out);
+/* One tensor by its name in the file; k 0 for vectors; ggml_type 0 (F32), 1 (F16), 30 (BF16; matrices must be BF16). */
+fh_status fh_decoder_load_tensor(fh_decoder *m, const char *name, uint32_t ggml_type, int64_t n, int64_t k,
+                                 const void *bytes, size_t len);
+fh_status fh_decoder_finalize(fh_decoder *m);
+fh_status fh_decoder_destroy(fh_decoder *m); /* not for a handle from fh_llama_decoder */
+fh_status fh_decoder_info(const fh_decoder *m, int32_t *vocab, int32_t *d_model, int32_t *n_layers, int32_t *ctx,
+                          int32_t *position);
+/* Ends the sequence: the next forward pass starts at position 0. */
+fh_status fh_decoder_reset(fh_decoder *m);
+/* Run `count` new tokens at the current position (long prompts in portions, the context trimmed as fh_llama_forward
+ * does).  want_host: the n_want places among these tokens whose logits are asked for, logits_host [n_want, vocab]; NULL:
+ * the last one.  hidden_host (optional): the final-norm state of the last wanted token. */
+fh_status fh_decoder_forward(fh_decoder *m, const uint32_t *tokens_host, int32_t count, const int32_t *want_host,
+                             int32_t n_want, float *logits_host, float *hidden_host);
+/* As fh_llama_decode_greedy / fh_llama_decode_sampled. */
+fh_status fh_decoder_decode_greedy(fh_decoder *m, uint32_t first_token, int32_t steps, uint32_t *out_tokens_host,
+                                   float *elapsed_ms);
+fh_status fh_decoder_decode_sampled(fh_decoder *m, uint32_t first_token, int32_t steps, const fh_sampler_params *params,
+                                    const float *randoms_host, const uint32_t *previous_host, uint32_t n_previous,
+                                    uint32_t repetition_range, float *mu, uint32_t *out_tokens_host, float *elapsed_ms);
+fh_status fh_decoder_weight_bytes(const fh_decoder *m, uint64_t *bytes);
+/* Keep the residual stream behind every layer of each forward pass; [tokens, d_model] of the last portion per layer. */
+fh_status fh_decoder_keep_layers(fh_decoder *m, int32_t on);
+fh_status fh_decoder_layer_output(fh_decoder *m, int32_t layer, float *out_host, int64_t count);
 
 #if defined(__GNUC__)
 #pragma GCC visibility pop

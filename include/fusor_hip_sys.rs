@@ -37,6 +37,7 @@ pub const FH_Q8_0: u32 = 8;
 pub const FH_Q4_K: u32 = 12;
 pub const FH_Q5_K: u32 = 13;
 pub const FH_Q6_K: u32 = 14;
+pub const FH_BF16: u32 = 30;
 
 /// `MaskKind` (fusor-ml/fusor/src/composite/flash_attention.rs:12-24)
 pub const FH_MASK_NONE: i32 = 0;
@@ -48,6 +49,8 @@ pub const FH_MASK_BATCH_KEY: i32 = 3;
 /// element types of attention operands and of the KV cache
 pub const FH_F32: i32 = 0;
 pub const FH_F16: i32 = 1;
+/// decoders of dense bf16 weights: operands of the matrix products in bf16
+pub const FH_DECODER_BF16: i32 = 2;
 
 /// `GgufMetadataValueType` ids (fusor-ml/gguf/src/lib.rs:349-379)
 pub const FH_GGUF_U8: u32 = 0;
@@ -68,7 +71,7 @@ pub const FH_GGUF_MAX_RANK: usize = 8;
 macro_rules! opaque {
     ($($name:ident),*) => { $(#[repr(C)] pub struct $name { _private: [u8; 0] })* };
 }
-opaque!(FhDevice, FhQMatrix, FhKvCache, FhLlama, FhGraph, FhGguf);
+opaque!(FhDevice, FhQMatrix, FhKvCache, FhLlama, FhDecoder, FhGraph, FhGguf);
 
 /// `fh_llama_config`
 #[repr(C)]
@@ -110,6 +113,16 @@ pub struct FhRopeScaling {
     pub high_freq_factor: f32,
     pub low_freq_factor: f32,
     pub original_max_position_embeddings: i32,
+}
+
+/// YaRN scaling of the rotation frequencies (`fh_rope_tables_yarn`)
+#[repr(C)]
+#[derive(Clone, Copy, Debug)]
+pub struct FhYarnScaling {
+    pub factor: f32,
+    pub original: f32,
+    pub fast: f32,
+    pub slow: f32,
 }
 
 /// `fh_sampler_params` (`GpuStandardSamplerParams` / `GpuMirostat2SamplerParams`, fusor-ml/core/src/sampling/mod.rs:96-114)
@@ -227,6 +240,21 @@ extern "C" {
     pub fn fh_llama_weight_bytes(m: *const FhLlama, bytes: *mut u64) -> FhStatus;
     pub fn fh_llama_config_from_gguf(g: *const FhGguf, cfg: *mut FhLlamaConfig) -> FhStatus;
     pub fn fh_llama_load_gguf(m: *mut FhLlama, g: *const FhGguf) -> FhStatus;
+    pub fn fh_rope_tables_yarn(dev: *mut FhDevice, dims: i32, ctx: i32, base: f64, scaling: *const FhYarnScaling, cos_dev: *mut f32, sin_dev: *mut f32) -> FhStatus;
+    pub fn fh_llama_decoder(m: *mut FhLlama, out: *mut *mut FhDecoder) -> FhStatus;
+    pub fn fh_decoder_create(dev: *mut FhDevice, config_json: *const c_char, dtype: i32, ctx: i32, out: *mut *mut FhDecoder) -> FhStatus;
+    pub fn fh_decoder_open(dev: *mut FhDevice, dir: *const c_char, dtype: i32, ctx: i32, out: *mut *mut FhDecoder) -> FhStatus;
+    pub fn fh_decoder_load_tensor(m: *mut FhDecoder, name: *const c_char, ggml_type: u32, n: i64, k: i64, bytes: *const c_void, len: usize) -> FhStatus;
+    pub fn fh_decoder_finalize(m: *mut FhDecoder) -> FhStatus;
+    pub fn fh_decoder_destroy(m: *mut FhDecoder) -> FhStatus;
+    pub fn fh_decoder_info(m: *const FhDecoder, vocab: *mut i32, d_model: *mut i32, n_layers: *mut i32, ctx: *mut i32, position: *mut i32) -> FhStatus;
+    pub fn fh_decoder_reset(m: *mut FhDecoder) -> FhStatus;
+    pub fn fh_decoder_forward(m: *mut FhDecoder, tokens_host: *const u32, count: i32, want_host: *const i32, n_want: i32, logits_host: *mut f32, hidden_host: *mut f32) -> FhStatus;
+    pub fn fh_decoder_decode_greedy(m: *mut FhDecoder, first_token: u32, steps: i32, out_tokens_host: *mut u32, elapsed_ms: *mut f32) -> FhStatus;
+    pub fn fh_decoder_decode_sampled(m: *mut FhDecoder, first_token: u32, steps: i32, params: *const FhSamplerParams, randoms_host: *const f32, previous_host: *const u32, n_previous: u32, repetition_range: u32, mu: *mut f32, out_tokens_host: *mut u32, elapsed_ms: *mut f32) -> FhStatus;
+    pub fn fh_decoder_weight_bytes(m: *const FhDecoder, bytes: *mut u64) -> FhStatus;
+    pub fn fh_decoder_keep_layers(m: *mut FhDecoder, on: i32) -> FhStatus;
+    pub fn fh_decoder_layer_output(m: *mut FhDecoder, layer: i32, out_host: *mut f32, count: i64) -> FhStatus;
 }
 
 /// The message of the last failed call on this thread.

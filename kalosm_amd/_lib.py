@@ -12,9 +12,10 @@ LIB_PATH = os.path.join(HERE, "libfusor_hip.so")
 
 FH_OK, FH_ERR_INVALID, FH_ERR_HIP, FH_ERR_UNSUPPORTED, FH_ERR_OOM, FH_ERR_NO_DEVICE = 0, -1, -2, -3, -4, -5
 FH_ERR_IO, FH_ERR_NOT_FOUND = -6, -7
-Q4_0, Q8_0, Q4_K, Q6_K = 2, 8, 12, 14
+Q4_0, Q8_0, Q4_K, Q6_K, BF16 = 2, 8, 12, 14, 30
 MASK_NONE, MASK_CAUSAL, MASK_ADDITIVE = 0, 1, 2
 F32, F16 = 0, 1
+DECODER_BF16 = 2
 
 
 class FusorHipError(RuntimeError):
@@ -37,6 +38,10 @@ class FiniteStats(C.Structure):
 class RopeScaling(C.Structure):
     _fields_ = [("factor", C.c_float), ("high_freq_factor", C.c_float), ("low_freq_factor", C.c_float),
                 ("original_max_position_embeddings", C.c_int32)]
+
+
+class YarnScaling(C.Structure):
+    _fields_ = [("factor", C.c_float), ("original", C.c_float), ("fast", C.c_float), ("slow", C.c_float)]
 
 
 class SamplerParams(C.Structure):
@@ -130,6 +135,22 @@ SIGNATURES = {
     "fh_llama_load_gguf": [_p, _p],
     "fh_rope_tables_weighted": [_p, _i32, _i32, _f32, _p, _p, _p],
     "fh_rope_tables_scaled": [_p, _i32, _i32, _f32, C.POINTER(RopeScaling), _p, _p, _p],
+    "fh_rope_tables_yarn": [_p, _i32, _i32, C.c_double, C.POINTER(YarnScaling), _p, _p],
+    "fh_llama_decoder": [_p, _pp],
+    "fh_decoder_create": [_p, C.c_char_p, _i32, _i32, _pp],
+    "fh_decoder_open": [_p, C.c_char_p, _i32, _i32, _pp],
+    "fh_decoder_load_tensor": [_p, C.c_char_p, _u32, _i64, _i64, _p, _sz],
+    "fh_decoder_finalize": [_p],
+    "fh_decoder_destroy": [_p],
+    "fh_decoder_info": [_p] + [C.POINTER(_i32)] * 5,
+    "fh_decoder_reset": [_p],
+    "fh_decoder_forward": [_p, _p, _i32, _p, _i32, _p, _p],
+    "fh_decoder_decode_greedy": [_p, _u32, _i32, _p, C.POINTER(_f32)],
+    "fh_decoder_decode_sampled": [_p, _u32, _i32, C.POINTER(SamplerParams), _p, _p, _u32, _u32, C.POINTER(_f32), _p,
+                                  C.POINTER(_f32)],
+    "fh_decoder_weight_bytes": [_p, C.POINTER(_u64)],
+    "fh_decoder_keep_layers": [_p, _i32],
+    "fh_decoder_layer_output": [_p, _i32, _p, _i64],
     "fh_gguf_open": [C.c_char_p, _pp],
     "fh_gguf_open_memory": [_p, _sz, _pp],
     "fh_gguf_close": [_p],

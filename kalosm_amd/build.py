@@ -2,6 +2,7 @@
 shared library beside this file.  Run as `python -m kalosm_amd.build` or through `__graft_entry__.build()`."""
 from __future__ import annotations
 
+import fcntl
 import glob
 import os
 import subprocess
@@ -45,12 +46,24 @@ def build(jobs: int = 8, verbose: bool = True) -> str:
         raise RuntimeError("no sources under " + CSRC)
     with ThreadPoolExecutor(max_workers=jobs) as ex:
         objs = list(ex.map(_compile, srcs))
-    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB, *objs, "-Wl,--no-undefined"]
+    part = LIB + f".{os.getpid()}"
+    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", part, *objs, "-Wl,--no-undefined"]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"link failed:\n{r.stdout}\n{r.stderr}")
+    os.replace(part, LIB)
     if verbose:
         print(f"built {LIB} from {len(srcs)} sources")
+    return LIB
+
+
+def ensure() -> str:
+    """The library, built first when it is not there (one process builds, others wait)."""
+    if not os.path.exists(LIB):
+        with open(os.path.join(HERE, ".build.lock"), "w") as lock:
+            fcntl.flock(lock, fcntl.LOCK_EX)
+            if not os.path.exists(LIB):
+                build(jobs=min(16, os.cpu_count() or 1), verbose=False)
     return LIB
 
 

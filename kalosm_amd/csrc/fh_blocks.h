@@ -170,10 +170,15 @@ __device__ __forceinline__ float deq_elem_f32(const QView &q, int64_t row, int64
     return ((const float *)q.data)[row * q.k + k];
 }
 
+__device__ __forceinline__ float deq_elem_bf16(const QView &q, int64_t row, int64_t k) {
+    return __uint_as_float((uint32_t)((const uint16_t *)q.data)[row * q.recs + k] << 16);
+}
+
 template <int T>
 __device__ __forceinline__ float deq_elem(const QView &q, int64_t row, int64_t k) {
     if (T == FH_Q5_0) return deq_elem_q5_0(q, row, k);
     if (T == FH_Q5_K) return deq_elem_q5_k(q, row, k);
+    if (T == FH_BF16) return deq_elem_bf16(q, row, k);
     if (T == 0) return deq_elem_f32(q, row, k);
     if (T == 1) return deq_elem_f16(q, row, k);
     if (T == FH_Q4_0) return deq_elem_q4_0(q, row, k);

@@ -285,4 +285,4 @@ extern "C" fh_status fh_graph_free(fh_graph *g) {
     return FH_OK;
 }
 
-size_t fh_dtype_size(int dtype) { return dtype == FH_F16 ? 2 : 4; }
+size_t fh_dtype_size(int dtype) { return dtype == FH_F32 ? 4 : 2; }

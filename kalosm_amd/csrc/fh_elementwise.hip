@@ -151,6 +151,42 @@ extern "C" fh_status fh_rope_tables_scaled(fh_device *dev, int32_t head_dim, int
     return FH_OK;
 }
 
+// YaRN: pairs that turn at least `fast` times inside the original context keep their frequency, pairs that turn at most
+// `slow` times are stretched by `factor`, a linear ramp over the pair index joins them; cos and sin carry the factor
+// 0.1 ln(factor) + 1.  Angles are f32 products of the position and the f32 frequency.
+extern "C" fh_status fh_rope_tables_yarn(fh_device *dev, int32_t dims, int32_t ctx, double base, const fh_yarn_scaling *scaling,
+                                         float *cos_dev, float *sin_dev) {
+    FH_REQUIRE(dev && cos_dev && sin_dev, "NULL argument");
+    FH_REQUIRE(dims > 0 && dims % 2 == 0 && ctx > 0 && base > 1.0, "bad dims %d / ctx %d / base %g", dims, ctx, base);
+    const int half = dims / 2;
+    std::vector<float> f(half), c((size_t)ctx * half), s((size_t)ctx * half);
+    double amp = 1.0, lo = 0.0, hi = 0.0;
+    if (scaling) {
+        FH_REQUIRE(scaling->factor > 0.f && scaling->original > 0.f && scaling->fast > 0.f && scaling->slow > 0.f, "bad YaRN scaling");
+        const double pi = 3.14159265358979323846;
+        auto at = [&](double turns) { return dims * log(scaling->original / (2.0 * pi * turns)) / (2.0 * log(base)); };
+        lo = fmax(floor(at(scaling->fast)), 0.0);
+        hi = fmin(ceil(at(scaling->slow)), dims - 1.0);
+        amp = 0.1 * log((double)scaling->factor) + 1.0;
+    }
+    for (int i = 0; i < half; i++) {
+        double w = pow(base, -2.0 * i / dims);
+        if (scaling) {
+            const double ramp = fmin(fmax((i - lo) / fmax(hi - lo, 0.001), 0.0), 1.0);
+            w = w / scaling->factor * ramp + w * (1.0 - ramp);
+        }
+        f[i] = (float)w;
+    }
+    for (int p = 0; p < ctx; p++)
+        for (int i = 0; i < half; i++) {
+            const float a = (float)p * f[i];
+            c[(size_t)p * half + i] = (float)(cos((double)a) * amp);
+            s[(size_t)p * half + i] = (float)(sin((double)a) * amp);
+        }
+    FH_TRY(fh_upload(dev, cos_dev, c.data(), c.size() * 4));
+    return fh_upload(dev, sin_dev, s.data(), s.size() * 4);
+}
+
 extern "C" fh_status fh_rope_tables_weighted(fh_device *dev, int32_t head_dim, int32_t ctx, float theta,
                                              const float *freq_weight_host, float *cos_dev, float *sin_dev) {
     return fh_rope_tables_scaled(dev, head_dim, ctx, theta, nullptr, freq_weight_host, cos_dev, sin_dev);
@@ -727,6 +763,15 @@ extern "C" fh_status fh_kvcache_create(fh_device *dev, int32_t layers, int32_t k
     return FH_OK;
 }
 
+fh_status fh_kvcache_create_ring(fh_device *dev, int row, int max_len, int dtype, fh_kvcache **out) {
+    FH_REQUIRE(row % 4 == 0 && (dtype == FH_F32 || dtype == 2), "bad ring cache of %d elements per row", row);
+    FH_TRY(fh_kvcache_create(dev, 1, 1, row, max_len, FH_F32, out));
+    (*out)->dtype = dtype;
+    (*out)->ring = true;
+    (*out)->has_v = false;
+    return FH_OK;
+}
+
 extern "C" fh_status fh_kvcache_destroy(fh_kvcache *c) {
     if (!c) return FH_OK;
     (void)hipStreamSynchronize(c->dev->stream);
@@ -758,6 +803,7 @@ __global__ void k_kv_regrow(const uint32_t *__restrict__ src, uint32_t *__restri
 }
 
 fh_status fh_kvcache_reserve(fh_kvcache *c, int required) {
+    if (c->ring && required > c->max_len) required = c->max_len;
     FH_REQUIRE(required <= c->max_len, "KV cache overflow: %d positions needed, max_len %d", required, c->max_len);
     if (required <= c->capacity) return FH_OK;
     int cap = kv_alloc_len(required, c->max_len);
@@ -765,7 +811,7 @@ fh_status fh_kvcache_reserve(fh_kvcache *c, int required) {
     size_t bytes = (size_t)c->layers * c->kv_heads * cap * c->head_dim * es;
     void *nk = nullptr, *nv = nullptr;
     FH_HIP(hipMalloc(&nk, bytes));
-    hipError_t e = hipMalloc(&nv, bytes);
+    hipError_t e = c->has_v ? hipMalloc(&nv, bytes) : hipSuccess;
     if (e != hipSuccess) {
         (void)hipFree(nk);
         FH_FAIL(FH_ERR_OOM, "hipMalloc(%zu) failed: %s", bytes, hipGetErrorString(e));
@@ -774,13 +820,15 @@ fh_status fh_kvcache_reserve(fh_kvcache *c, int required) {
     // New cache memory starts as NaN bit patterns (f32 and f16 alike): a kernel that lets a row past the live length
     // reach its result then fails in every run, not only when the allocation happens to hold such bytes.
     FH_HIP(hipMemsetAsync(nk, 0xFF, bytes, s));
-    FH_HIP(hipMemsetAsync(nv, 0xFF, bytes, s));
+    if (nv) FH_HIP(hipMemsetAsync(nv, 0xFF, bytes, s));
     if (c->len > 0 && c->k) {
         int wpp = (int)(c->head_dim * es / 4);
-        int64_t rows = (int64_t)c->layers * c->kv_heads, total = rows * c->len * wpp;
+        const int live = c->len < c->capacity ? c->len : c->capacity; // a ring that still grows has not wrapped
+        int64_t rows = (int64_t)c->layers * c->kv_heads, total = rows * live * wpp;
         dim3 grid((unsigned)((total + 255) / 256));
-        k_kv_regrow<<<grid, 256, 0, s>>>((const uint32_t *)c->k, (uint32_t *)nk, rows, c->len, c->capacity, cap, wpp);
-        k_kv_regrow<<<grid, 256, 0, s>>>((const uint32_t *)c->v, (uint32_t *)nv, rows, c->len, c->capacity, cap, wpp);
+        k_kv_regrow<<<grid, 256, 0, s>>>((const uint32_t *)c->k, (uint32_t *)nk, rows, live, c->capacity, cap, wpp);
+        if (nv)
+            k_kv_regrow<<<grid, 256, 0, s>>>((const uint32_t *)c->v, (uint32_t *)nv, rows, live, c->capacity, cap, wpp);
     }
     FH_HIP(hipStreamSynchronize(s));
     if (c->k) (void)hipFree(c->k);

@@ -140,14 +140,15 @@ struct fh_qmatrix {
 };
 
 // Weight types kept in the file's own row-major order (no tiled re-layout): dense f32 / f16 rows.
-enum { FH_W_F32 = 0, FH_W_F16 = 1 };
-static inline bool fh_is_plain(uint32_t t) { return t == FH_W_F32 || t == FH_W_F16; }
+// FH_BF16 rows have a stride of k rounded up to 64 (kept in `recs`) and are rounded up to 16 rows, zeros in the padding.
+enum { FH_W_F32 = 0, FH_W_F16 = 1, FH_GGML_I32 = 26 };
+static inline bool fh_is_plain(uint32_t t) { return t == FH_W_F32 || t == FH_W_F16 || t == FH_BF16; }
 // Types without kernels for several activation rows (batch, row and tile kernels): those go row by row or element by
 // element.  The 5-bit formats have the single-row matrix-core kernel only.
 static inline bool fh_single_row_only(uint32_t t) { return fh_is_plain(t) || t == FH_Q5_0 || t == FH_Q5_K; }
 static inline int fh_block_elems(uint32_t t) {
     switch (t) {
-    case FH_W_F32: case FH_W_F16: return 1;
+    case FH_W_F32: case FH_W_F16: case FH_BF16: return 1;
     case FH_Q4_0: case FH_Q8_0: case FH_Q5_0: return 32;
     case FH_Q4_K: case FH_Q6_K: case FH_Q5_K: return 256;
     default: return 0;
@@ -156,7 +157,7 @@ static inline int fh_block_elems(uint32_t t) {
 static inline int fh_block_bytes(uint32_t t) { // gguf/src/lib.rs:109-121
     switch (t) {
     case FH_W_F32: return 4;
-    case FH_W_F16: return 2;
+    case FH_W_F16: case FH_BF16: return 2;
     case FH_Q4_0: return 18;
     case FH_Q5_0: return 22;
     case FH_Q8_0: return 34;
@@ -174,6 +175,10 @@ static inline int fh_rec_blocks(uint32_t t) {   // blocks per record (per row)
     }
 }
 static inline int fh_rec_bytes(uint32_t t) { return 16 * fh_rec_blocks(t) * fh_block_bytes(t); }
+
+// An FH_BF16 matrix of zeros, and n rows of k values into it (interleave: row r goes to row0 + 32 (r / 16) + r % 16).
+fh_status fh_qmatrix_alloc_bf16(fh_device *dev, int64_t n, int64_t k, fh_qmatrix **out);
+fh_status fh_qmatrix_put_bf16(fh_qmatrix *q, int64_t row0, int64_t n, int64_t k, const void *bytes, bool interleave);
 
 // A plain-data view passed to kernels by value.
 struct QView {
@@ -226,11 +231,17 @@ struct fh_kvcache {
     int layers = 0, kv_heads = 0, head_dim = 0, max_len = 0, dtype = FH_F32;
     int len = 0, capacity = 0;
     bool sliding = false;            // past max_len: keep the last max_len positions instead of failing
+    bool ring = false;               // position p lives in row p % capacity: never more than max_len rows, no shifting
+    bool has_v = true;               // without: one plane (k) of rows that are not keys and values (latent attention)
     void *k = nullptr, *v = nullptr; // [layers][kv_heads][capacity][head_dim]
     int *len_dev = nullptr;          // device copy of len (for graph-replayed decode steps)
 };
 size_t fh_dtype_size(int dtype);
 fh_status fh_kvcache_reserve(fh_kvcache *c, int required);
+// One layer of `row` elements per position (FH_F32, or 2 for bf16), a ring of at most max_len rows, no V plane.
+fh_status fh_kvcache_create_ring(fh_device *dev, int row, int max_len, int dtype, fh_kvcache **out);
+// dense bf16 rows (fh_dense.hip): x f32 [m, k]
+fh_status fh_launch_bf16_matmul(const fh_qmatrix *q, const void *x, int x_is_bf16, int m, float *y);
 // append reading the write position from c->len_dev (graph friendly), s == 1
 fh_status fh_kvcache_append_devpos(fh_kvcache *c, int layer, const float *k, const float *v, int64_t sh);
 fh_status fh_launch_q4k_m1_ropekv(const fh_qmatrix *q, const float *x, const float *nw, float eps, fh_kvcache *c,

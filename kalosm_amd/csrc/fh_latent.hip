@@ -1,0 +1,514 @@
+// Latent attention (fh_latent.h): cache rows, prefill on the matrix cores, decode step over the cached rows.
+#include "fh_latent.h"
+
+static constexpr float FH_LOG2E = 1.4426950408889634f;
+
+// ------------------------------------------------------------------------------ cache rows of a portion
+// Rows 0 .. old - 1 come out of the ring, the others are computed from the projections.  One workgroup per row.
+template <typename T>
+__global__ __launch_bounds__(128) void k_latent_rows(FhLatent a, const float *__restrict__ proj, int64_t ldp, int old, int pos,
+                                                     const T *__restrict__ ring, int cap, T *__restrict__ lat, T *__restrict__ kr) {
+    __shared__ float red[2];
+    const int i = blockIdx.x, tid = threadIdx.x, row = a.r8 + a.drp;
+    T *lr = lat + (int64_t)i * a.rp, *kd = kr + (int64_t)i * a.drp;
+    if (i < old) {
+        const T *src = ring + (int64_t)((pos - old + i) % cap) * row;
+        for (int c = tid; c < a.rp; c += 128) lr[c] = c < a.r8 ? src[c] : fh_to<T>(0.f);
+        for (int c = tid; c < a.drp; c += 128) kd[c] = src[a.r8 + c];
+        return;
+    }
+    const int t = i - old;
+    const float *p = proj + (int64_t)t * ldp + a.col_kv;
+    float ss = 0.f;
+    for (int c = tid; c < a.rank; c += 128) ss = fmaf(p[c], p[c], ss);
+    ss = fh_wave_sum(ss);
+    if ((tid & 63) == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    const float inv = 1.0f / sqrtf((red[0] + red[1]) / (float)a.rank + a.eps);
+    for (int c = tid; c < a.rp; c += 128) lr[c] = fh_to<T>(c < a.rank ? p[c] * inv * a.c_norm[c] : 0.f);
+    const float *ct = a.cos_t + (int64_t)(pos + t) * a.pairs, *st = a.sin_t + (int64_t)(pos + t) * a.pairs;
+    for (int c = tid; c < a.drp; c += 128) {
+        float v = c < a.dr ? p[a.rank + c] : 0.f;
+        const int pr = c >> 1;
+        if (c < a.dr && pr < a.pairs) {
+            const float o = p[a.rank + (c ^ 1)];
+            v = (c & 1) ? v * ct[pr] + o * st[pr] : v * ct[pr] - o * st[pr];
+        }
+        kd[c] = fh_to<T>(v);
+    }
+}
+
+// The last `n` rows of the portion into the ring.
+template <typename T>
+__global__ __launch_bounds__(128) void k_latent_append(FhLatent a, const T *__restrict__ lat, const T *__restrict__ kr, int first,
+                                                       int pos_first, T *__restrict__ ring, int cap) {
+    const int i = blockIdx.x, row = a.r8 + a.drp;
+    T *dst = ring + (int64_t)((pos_first + i) % cap) * row;
+    for (int c = threadIdx.x; c < row; c += 128)
+        dst[c] = c < a.r8 ? lat[(int64_t)(first + i) * a.rp + c] : kr[(int64_t)(first + i) * a.drp + c - a.r8];
+}
+
+// Queries [s, heads, dq]: unrotated part, rotated part, zeros.
+template <typename T>
+__global__ __launch_bounds__(256) void k_latent_q(FhLatent a, const float *__restrict__ proj, int64_t ldp, int pos, int dq,
+                                                  T *__restrict__ q) {
+    const int t = blockIdx.x, d0 = a.dn + a.dr;
+    const float *p = proj + (int64_t)t * ldp + a.col_q;
+    const float *ct = a.cos_t + (int64_t)(pos + t) * a.pairs, *st = a.sin_t + (int64_t)(pos + t) * a.pairs;
+    for (int i = threadIdx.x; i < a.heads * dq; i += 256) {
+        const int h = i / dq, c = i % dq;
+        float v = 0.f;
+        if (c < a.dn) v = p[h * d0 + c];
+        else if (c >= a.dnp && c - a.dnp < a.dr) {
+            const int r = c - a.dnp, pr = r >> 1;
+            const float *pp = p + h * d0 + a.dn;
+            v = pp[r];
+            if (pr < a.pairs) {
+                const float o = pp[r ^ 1];
+                v = (r & 1) ? v * ct[pr] + o * st[pr] : v * ct[pr] - o * st[pr];
+            }
+        }
+        q[((int64_t)t * a.heads + h) * dq + c] = fh_to<T>(v);
+    }
+}
+
+// ------------------------------------------------------------------------------ prefill attention
+// grid (heads, query blocks, value blocks of 16 DVT): four wavefronts of 16 QF queries.  Both products are computed
+// transposed, as in the other prefill attention: S^T = K . Q^T, O^T = V^T . P^T, so a lane (column) is one query and the
+// softmax statistics are per-lane scalars.  MFMA row i of half hf of a 32-key group reads key 8 (i / 4) + 4 hf + i % 4:
+// with that order the accumulators of a lane are keys 8 g .. 8 g + 7 (g = lane / 16), the k-slots of its P^T operand.
+// Key tiles of 64 go through the LDS (K as [key][dq], V transposed as [value][key]); the next tile is requested into
+// registers while the current one is multiplied.
+template <typename T> struct FhPiece { T v[8]; };
+template <typename T>
+__device__ __forceinline__ FhPiece<T> fh_zero_piece() {
+    FhPiece<T> p;
+#pragma unroll
+    for (int e = 0; e < 8; e++) p.v[e] = 0;
+    return p;
+}
+template <typename T>
+__device__ __forceinline__ FhPiece<T> fh_ld_piece(const T *p) {
+    FhPiece<T> r;
+    struct alignas(16) A { T v[8]; };
+    const A a = *(const A *)p;
+    __builtin_memcpy(&r, &a, sizeof r);
+    return r;
+}
+template <typename T>
+__device__ __forceinline__ void fh_st_piece(T *p, const FhPiece<T> &r) {
+    struct alignas(16) A { T v[8]; };
+    A a;
+    __builtin_memcpy(&a, &r, sizeof r);
+    *(A *)p = a;
+}
+// P^T operands: bf16 as hi + lo
+__device__ __forceinline__ void fh_pv(fh_f4 &acc, const fh_bf8 &v, const float *p) {
+    fh_bf8 hi, lo;
+#pragma unroll
+    for (int e = 0; e < 8; e++) {
+        hi[e] = (fh_bf)p[e];
+        lo[e] = (fh_bf)(p[e] - (float)hi[e]);
+    }
+    acc = fh_mma32(v, hi, acc);
+    acc = fh_mma32(v, lo, acc);
+}
+__device__ __forceinline__ void fh_pv(fh_f4 &acc, const fh_f8 &v, const float *p) {
+    fh_f8 b;
+#pragma unroll
+    for (int e = 0; e < 8; e++) b.v[e] = p[e];
+    acc = fh_mma32(v, b, acc);
+}
+
+template <typename T, int DQS, int DVT, int QF>
+__global__ __launch_bounds__(256) void k_latent_attn(FhLatent a, const T *__restrict__ q, const T *__restrict__ kn,
+                                                     const T *__restrict__ kr, const T *__restrict__ vt, int64_t ldt, int s,
+                                                     int old, T *__restrict__ o, int kp) {
+    typedef typename FhFrag<T>::type Frag;
+    constexpr int DQ = DQS * 32, KS = DQ + 8, VS = 64 + 8, QB = 64 * QF;
+    constexpr int NK = 64 * DQ / 8 / 256, NV = DVT * 16 * 8 / 256; // pieces per thread
+    static_assert(DVT % 2 == 0, "value pieces are shared out evenly");
+    extern __shared__ __attribute__((aligned(16))) char la_lds[];
+    T *sk = (T *)la_lds, *sv = sk + 64 * KS;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, li = lane & 15, g = lane >> 4;
+    const int h = blockIdx.x, qb = (int)(gridDim.y - 1 - blockIdx.y) * QB, dv0 = (int)blockIdx.z * DVT * 16;
+    const int keys = old + s, npk = a.dnp / 8, nrk = a.drp / 8;
+    Frag qf[DQS][QF];
+    int qi[QF];
+#pragma unroll
+    for (int f = 0; f < QF; f++) {
+        qi[f] = qb + wave * 16 * QF + f * 16 + li;
+        const T *qp = q + ((int64_t)(qi[f] < s ? qi[f] : s - 1) * a.heads + h) * DQ + 8 * g;
+#pragma unroll
+        for (int k = 0; k < DQS; k++) fh_frag_load(qf[k][f], qp + 32 * k);
+    }
+    fh_f4 acc[DVT][QF];
+    float mx[QF], den[QF];
+#pragma unroll
+    for (int f = 0; f < QF; f++) {
+        mx[f] = -INFINITY, den[f] = 0.f;
+#pragma unroll
+        for (int d = 0; d < DVT; d++) acc[d][f] = fh_f4{0.f, 0.f, 0.f, 0.f};
+    }
+    const float sc = a.scale * FH_LOG2E;
+    const int last = qb + QB - 1 < s ? qb + QB - 1 : s - 1;          // last query of the block
+    int j0 = a.window && qb + old - a.window + 1 > 0 ? qb + old - a.window + 1 : 0;
+    j0 = j0 / 64 * 64;
+    const int j1 = last + old + 1;                                   // one past the last visible key
+    FhPiece<T> pk[NK], pv[NV];
+    auto fetch = [&](int j) {
+#pragma unroll
+        for (int i = 0; i < NK; i++) {
+            const int x = tid + 256 * i, r = x / (DQ / 8), c = x % (DQ / 8);
+            const int key = j + r;
+            if (key < keys && c < npk) pk[i] = fh_ld_piece(kn + (int64_t)key * a.heads * a.dnp + h * a.dnp + c * 8);
+            else if (key < keys && c - npk < nrk && c >= npk) pk[i] = fh_ld_piece(kr + (int64_t)key * a.drp + (c - npk) * 8);
+            else pk[i] = fh_zero_piece<T>();
+        }
+#pragma unroll
+        for (int i = 0; i < NV; i++) {
+            const int x = tid + 256 * i, r = x >> 3, c = (x & 7) * 8;
+            if (dv0 + r < a.dv && j + c < keys) {
+                pv[i] = fh_ld_piece(vt + (int64_t)(h * a.dv + dv0 + r) * ldt + j + c);
+                if (j + c + 8 > keys)
+#pragma unroll
+                    for (int e = 0; e < 8; e++)
+                        if (j + c + e >= keys) pv[i].v[e] = 0;
+            } else pv[i] = fh_zero_piece<T>();
+        }
+    };
+    fetch(j0);
+    for (int j = j0; j < j1; j += 64) {
+        __syncthreads(); // the previous tile has been read
+#pragma unroll
+        for (int i = 0; i < NK; i++) {
+            const int x = tid + 256 * i, r = x / (DQ / 8), c = x % (DQ / 8);
+            fh_st_piece(sk + r * KS + c * 8, pk[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < NV; i++) {
+            const int x = tid + 256 * i, r = x >> 3, c = (x & 7) * 8;
+            fh_st_piece(sv + r * VS + c, pv[i]);
+        }
+        __syncthreads();
+        if (j + 64 < j1) fetch(j + 64);
+        fh_f4 S[4][QF];
+#pragma unroll
+        for (int t = 0; t < 4; t++) {
+#pragma unroll
+            for (int f = 0; f < QF; f++) S[t][f] = fh_f4{0.f, 0.f, 0.f, 0.f};
+            const T *kp_ = sk + (32 * (t >> 1) + 8 * (li >> 2) + 4 * (t & 1) + (li & 3)) * KS + 8 * g;
+#pragma unroll
+            for (int k = 0; k < DQS; k++) {
+                Frag kf;
+                fh_frag_load(kf, kp_ + 32 * k);
+#pragma unroll
+                for (int f = 0; f < QF; f++) S[t][f] = fh_mma32(kf, qf[k][f], S[t][f]);
+            }
+        }
+        float p[QF][2][8];
+#pragma unroll
+        for (int f = 0; f < QF; f++) {
+            float tm = -INFINITY;
+#pragma unroll
+            for (int t = 0; t < 4; t++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) {
+                    const int d = qi[f] + old - (j + 32 * (t >> 1) + 8 * g + 4 * (t & 1) + r); // query minus key position
+                    const bool vis = d >= 0 && (!a.window || d < a.window);
+                    const float v = vis ? S[t][f][r] * sc : -INFINITY;
+                    p[f][t >> 1][4 * (t & 1) + r] = v;
+                    tm = fmaxf(tm, v);
+                }
+            tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+            tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+            const float mn = fmaxf(mx[f], tm), mb = mn == -INFINITY ? 0.f : mn;
+            const float resc = exp2f(mx[f] - mb);
+            float sum = 0.f;
+#pragma unroll
+            for (int u = 0; u < 2; u++)
+#pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    const float w = exp2f(p[f][u][e] - mb);
+                    p[f][u][e] = w;
+                    sum += w;
+                }
+            den[f] = den[f] * resc + sum;
+            mx[f] = mn;
+#pragma unroll
+            for (int d = 0; d < DVT; d++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) acc[d][f][r] *= resc;
+        }
+#pragma unroll
+        for (int u = 0; u < 2; u++)
+#pragma unroll
+            for (int d = 0; d < DVT; d++) {
+                Frag vf;
+                fh_frag_load(vf, sv + (16 * d + li) * VS + 32 * u + 8 * g);
+#pragma unroll
+                for (int f = 0; f < QF; f++) fh_pv(acc[d][f], vf, p[f][u]);
+            }
+    }
+#pragma unroll
+    for (int f = 0; f < QF; f++) {
+        float l = den[f];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        if (qi[f] >= s) continue;
+        float m = mx[f], up = 1.f;
+        if (a.sink) { // the sink joins the denominator only
+            const float z = a.sink[h] * FH_LOG2E, mm = fmaxf(m, z);
+            up = exp2f(m - mm);
+            l = l * up + exp2f(z - mm);
+        }
+        const float inv = up / l;
+        T *orow = o + (int64_t)qi[f] * kp;
+#pragma unroll
+        for (int d = 0; d < DVT; d++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int c = dv0 + 16 * d + 4 * g + r;
+                if (c < a.dv) orow[h * a.dv + c] = fh_to<T>(acc[d][f][r] * inv);
+            }
+        if (h == a.heads - 1 && dv0 == 0)
+            for (int c = a.heads * a.dv + g; c < kp; c += 4) orow[c] = fh_to<T>(0.f);
+    }
+}
+
+int fh_latent_dq(const FhLatent &a) {
+    const int d = (a.dnp + a.drp + 31) / 32;
+    return d <= 2 ? 64 : d <= 4 ? 128 : d <= 6 ? 192 : d <= 8 ? 256 : 0;
+}
+
+template <typename T, int DQS, int DVT>
+static fh_status latent_attn_go(fh_device *dev, const FhLatent &a, const FhLatentWork &w, int s, int old, void *o, int kp) {
+    constexpr int QF = sizeof(T) == 2 ? 2 : 1;
+    const size_t lds = (size_t)(64 * (DQS * 32 + 8) + DVT * 16 * 72) * sizeof(T);
+    auto fn = k_latent_attn<T, DQS, DVT, QF>;
+    if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)fn, lds));
+    const dim3 grid((unsigned)a.heads, (unsigned)((s + 64 * QF - 1) / (64 * QF)), (unsigned)((a.dv + DVT * 16 - 1) / (DVT * 16)));
+    fn<<<grid, 256, lds, dev->stream>>>(a, (const T *)w.q, (const T *)w.kn, (const T *)w.kr, (const T *)w.vt, w.ldt, s, old,
+                                        (T *)o, kp);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+template <typename T>
+static fh_status latent_prefill_t(fh_device *dev, int dtype, const FhLatent &a, fh_kvcache *cache, const float *proj, int64_t ldp,
+                                  int s, int pos, const FhLatentWork &w, void *o, int kp) {
+    hipStream_t str = dev->stream;
+    const int old = fh_latent_old(a, pos), keys = old + s, dq = fh_latent_dq(a);
+    FH_REQUIRE(dq, "attention over %d + %d query dimensions (at most 256)", a.dn, a.dr);
+    k_latent_rows<T><<<dim3((unsigned)keys), 128, 0, str>>>(a, proj, ldp, old, pos, (const T *)cache->k, cache->capacity, (T *)w.lat,
+                                                           (T *)w.kr);
+    const int n = s < cache->capacity ? s : cache->capacity;
+    k_latent_append<T><<<dim3((unsigned)n), 128, 0, str>>>(a, (const T *)w.lat, (const T *)w.kr, keys - n, pos + s - n, (T *)cache->k,
+                                                          cache->capacity);
+    k_latent_q<T><<<dim3((unsigned)s), 256, 0, str>>>(a, proj, ldp, pos, dq, (T *)w.q);
+    FH_HIP(hipGetLastError());
+    FhGemm g;
+    g.kp = a.rp, g.m = keys, g.x = w.lat;
+    g.w = a.uk, g.n = a.heads * a.dnp, g.y = w.kn, g.ldy = (int64_t)a.heads * a.dnp;
+    FH_TRY(fh_gemm(dev, dtype, FH_GEMM_ACT, g));
+    g.w = a.uv, g.n = a.heads * a.dv, g.y = w.vt, g.ldy = w.ldt;
+    FH_TRY(fh_gemm(dev, dtype, FH_GEMM_ACT_T, g));
+#define FH_GO(DQS_)                                                                           \
+    return a.dv <= 64 ? latent_attn_go<T, DQS_, 4>(dev, a, w, s, old, o, kp) : latent_attn_go<T, DQS_, 8>(dev, a, w, s, old, o, kp)
+    switch (dq) {
+    case 64: FH_GO(2);
+    case 128: FH_GO(4);
+    case 192: FH_GO(6);
+    default: FH_GO(8);
+    }
+#undef FH_GO
+}
+
+fh_status fh_latent_prefill(fh_device *dev, int dtype, const FhLatent &a, fh_kvcache *cache, const float *proj, int64_t ldp,
+                            int s, int pos, const FhLatentWork &w, void *o, int kp) {
+    return dtype == FH_F32 ? latent_prefill_t<float>(dev, dtype, a, cache, proj, ldp, s, pos, w, o, kp)
+                           : latent_prefill_t<uint16_t>(dev, dtype, a, cache, proj, ldp, s, pos, w, o, kp);
+}
+
+// ------------------------------------------------------------------------------ decode step
+// grid (splits, head groups of HB).  The live rows of the ring are 0 .. min(position + 1, capacity) - 1 in any order (the
+// softmax does not care, the rotation is already in the row).  The 16 lanes of a DPP row take one cached row, pieces of 8
+// elements dealt round-robin; each row group keeps running statistics and a weighted sum of its own.
+template <typename T, int NP, int HB> // NP pieces per lane: rows of at most 128 NP elements
+__global__ __launch_bounds__(256) void k_latent_decode(FhLatent a, const T *__restrict__ ring, int cap, const int *__restrict__ pos_dev,
+                                                       const float *__restrict__ qa, float *__restrict__ part) {
+    extern __shared__ float od[]; // [4 waves][HB][r8 + 2]
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l16 = lane & 15, rg = tid >> 4;
+    const int row = a.r8 + a.drp, np = row / 8, h0 = (int)blockIdx.y * HB;
+    const int n = *pos_dev + 1 < cap ? *pos_dev + 1 : cap;
+    const int per = ((n + (int)gridDim.x - 1) / (int)gridDim.x + 15) / 16 * 16;
+    const int k0 = (int)blockIdx.x * per, k1 = k0 + per < n ? k0 + per : n;
+    float q[HB][NP][8], o[HB][NP][8], m[HB], l[HB];
+#pragma unroll
+    for (int b = 0; b < HB; b++) {
+        m[b] = -INFINITY, l[b] = 0.f;
+        const float *qp = qa + (int64_t)(h0 + b < a.heads ? h0 + b : a.heads - 1) * row;
+#pragma unroll
+        for (int i = 0; i < NP; i++)
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                q[b][i][e] = l16 + 16 * i < np ? qp[(l16 + 16 * i) * 8 + e] : 0.f;
+                o[b][i][e] = 0.f;
+            }
+    }
+    FhPiece<T> nx[NP];
+    auto fetch = [&](int k) {
+#pragma unroll
+        for (int i = 0; i < NP; i++)
+            nx[i] = l16 + 16 * i < np ? fh_ld_piece(ring + (int64_t)k * row + (l16 + 16 * i) * 8) : fh_zero_piece<T>();
+    };
+    if (k0 + rg < k1) fetch(k0 + rg);
+    for (int k = k0 + rg; k < k1; k += 16) {
+        float c[NP][8];
+#pragma unroll
+        for (int i = 0; i < NP; i++)
+#pragma unroll
+            for (int e = 0; e < 8; e++) c[i][e] = fh_up(nx[i].v[e]);
+        if (k + 16 < k1) fetch(k + 16);
+#pragma unroll
+        for (int b = 0; b < HB; b++) {
+            float d = 0.f;
+#pragma unroll
+            for (int i = 0; i < NP; i++)
+#pragma unroll
+                for (int e = 0; e < 8; e++) d = fmaf(q[b][i][e], c[i][e], d);
+            d = fh_row16_sum(d);
+            const float mn = fmaxf(m[b], d), r = exp2f(m[b] - mn), w = exp2f(d - mn);
+            l[b] = l[b] * r + w;
+            m[b] = mn;
+#pragma unroll
+            for (int i = 0; i < NP; i++)
+#pragma unroll
+                for (int e = 0; e < 8; e++) o[b][i][e] = fmaf(w, c[i][e], o[b][i][e] * r);
+        }
+    }
+    const int st = a.r8 + 2;
+#pragma unroll
+    for (int b = 0; b < HB; b++) {
+        // the four row groups of the wavefront, then the four wavefronts through the LDS
+        float mm = fmaxf(m[b], __shfl_xor(m[b], 16, 64));
+        mm = fmaxf(mm, __shfl_xor(mm, 32, 64));
+        const float f = m[b] == -INFINITY ? 0.f : exp2f(m[b] - mm);
+        float ll = l[b] * f;
+        ll += __shfl_xor(ll, 16, 64);
+        ll += __shfl_xor(ll, 32, 64);
+        float *dst = od + (wave * HB + b) * st;
+#pragma unroll
+        for (int i = 0; i < NP; i++)
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                float v = o[b][i][e] * f;
+                v += __shfl_xor(v, 16, 64);
+                v += __shfl_xor(v, 32, 64);
+                const int x = (l16 + 16 * i) * 8 + e;
+                if (lane < 16 && x < a.r8) dst[x] = v;
+            }
+        if (lane == 0) dst[a.r8] = mm, dst[a.r8 + 1] = ll;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int b = 0; b < HB; b++) {
+        if (h0 + b >= a.heads) break;
+        float mm = -INFINITY, f[4], ll = 0.f;
+#pragma unroll
+        for (int w = 0; w < 4; w++) mm = fmaxf(mm, od[(w * HB + b) * st + a.r8]);
+#pragma unroll
+        for (int w = 0; w < 4; w++) {
+            const float mw = od[(w * HB + b) * st + a.r8];
+            f[w] = mw == -INFINITY ? 0.f : exp2f(mw - mm);
+            ll += f[w] * od[(w * HB + b) * st + a.r8 + 1];
+        }
+        float *dst = part + ((int64_t)(h0 + b) * gridDim.x + blockIdx.x) * st;
+        for (int x = tid; x < a.r8; x += 256) {
+            float v = 0.f;
+#pragma unroll
+            for (int w = 0; w < 4; w++) v = fmaf(f[w], od[(w * HB + b) * st + x], v);
+            dst[x] = v;
+        }
+        if (tid == 0) dst[a.r8] = mm, dst[a.r8 + 1] = ll;
+    }
+}
+
+// Merge of the splits (with the sink) and the value projection: grid (heads, blocks of 32 values).
+__global__ __launch_bounds__(256) void k_latent_values(FhLatent a, const float *__restrict__ part, int splits, float *__restrict__ o) {
+    extern __shared__ __attribute__((aligned(16))) float oc[]; // [rp]
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.x, st = a.r8 + 2;
+    const float *p = part + (int64_t)h * splits * st;
+    const float z = a.sink ? a.sink[h] * FH_LOG2E : -INFINITY;
+    float mm = z, l = 0.f;
+    for (int i = 0; i < splits; i++) mm = fmaxf(mm, p[i * st + a.r8]);
+    for (int i = 0; i < splits; i++) {
+        const float m = p[i * st + a.r8];
+        l += m == -INFINITY ? 0.f : exp2f(m - mm) * p[i * st + a.r8 + 1];
+    }
+    if (a.sink) l += exp2f(z - mm);
+    const float inv = 1.0f / l;
+    for (int x = tid; x < a.rp; x += 256) {
+        float v = 0.f;
+        if (x < a.r8)
+            for (int i = 0; i < splits; i++) {
+                const float m = p[i * st + a.r8];
+                if (m != -INFINITY) v = fmaf(exp2f(m - mm), p[i * st + x], v);
+            }
+        oc[x] = v * inv;
+    }
+    __syncthreads();
+    for (int i = 0; i < 8; i++) {
+        const int r = (int)blockIdx.y * 32 + wave * 8 + i;
+        if (r >= a.dv) break;
+        const uint16_t *w = a.uv + (int64_t)(h * a.dv + r) * a.rp;
+        float acc = 0.f;
+        for (int c = lane * 8; c < a.rp; c += 512) {
+            const uint4 u = *(const uint4 *)(w + c);
+            const float4 x = *(const float4 *)(oc + c), y = *(const float4 *)(oc + c + 4);
+            acc = fmaf(fh_bf_lo(u.x), x.x, acc);
+            acc = fmaf(fh_bf_hi(u.x), x.y, acc);
+            acc = fmaf(fh_bf_lo(u.y), x.z, acc);
+            acc = fmaf(fh_bf_hi(u.y), x.w, acc);
+            acc = fmaf(fh_bf_lo(u.z), y.x, acc);
+            acc = fmaf(fh_bf_hi(u.z), y.y, acc);
+            acc = fmaf(fh_bf_lo(u.w), y.z, acc);
+            acc = fmaf(fh_bf_hi(u.w), y.w, acc);
+        }
+        acc = fh_wave_sum(acc);
+        if (lane == 0) o[h * a.dv + r] = acc;
+    }
+}
+
+template <typename T>
+static fh_status latent_decode_t(fh_device *dev, const FhLatent &a, const fh_kvcache *cache, const int *pos_dev, const float *qa,
+                                 float *part, float *o) {
+    const int row = fh_latent_row(a), hb = a.heads % 2 == 0 ? 2 : 1;
+    int splits = cache->capacity / 64;
+    splits = splits < 1 ? 1 : splits > FH_LATENT_MAX_SPLITS ? FH_LATENT_MAX_SPLITS : splits;
+    const dim3 grid((unsigned)splits, (unsigned)(a.heads / hb));
+    const size_t lds = (size_t)4 * hb * (a.r8 + 2) * 4;
+    const T *ring = (const T *)cache->k;
+#define FH_GO(NP_)                                                                                                         \
+    do {                                                                                                                   \
+        if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, hb == 2 ? (const void *)k_latent_decode<T, NP_, 2> : (const void *)k_latent_decode<T, NP_, 1>, lds)); \
+        if (hb == 2) k_latent_decode<T, NP_, 2><<<grid, 256, lds, dev->stream>>>(a, ring, cache->capacity, pos_dev, qa, part); \
+        else k_latent_decode<T, NP_, 1><<<grid, 256, lds, dev->stream>>>(a, ring, cache->capacity, pos_dev, qa, part);     \
+    } while (0)
+    if (row <= 128) FH_GO(1);
+    else if (row <= 256) FH_GO(2);
+    else if (row <= 384) FH_GO(3);
+    else if (row <= 640) FH_GO(5);
+    else if (row <= 1152) FH_GO(9);
+    else FH_FAIL(FH_ERR_UNSUPPORTED, "latent rows of %d elements (at most 1152)", row);
+#undef FH_GO
+    k_latent_values<<<dim3((unsigned)a.heads, (unsigned)((a.dv + 31) / 32)), 256, (size_t)a.rp * 4, dev->stream>>>(a, part, splits, o);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+fh_status fh_latent_decode(fh_device *dev, int dtype, const FhLatent &a, const fh_kvcache *cache, const int *pos_dev,
+                           const float *qa, float *part, float *o) {
+    return dtype == FH_F32 ? latent_decode_t<float>(dev, a, cache, pos_dev, qa, part, o)
+                           : latent_decode_t<uint16_t>(dev, a, cache, pos_dev, qa, part, o);
+}

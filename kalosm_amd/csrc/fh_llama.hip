@@ -3,7 +3,7 @@
 // raw/attention_layer.rs:130-237 (feed-forward), :281-426 / :514-694 (attention),
 // raw/rope.rs:87-112 (interleaved RoPE for the llama architecture), model/inference.rs:11-396
 // (decode loop, here greedy).
-#include "fh_internal.h"
+#include "fh_decoder.h"
 
 #include <algorithm>
 #include <cstdarg>
@@ -19,10 +19,9 @@ struct fh_llama_layer {
     float *attn_norm = nullptr, *ffn_norm = nullptr;
 };
 
-struct fh_llama {
-    fh_device *dev = nullptr;
+struct fh_llama : fh_decoder {
     fh_llama_config c{};
-    std::vector<fh_llama_layer> layers;
+    std::vector<fh_llama_layer> layer;
     fh_qmatrix *embd = nullptr, *output = nullptr;
     bool output_is_embd = false;
     float *out_norm = nullptr;
@@ -31,37 +30,34 @@ struct fh_llama {
     bool has_rope_scaling = false;
     fh_rope_scaling rope_scaling = {};
     fh_kvcache *cache = nullptr;
-    bool finalized = false;
-    int pos = 0;
-    // the token ids whose keys and values the cache holds (KvCache::tokens of the reference, raw/cache.rs): what a
-    // forward pass re-runs the tail of when the context is full
-    std::vector<uint32_t> history;
     // step buffers (sized for `cap_s` tokens)
     int cap_s = 0;
-    uint32_t *ids = nullptr;
     float *x = nullptr, *xn = nullptr, *qkv = nullptr, *qrot = nullptr, *krot = nullptr, *att = nullptr, *att_t = nullptr,
-          *attn_out = nullptr, *gu = nullptr, *act = nullptr, *ff = nullptr, *logits = nullptr;
-    // greedy decode state
-    uint32_t *tok_dev = nullptr, *out_tok_dev = nullptr;
-    int *step_dev = nullptr;
-    hipGraphExec_t graph_exec = nullptr;
-    hipGraph_t graph = nullptr;
-    int captured_capacity = -1;
-    uint64_t captured_gen = 0, samp_gen = 0; // dev->scratch_gen at the captures
-    uint64_t captured_opt = 0, samp_opt = 0; // dev->opt_gen at the captures (options pick the kernels of a step)
-    // sampled decode state: [0..63] previous ids, [64] their count, [65] next slot, [66] Mirostat mu (f32),
-    // [68..69] status and token of the last step, [128..] one random number per step
-    uint32_t *samp_dev = nullptr;
-    hipGraphExec_t samp_exec = nullptr;
-    hipGraph_t samp_graph = nullptr;
-    int samp_capacity = -1;
-    uint32_t samp_range = 0;
-    fh_sampler_params samp_params = {};
-    // trace of the last fh_llama_forward (options trace_nan / trace_timing): the lines, and the stage marks
+          *attn_out = nullptr, *gu = nullptr, *act = nullptr, *ff = nullptr;
+    // trace of the last forward pass (options trace_nan / trace_timing): the lines, and the stage marks
     std::string trace_text;
     std::vector<hipEvent_t> trace_ev;      // pool, reused from call to call
     std::vector<std::string> trace_label;  // label of the stage that ends at mark i (marks used: trace_label.size())
     int trace_first = -1, trace_last = -1; // the marks before the first and after the last layer
+    bool tracing = false;                  // the last layers() call was traced
+
+    ~fh_llama() override;
+    fh_status ensure_steps(int s) override;
+    fh_status layers(int s, bool dev_pos) override;
+    fh_status head(int row, float *out) override;
+    const float *hidden() const override { return xn; }
+    fh_status reserve(int positions) override { return fh_kvcache_reserve(cache, positions); }
+    int64_t capacity() const override { return cache->capacity; }
+    fh_status set_len(int len, bool device) override {
+        cache->len = len;
+        return device ? fh_kvcache_set_len_dev(cache, len) : FH_OK;
+    }
+    int *len_dev() override { return cache->len_dev; }
+    uint64_t weight_bytes() const override;
+    fh_status load_tensor(const char *name, uint32_t ggml_type, int64_t n, int64_t k, const void *bytes, size_t len) override;
+    fh_status finalize() override;
+    fh_status forward_begin() override;
+    fh_status forward_end(int count) override;
 };
 
 // Tracing of the eager forward pass, off unless an option (or the reference's environment variable, read when the
@@ -147,7 +143,12 @@ extern "C" fh_status fh_llama_create(fh_device *dev, const fh_llama_config *cfg,
     fh_llama *m = new fh_llama();
     m->dev = dev;
     m->c = *cfg;
-    m->layers.resize(cfg->n_layers);
+    m->layer.resize(cfg->n_layers);
+    m->vocab = cfg->vocab;
+    m->d_model = cfg->d_model;
+    m->ctx = cfg->ctx;
+    m->n_layers = cfg->n_layers;
+    m->use_graph = cfg->use_graph != 0;
     *out = m;
     return FH_OK;
 }
@@ -170,31 +171,32 @@ static void free_steps(fh_llama *m) {
     m->ids = nullptr;
     m->x = m->xn = m->qkv = m->qrot = m->krot = m->att = m->att_t = m->attn_out = m->gu = m->act = m->ff = nullptr;
     m->cap_s = 0;
-    m->captured_capacity = -1; // a captured decode step holds these pointers
-    m->samp_capacity = -1;
+    m->drop_captures(); // a captured decode step holds these pointers
 }
 
-extern "C" fh_status fh_llama_destroy(fh_llama *m) {
-    if (!m) return FH_OK;
-    (void)hipStreamSynchronize(m->dev->stream);
-    if (m->graph_exec) (void)hipGraphExecDestroy(m->graph_exec);
-    if (m->graph) (void)hipGraphDestroy(m->graph);
-    for (auto &l : m->layers) {
+fh_llama::~fh_llama() {
+    (void)hipStreamSynchronize(dev->stream);
+    for (auto &l : layer) {
         fh_qmatrix_free(l.wq); fh_qmatrix_free(l.wk); fh_qmatrix_free(l.wv); fh_qmatrix_free(l.wo);
         fh_qmatrix_free(l.gate); fh_qmatrix_free(l.up); fh_qmatrix_free(l.down);
         fh_qmatrix_free(l.qkv); fh_qmatrix_free(l.gate_up);
         free_dev(l.attn_norm); free_dev(l.ffn_norm);
     }
-    fh_qmatrix_free(m->embd);
-    if (!m->output_is_embd) fh_qmatrix_free(m->output);
-    free_dev(m->out_norm); free_dev(m->cos_t); free_dev(m->sin_t);
-    free_dev(m->logits); free_dev(m->tok_dev); free_dev(m->out_tok_dev); free_dev(m->step_dev); free_dev(m->samp_dev);
-    if (m->samp_exec) (void)hipGraphExecDestroy(m->samp_exec);
-    if (m->samp_graph) (void)hipGraphDestroy(m->samp_graph);
-    free_steps(m);
-    fh_kvcache_destroy(m->cache);
-    for (hipEvent_t e : m->trace_ev) (void)hipEventDestroy(e);
+    fh_qmatrix_free(embd);
+    if (!output_is_embd) fh_qmatrix_free(output);
+    free_dev(out_norm); free_dev(cos_t); free_dev(sin_t);
+    free_steps(this);
+    fh_kvcache_destroy(cache);
+    for (hipEvent_t e : trace_ev) (void)hipEventDestroy(e);
+}
+extern "C" fh_status fh_llama_destroy(fh_llama *m) {
     delete m;
+    return FH_OK;
+}
+// The shared handle of a Llama decoder (fh_decoder_* calls); it stays owned by the fh_llama.
+extern "C" fh_status fh_llama_decoder(fh_llama *m, fh_decoder **out) {
+    FH_REQUIRE(m && out, "NULL argument");
+    *out = m;
     return FH_OK;
 }
 
@@ -212,6 +214,10 @@ static fh_status load_f32(fh_llama *m, float **dst, int64_t want, int64_t n, int
 extern "C" fh_status fh_llama_load_tensor(fh_llama *m, const char *name, uint32_t ggml_type, int64_t n, int64_t k,
                                           const void *bytes, size_t len) {
     FH_REQUIRE(m && name && bytes, "NULL argument");
+    return m->load_tensor(name, ggml_type, n, k, bytes, len);
+}
+fh_status fh_llama::load_tensor(const char *name, uint32_t ggml_type, int64_t n, int64_t k, const void *bytes, size_t len) {
+    fh_llama *m = this;
     FH_REQUIRE(!m->finalized, "decoder already finalized");
     const fh_llama_config &c = m->c;
     const int64_t D = c.d_model, QD = (int64_t)c.n_heads * c.head_dim, KD = (int64_t)c.n_kv_heads * c.head_dim;
@@ -237,7 +243,7 @@ extern "C" fh_status fh_llama_load_tensor(fh_llama *m, const char *name, uint32_
     int li = -1;
     char field[64] = "";
     if (sscanf(name, "blk.%d.%63s", &li, field) == 2 && li >= 0 && li < c.n_layers) {
-        fh_llama_layer &l = m->layers[li];
+        fh_llama_layer &l = m->layer[li];
         if (!strcmp(field, "attn_q.weight")) return loadq(&l.wq, QD, D);
         if (!strcmp(field, "attn_k.weight")) return loadq(&l.wk, KD, D);
         if (!strcmp(field, "attn_v.weight")) return loadq(&l.wv, KD, D);
@@ -251,7 +257,8 @@ extern "C" fh_status fh_llama_load_tensor(fh_llama *m, const char *name, uint32_
     FH_FAIL(FH_ERR_INVALID, "unknown tensor name '%s'", name);
 }
 
-static fh_status ensure_steps(fh_llama *m, int s) {
+fh_status fh_llama::ensure_steps(int s) {
+    fh_llama *m = this;
     if (s <= m->cap_s) return FH_OK;
     (void)hipStreamSynchronize(m->dev->stream);
     free_steps(m);
@@ -276,6 +283,10 @@ static fh_status ensure_steps(fh_llama *m, int s) {
 
 extern "C" fh_status fh_llama_finalize(fh_llama *m) {
     FH_REQUIRE(m, "NULL argument");
+    return m->finalize();
+}
+fh_status fh_llama::finalize() {
+    fh_llama *m = this;
     FH_REQUIRE(!m->finalized, "decoder already finalized");
     const fh_llama_config &c = m->c;
     FH_REQUIRE(m->embd && m->out_norm, "token_embd.weight / output_norm.weight missing");
@@ -284,7 +295,7 @@ extern "C" fh_status fh_llama_finalize(fh_llama *m) {
         m->output_is_embd = true;
     }
     for (int i = 0; i < c.n_layers; i++) {
-        fh_llama_layer &l = m->layers[i];
+        fh_llama_layer &l = m->layer[i];
         FH_REQUIRE(l.wq && l.wk && l.wv && l.wo && l.gate && l.up && l.down && l.attn_norm && l.ffn_norm,
                    "layer %d is missing tensors", i);
         if (c.fuse_qkv) {
@@ -312,40 +323,38 @@ extern "C" fh_status fh_llama_finalize(fh_llama *m) {
     FH_TRY(fh_rope_tables_scaled(m->dev, c.head_dim, c.ctx, c.theta, m->has_rope_scaling ? &m->rope_scaling : nullptr,
                                  m->rope_freq_weight.empty() ? nullptr : m->rope_freq_weight.data(), m->cos_t, m->sin_t));
     FH_TRY(fh_kvcache_create(m->dev, c.n_layers, c.n_kv_heads, c.head_dim, c.ctx, c.kv_dtype, &m->cache));
-    FH_TRY(fh_malloc(m->dev, (size_t)c.vocab * 4, (void **)&m->logits));
-    FH_TRY(fh_malloc(m->dev, 256, (void **)&m->tok_dev));
-    FH_TRY(fh_malloc(m->dev, (size_t)c.ctx * 4 + 256, (void **)&m->out_tok_dev));
-    FH_TRY(fh_malloc(m->dev, 256, (void **)&m->step_dev));
-    FH_TRY(fh_malloc(m->dev, (size_t)(128 + c.ctx) * 4, (void **)&m->samp_dev));
-    FH_TRY(ensure_steps(m, 1));
+    FH_TRY(m->create_loop_buffers());
+    FH_TRY(m->ensure_steps(1));
     m->finalized = true;
     return FH_OK;
 }
 
 extern "C" fh_status fh_llama_reset(fh_llama *m) {
     FH_REQUIRE(m && m->finalized, "decoder not finalized");
-    m->pos = 0;
-    m->history.clear();
-    return fh_kvcache_reset(m->cache);
+    return m->reset();
 }
 
 extern "C" fh_status fh_llama_weight_bytes(const fh_llama *m, uint64_t *bytes) {
     FH_REQUIRE(m && bytes, "NULL argument");
+    *bytes = m->weight_bytes();
+    return FH_OK;
+}
+uint64_t fh_llama::weight_bytes() const {
     uint64_t t = 0;
     auto add = [&](const fh_qmatrix *q) {
         if (q) t += (uint64_t)q->n * q->kb * fh_block_bytes(q->type);
     };
-    for (auto &l : m->layers) {
+    for (auto &l : layer) {
         add(l.wq); add(l.wk); add(l.wv); add(l.wo); add(l.gate); add(l.up); add(l.down); add(l.qkv); add(l.gate_up);
     }
-    add(m->output); // the lm-head; the embedding table contributes one row per token
-    *bytes = t;
-    return FH_OK;
+    add(output); // the lm-head; the embedding table contributes one row per token
+    return t;
 }
 
 // One decoder pass over `s` tokens whose ids are already in m->ids.  dev_pos: read the position
 // from the cache's device-side length (graph replay, s == 1) instead of m->pos.
-static fh_status run_layers(fh_llama *m, int s, bool dev_pos) {
+fh_status fh_llama::layers(int s, bool dev_pos) {
+    fh_llama *m = this;
     const fh_llama_config &c = m->c;
     fh_device *dev = m->dev;
     const int D = c.d_model, H = c.n_heads, HK = c.n_kv_heads, hd = c.head_dim, F = c.ffn;
@@ -353,14 +362,14 @@ static fh_status run_layers(fh_llama *m, int s, bool dev_pos) {
     const int pos = m->pos;
     const float scale = (float)(1.0 / sqrt((double)hd)); // attention_layer.rs:674
     FH_TRY(fh_embed_rows(m->embd, m->ids, nullptr, s, m->x));
-    const bool trace = !dev_pos && (dev->opt_trace_nan || dev->opt_trace_timing); // never inside a captured step
+    const bool trace = tracing = !dev_pos && (dev->opt_trace_nan || dev->opt_trace_timing); // never inside a captured step
     if (trace) {
         FH_TRY(trace_probe(m, m->x, s, D, -1, "embed"));
         FH_TRY(trace_mark(m, 1, -1, "embed"));
         m->trace_first = (int)m->trace_label.size() - 1;
     }
     for (int li = 0; li < c.n_layers; li++) {
-        fh_llama_layer &l = m->layers[li];
+        fh_llama_layer &l = m->layer[li];
         // Decode steps fold each rms_norm into the matvec that consumes it (one launch instead of two).
         const bool fuse = dev_pos && s == 1 && dev->opt_fuse_norm == 0 && dev->opt_matvec_kernel == 0;
         bool qkv_done = false, wo_done = false, xacc = false;
@@ -508,50 +517,27 @@ static fh_status run_layers(fh_llama *m, int s, bool dev_pos) {
         if (dev->opt_trace_timing == 1) FH_TRY(trace_mark(m, 1, -1, "layers"));
         m->trace_last = (int)m->trace_label.size() - 1;
     }
-    FH_TRY(fh_rms_norm(dev, m->x + (size_t)(s - 1) * D, nullptr, m->out_norm, nullptr, c.eps, 1, D, m->xn));
-    FH_TRY(fh_qmatmul(m->output, m->xn, 1, m->logits));
-    if (trace) FH_TRY(trace_mark(m, 2, -1, "out_norm+lm_head"));
     return FH_OK;
 }
 
+fh_status fh_llama::head(int row, float *out) {
+    FH_TRY(fh_rms_norm(dev, x + (size_t)row * c.d_model, nullptr, out_norm, nullptr, c.eps, 1, c.d_model, xn));
+    FH_TRY(fh_qmatmul(output, xn, 1, out));
+    return tracing ? trace_mark(this, 2, -1, "out_norm+lm_head") : FH_OK;
+}
+
+fh_status fh_llama::forward_begin() {
+    trace_text.clear();
+    trace_label.clear();
+    trace_first = trace_last = -1;
+    return FH_OK;
+}
+fh_status fh_llama::forward_end(int count) { return dev->opt_trace_timing ? trace_report(this, count) : FH_OK; }
+
 extern "C" fh_status fh_llama_forward(fh_llama *m, const uint32_t *tokens_host, int32_t count, float *logits_host,
                                       float *hidden_host) {
-    FH_REQUIRE(m && m->finalized && tokens_host, "decoder not finalized or NULL tokens");
-    FH_REQUIRE(count > 0 && count <= 65535, "count %d out of range", count);
-    for (int i = 0; i < count; i++)
-        FH_REQUIRE(tokens_host[i] < (uint32_t)m->c.vocab, "token id %u at %d outside the vocabulary of %d", tokens_host[i], i,
-                   m->c.vocab);
-    // Model::forward, raw/mod.rs:769-801: when the new tokens do not fit the context, the cache is cleared and the last
-    // context_length - 32 (at least 8) of all tokens, cached and new, are run again from position 0.
-    std::vector<uint32_t> trimmed;
-    if (m->pos + count > m->c.ctx) {
-        const int cutoff = std::max(m->c.ctx - 32, 8);
-        FH_REQUIRE(cutoff <= m->c.ctx && cutoff <= 65535, "context of %d positions is too short to trim to %d", m->c.ctx, cutoff);
-        FH_REQUIRE((int)m->history.size() == m->pos, "the cache holds %d positions but %zu token ids are on record", m->pos,
-                   m->history.size());
-        trimmed = m->history;
-        trimmed.insert(trimmed.end(), tokens_host, tokens_host + count);
-        trimmed.erase(trimmed.begin(), trimmed.end() - cutoff);
-        FH_TRY(fh_llama_reset(m));
-        tokens_host = trimmed.data();
-        count = cutoff;
-    }
-    FH_TRY(ensure_steps(m, count));
-    FH_TRY(fh_upload(m->dev, m->ids, tokens_host, (size_t)count * 4));
-    m->trace_text.clear();
-    m->trace_label.clear();
-    m->trace_first = m->trace_last = -1;
-    FH_TRY(run_layers(m, count, false));
-    // all layers appended: advance the cache
-    m->history.insert(m->history.end(), tokens_host, tokens_host + count);
-    m->pos += count;
-    m->cache->len = m->pos;
-    FH_TRY(fh_kvcache_set_len_dev(m->cache, m->pos));
-    if (hidden_host) FH_TRY(fh_download(m->dev, hidden_host, m->xn, (size_t)m->c.d_model * 4));
-    if (logits_host) FH_TRY(fh_download(m->dev, logits_host, m->logits, (size_t)m->c.vocab * 4));
-    FH_TRY(fh_device_sync(m->dev));
-    if (m->dev->opt_trace_timing) FH_TRY(trace_report(m, count));
-    return FH_OK;
+    FH_REQUIRE(m, "NULL decoder");
+    return m->forward(tokens_host, count, nullptr, 0, logits_host, hidden_host);
 }
 
 extern "C" fh_status fh_llama_trace_text(const fh_llama *m, char *buf, size_t capacity, size_t *length) {
@@ -565,177 +551,17 @@ extern "C" fh_status fh_llama_trace_text(const fh_llama *m, char *buf, size_t ca
     return FH_OK;
 }
 
-__global__ void k_set_u32(uint32_t *p, uint32_t v) { *p = v; }
-
-static fh_status decode_step_enqueue(fh_llama *m) {
-    FH_TRY(run_layers(m, 1, true));
-    // the last stage of the pick also stores the token, feeds it to the next step and advances the cache length
-    return fh_argmax_step(m->dev, m->logits, m->c.vocab, m->tok_dev,
-                          FhStepTail{m->ids, m->out_tok_dev, m->step_dev, m->cache->len_dev});
-}
-
 extern "C" fh_status fh_llama_decode_greedy(fh_llama *m, uint32_t first_token, int32_t steps, uint32_t *out_tokens_host,
                                             float *elapsed_ms) {
-    FH_REQUIRE(m && m->finalized && out_tokens_host, "decoder not finalized or NULL output");
-    FH_REQUIRE(steps > 0 && m->pos + steps <= m->c.ctx,
-               "context overflow: %d + %d > %d (the device-side loops stop at the context length; fh_llama_forward trims)", m->pos,
-               steps, m->c.ctx);
-    FH_REQUIRE(first_token < (uint32_t)m->c.vocab, "token id %u outside the vocabulary", first_token);
-    fh_device *dev = m->dev;
-    hipStream_t s = dev->stream;
-    // capacity is fixed for the whole run so that no reallocation happens between steps
-    FH_TRY(fh_kvcache_reserve(m->cache, m->pos + steps));
-    k_set_u32<<<1, 1, 0, s>>>(m->ids, first_token);
-    k_set_u32<<<1, 1, 0, s>>>((uint32_t *)m->step_dev, 0u);
-    FH_HIP(hipGetLastError());
-    int done = 0;
-    if (m->c.use_graph) {
-        // One eager step sizes every scratch buffer and sets kernel attributes; the capture then
-        // records launches only.  The graph depends on the cache capacity (strides), so it is
-        // rebuilt when the capacity changed since the last capture.
-        if (!m->graph_exec || m->captured_capacity != m->cache->capacity || m->captured_gen != dev->scratch_gen ||
-            m->captured_opt != dev->opt_gen) {
-            FH_TRY(fh_timer_start(dev));
-            FH_TRY(decode_step_enqueue(m));
-            done = 1;
-            FH_HIP(hipStreamSynchronize(s));
-            if (m->graph_exec) { (void)hipGraphExecDestroy(m->graph_exec); m->graph_exec = nullptr; }
-            if (m->graph) { (void)hipGraphDestroy(m->graph); m->graph = nullptr; }
-            FH_HIP(hipStreamBeginCapture(s, hipStreamCaptureModeThreadLocal));
-            fh_status st = decode_step_enqueue(m);
-            hipError_t e = hipStreamEndCapture(s, &m->graph);
-            if (st != FH_OK) return st;
-            FH_HIP(e);
-            FH_HIP(hipGraphInstantiate(&m->graph_exec, m->graph, nullptr, nullptr, 0));
-            m->captured_capacity = m->cache->capacity;
-            m->captured_gen = dev->scratch_gen;
-            m->captured_opt = dev->opt_gen;
-        } else {
-            FH_TRY(fh_timer_start(dev));
-        }
-        for (; done < steps; done++) FH_HIP(hipGraphLaunch(m->graph_exec, s));
-    } else {
-        FH_TRY(fh_timer_start(dev));
-        for (; done < steps; done++) FH_TRY(decode_step_enqueue(m));
-    }
-    float ms = 0.f;
-    FH_TRY(fh_timer_stop(dev, &ms));
-    if (elapsed_ms) *elapsed_ms = ms;
-    m->pos += steps;
-    m->cache->len = m->pos;
-    FH_TRY(fh_download(dev, out_tokens_host, m->out_tok_dev, (size_t)steps * 4));
-    m->history.push_back(first_token); // the cache now holds the step inputs: the first token and all outputs but the last
-    m->history.insert(m->history.end(), out_tokens_host, out_tokens_host + steps - 1);
-    return FH_OK;
-}
-
-// Sampled decode (models/kalosm-llama/src/model/inference.rs:38-173, forward.rs:346-404): the sampled id stays in
-// device memory and feeds the next step; it also joins the window of previous ids that the repetition penalty
-// looks at (membership only, so the window is a ring).
-__global__ void k_store_sampled(const uint32_t *result, uint32_t *ids, uint32_t *out, int *step, uint32_t *prev,
-                                uint32_t range, int *kv_len) {
-    *kv_len = *kv_len + 1;
-    const uint32_t t = result[0] == FH_SAMPLE_STATUS_SAMPLED ? result[1] : 0xFFFFFFFFu;
-    const uint32_t next = t == 0xFFFFFFFFu ? 0u : t;
-    ids[0] = next;
-    out[*step] = t;
-    *step = *step + 1;
-    if (range) {
-        const uint32_t slot = prev[65];
-        prev[slot] = next;
-        prev[65] = slot + 1 == range ? 0u : slot + 1;
-        if (prev[64] < range) prev[64] = prev[64] + 1;
-    }
-}
-
-static fh_status sampled_step_enqueue(fh_llama *m) {
-    FH_TRY(run_layers(m, 1, true));
-    uint32_t *sd = m->samp_dev;
-    FH_TRY(fh_sample_token_dev(m->dev, m->logits, m->c.vocab, &m->samp_params, sd, sd + 64, 0, (const float *)(sd + 128),
-                               m->step_dev, (float *)(sd + 66), sd + 68, nullptr, nullptr));
-    k_store_sampled<<<1, 1, 0, m->dev->stream>>>(sd + 68, m->ids, m->out_tok_dev, m->step_dev, sd, m->samp_range,
-                                                m->cache->len_dev);
-    FH_HIP(hipGetLastError());
-    return FH_OK;
+    FH_REQUIRE(m, "NULL decoder");
+    return m->decode_greedy(first_token, steps, out_tokens_host, elapsed_ms);
 }
 
 extern "C" fh_status fh_llama_decode_sampled(fh_llama *m, uint32_t first_token, int32_t steps,
                                              const fh_sampler_params *params, const float *randoms_host,
                                              const uint32_t *previous_host, uint32_t n_previous, uint32_t repetition_range,
                                              float *mu, uint32_t *out_tokens_host, float *elapsed_ms) {
-    FH_REQUIRE(m && m->finalized && out_tokens_host && params && randoms_host, "decoder not finalized or NULL argument");
-    FH_REQUIRE(steps > 0 && m->pos + steps <= m->c.ctx,
-               "context overflow: %d + %d > %d (the device-side loops stop at the context length; fh_llama_forward trims)", m->pos,
-               steps, m->c.ctx);
-    FH_REQUIRE(first_token < (uint32_t)m->c.vocab, "token id %u outside the vocabulary", first_token);
-    FH_REQUIRE(n_previous == 0 || previous_host, "previous tokens missing");
-    FH_REQUIRE(params->kind != FH_SAMPLER_MIROSTAT2 || mu, "Mirostat 2 needs its state");
-    fh_device *dev = m->dev;
-    hipStream_t s = dev->stream;
-    const uint32_t range = repetition_range < FH_SAMPLER_PREVIOUS_TOKENS ? repetition_range : FH_SAMPLER_PREVIOUS_TOKENS;
-    // window = the last `range` ids of (history, first_token)
-    uint32_t head[128] = {0};
-    uint32_t len = 0;
-    if (range) {
-        const uint32_t keep = n_previous < range - 1 ? n_previous : range - 1;
-        for (uint32_t i = 0; i < keep; i++) head[len++] = previous_host[n_previous - keep + i];
-        head[len++] = first_token;
-    }
-    head[64] = len;
-    head[65] = range ? len % range : 0u;
-    const float mu0 = mu ? *mu : 0.f;
-    memcpy(&head[66], &mu0, 4);
-    FH_TRY(fh_upload(dev, m->samp_dev, head, sizeof(head)));
-    FH_TRY(fh_upload(dev, m->samp_dev + 128, randoms_host, (size_t)steps * 4));
-    FH_TRY(fh_kvcache_reserve(m->cache, m->pos + steps));
-    k_set_u32<<<1, 1, 0, s>>>(m->ids, first_token);
-    k_set_u32<<<1, 1, 0, s>>>((uint32_t *)m->step_dev, 0u);
-    FH_HIP(hipGetLastError());
-    int done = 0;
-    if (m->c.use_graph) {
-        // the captured step holds the sampler's parameters and the window size as kernel arguments
-        fh_sampler_params want = *params;
-        want.random = 0.f; // every step takes its number from randoms_host
-        const bool same = m->samp_exec && m->samp_capacity == m->cache->capacity && m->samp_range == range &&
-                          m->samp_gen == dev->scratch_gen && m->samp_opt == dev->opt_gen &&
-                          memcmp(&m->samp_params, &want, sizeof(want)) == 0;
-        m->samp_params = want;
-        m->samp_range = range;
-        if (!same) {
-            FH_TRY(fh_timer_start(dev));
-            FH_TRY(sampled_step_enqueue(m));
-            done = 1;
-            FH_HIP(hipStreamSynchronize(s));
-            if (m->samp_exec) { (void)hipGraphExecDestroy(m->samp_exec); m->samp_exec = nullptr; }
-            if (m->samp_graph) { (void)hipGraphDestroy(m->samp_graph); m->samp_graph = nullptr; }
-            m->samp_capacity = -1;
-            FH_HIP(hipStreamBeginCapture(s, hipStreamCaptureModeThreadLocal));
-            fh_status st = sampled_step_enqueue(m);
-            hipError_t e = hipStreamEndCapture(s, &m->samp_graph);
-            if (st != FH_OK) return st;
-            FH_HIP(e);
-            FH_HIP(hipGraphInstantiate(&m->samp_exec, m->samp_graph, nullptr, nullptr, 0));
-            m->samp_capacity = m->cache->capacity;
-            m->samp_gen = dev->scratch_gen;
-            m->samp_opt = dev->opt_gen;
-        } else {
-            FH_TRY(fh_timer_start(dev));
-        }
-        for (; done < steps; done++) FH_HIP(hipGraphLaunch(m->samp_exec, s));
-    } else {
-        m->samp_params = *params;
-        m->samp_range = range;
-        FH_TRY(fh_timer_start(dev));
-        for (; done < steps; done++) FH_TRY(sampled_step_enqueue(m));
-    }
-    float ms = 0.f;
-    FH_TRY(fh_timer_stop(dev, &ms));
-    if (elapsed_ms) *elapsed_ms = ms;
-    m->pos += steps;
-    m->cache->len = m->pos;
-    FH_TRY(fh_download(dev, out_tokens_host, m->out_tok_dev, (size_t)steps * 4));
-    if (mu) FH_TRY(fh_download(dev, mu, m->samp_dev + 66, 4));
-    m->history.push_back(first_token);
-    m->history.insert(m->history.end(), out_tokens_host, out_tokens_host + steps - 1);
-    return FH_OK;
+    FH_REQUIRE(m, "NULL decoder");
+    return m->decode_sampled(first_token, steps, params, randoms_host, previous_host, n_previous, repetition_range, mu,
+                             out_tokens_host, elapsed_ms);
 }

@@ -3,6 +3,8 @@
 // Reference: fusor-ml/fusor/src/quantized.rs:80-279, fusor-ml/fusor/src/layers/embedding.rs:43-89.
 #include "fh_blocks.h"
 
+#include <cstring>
+
 // ------------------------------------------------------------------------------ repack
 // One thread per (row, source block).  The source is the GGUF stream ([n][kb] blocks); the
 // destination is the tile record.  Upload-time only.
@@ -106,7 +108,7 @@ static fh_status qm_alloc(fh_device *dev, uint32_t type, int64_t n, int64_t k, f
     int e = fh_block_elems(type);
     if (!e)
         FH_FAIL(FH_ERR_UNSUPPORTED, "unsupported ggml type %u (supported: F32=0, F16=1, Q4_0=2, Q5_0=6, Q8_0=8, Q4_K=12, "
-                                    "Q5_K=13, Q6_K=14)", type);
+                                    "Q5_K=13, Q6_K=14, BF16=30)", type);
     FH_REQUIRE(n > 0 && k > 0, "empty weight [%lld, %lld]", (long long)n, (long long)k);
     FH_REQUIRE(k % e == 0, "k=%lld is not a multiple of the block size %d", (long long)k, e);
     FH_REQUIRE(n < (1ll << 31) && k < (1ll << 31), "weight too large");
@@ -125,6 +127,10 @@ static fh_status qm_alloc(fh_device *dev, uint32_t type, int64_t n, int64_t k, f
         q->recs = 0;
         q->rec_bytes = fh_block_bytes(type);
         q->bytes = (size_t)n * (size_t)q->kb * (size_t)fh_block_bytes(type);
+        if (type == FH_BF16) { // padded rows (see fh_internal.h)
+            q->recs = (k + 63) / 64 * 64;
+            q->bytes = (size_t)q->n_pad * (size_t)q->recs * 2;
+        }
     }
     hipError_t err = hipMalloc((void **)&q->data, q->bytes + 256); // slack: kernels may prefetch one record ahead
     if (err != hipSuccess) {
@@ -150,7 +156,13 @@ extern "C" fh_status fh_qmatrix_from_gguf_bytes(fh_device *dev, uint32_t ggml_ty
                 (long long)n, (long long)k, ggml_type, want);
     }
     if (fh_is_plain(ggml_type)) {
-        hipError_t e = hipMemcpyAsync(q->data, bytes, len, hipMemcpyHostToDevice, dev->stream);
+        hipError_t e = hipSuccess;
+        if (ggml_type == FH_BF16) {
+            e = hipMemsetAsync(q->data, 0, q->bytes + 256, dev->stream);
+            if (e == hipSuccess)
+                e = hipMemcpy2DAsync(q->data, (size_t)q->recs * 2, bytes, (size_t)k * 2, (size_t)k * 2, (size_t)n, hipMemcpyHostToDevice,
+                                     dev->stream);
+        } else e = hipMemcpyAsync(q->data, bytes, len, hipMemcpyHostToDevice, dev->stream);
         if (e == hipSuccess) e = hipStreamSynchronize(dev->stream);
         if (e != hipSuccess) {
             fh_qmatrix_free(q);
@@ -199,6 +211,40 @@ extern "C" fh_status fh_qmatrix_from_gguf_bytes(fh_device *dev, uint32_t ggml_ty
     return FH_OK;
 }
 
+fh_status fh_qmatrix_alloc_bf16(fh_device *dev, int64_t n, int64_t k, fh_qmatrix **out) {
+    FH_HIP(hipSetDevice(dev->ordinal));
+    fh_qmatrix *q = nullptr;
+    FH_TRY(qm_alloc(dev, FH_BF16, n, k, &q));
+    hipError_t e = hipMemsetAsync(q->data, 0, q->bytes + 256, dev->stream);
+    if (e == hipSuccess) e = hipStreamSynchronize(dev->stream);
+    if (e != hipSuccess) {
+        fh_qmatrix_free(q);
+        FH_FAIL(FH_ERR_HIP, "hipMemsetAsync failed: %s", hipGetErrorString(e));
+    }
+    *out = q;
+    return FH_OK;
+}
+
+fh_status fh_qmatrix_put_bf16(fh_qmatrix *q, int64_t row0, int64_t n, int64_t k, const void *bytes, bool interleave) {
+    FH_REQUIRE(q && q->type == FH_BF16 && k == q->k && bytes && n > 0, "bad rows for a bf16 matrix");
+    const int64_t ld = q->recs, last = interleave ? row0 + 32 * ((n - 1) / 16) + (n - 1) % 16 : row0 + n - 1;
+    FH_REQUIRE(row0 >= 0 && last < q->n, "rows %lld .. %lld of %lld", (long long)row0, (long long)last, (long long)q->n);
+    hipStream_t s = q->dev->stream;
+    uint8_t *dst = q->data + (size_t)row0 * ld * 2;
+    if (!interleave) {
+        FH_HIP(hipMemcpy2DAsync(dst, (size_t)ld * 2, bytes, (size_t)k * 2, (size_t)k * 2, (size_t)n, hipMemcpyHostToDevice, s));
+    } else {
+        // whole groups of 16 padded rows at a time; the rows that complete the last group are zero already
+        const int64_t groups = (n + 15) / 16;
+        std::vector<uint8_t> rows((size_t)groups * 16 * ld * 2, 0);
+        for (int64_t r = 0; r < n; r++) memcpy(rows.data() + (size_t)r * ld * 2, (const uint8_t *)bytes + (size_t)r * k * 2, (size_t)k * 2);
+        FH_HIP(hipMemcpy2DAsync(dst, (size_t)ld * 64, rows.data(), (size_t)ld * 32, (size_t)ld * 32, (size_t)groups, hipMemcpyHostToDevice, s));
+        FH_HIP(hipStreamSynchronize(s));
+    }
+    FH_HIP(hipStreamSynchronize(s));
+    return FH_OK;
+}
+
 extern "C" fh_status fh_qmatrix_free(fh_qmatrix *q) {
     if (!q) return FH_OK;
     if (q->data) {
@@ -238,13 +284,19 @@ extern "C" fh_status fh_qmatrix_concat_rows(fh_device *dev, const fh_qmatrix *co
     fh_qmatrix *q = nullptr;
     FH_TRY(qm_alloc(dev, parts[0]->type, n, parts[0]->k, &q));
     size_t off = 0;
+    const bool bf = q->type == FH_BF16;
+    if (bf && hipMemsetAsync(q->data, 0, q->bytes + 256, dev->stream) != hipSuccess) {
+        fh_qmatrix_free(q);
+        FH_FAIL(FH_ERR_HIP, "hipMemsetAsync failed");
+    }
     for (int i = 0; i < count; i++) {
-        hipError_t e = hipMemcpyAsync(q->data + off, parts[i]->data, parts[i]->bytes, hipMemcpyDeviceToDevice, dev->stream);
+        const size_t part = bf ? (size_t)parts[i]->n * parts[i]->recs * 2 : parts[i]->bytes; // without the padding rows
+        hipError_t e = hipMemcpyAsync(q->data + off, parts[i]->data, part, hipMemcpyDeviceToDevice, dev->stream);
         if (e != hipSuccess) {
             fh_qmatrix_free(q);
             FH_FAIL(FH_ERR_HIP, "hipMemcpyAsync failed: %s", hipGetErrorString(e));
         }
-        off += parts[i]->bytes;
+        off += part;
         if (i == 0 || parts[i]->wscale < q->wscale) q->wscale = parts[i]->wscale; // the largest |w| decides
     }
     *out = q;
@@ -277,6 +329,7 @@ extern "C" fh_status fh_qmatrix_dequantize(const fh_qmatrix *q, float *out_dev) 
     case FH_Q5_K: k_dequantize<FH_Q5_K><<<grid, block, 0, s>>>(v, out_dev); break;
     case FH_W_F32: k_dequantize<FH_W_F32><<<grid, block, 0, s>>>(v, out_dev); break;
     case FH_W_F16: k_dequantize<FH_W_F16><<<grid, block, 0, s>>>(v, out_dev); break;
+    case FH_BF16: k_dequantize<FH_BF16><<<grid, block, 0, s>>>(v, out_dev); break;
     }
     FH_HIP(hipGetLastError());
     return FH_OK;
@@ -315,6 +368,7 @@ extern "C" fh_status fh_embed_rows(const fh_qmatrix *q, const uint32_t *ids_dev,
     case FH_Q5_K: k_embed_rows<FH_Q5_K><<<grid, block, 0, s>>>(v, ids_dev, count, out_dev); break;
     case FH_W_F32: k_embed_rows<FH_W_F32><<<grid, block, 0, s>>>(v, ids_dev, count, out_dev); break;
     case FH_W_F16: k_embed_rows<FH_W_F16><<<grid, block, 0, s>>>(v, ids_dev, count, out_dev); break;
+    case FH_BF16: k_embed_rows<FH_BF16><<<grid, block, 0, s>>>(v, ids_dev, count, out_dev); break;
     }
     FH_HIP(hipGetLastError());
     return FH_OK;

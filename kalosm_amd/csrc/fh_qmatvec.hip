@@ -387,6 +387,7 @@ fh_status fh_launch_qmatvec(const fh_qmatrix *q, const float *x, int m, float *y
     case FH_Q5_K: return launch_generic<FH_Q5_K>(q, x, m, y, epi, a, b);
     case FH_W_F32: return launch_generic<FH_W_F32>(q, x, m, y, epi, a, b);
     case FH_W_F16: return launch_generic<FH_W_F16>(q, x, m, y, epi, a, b);
+    case FH_BF16: return launch_generic<FH_BF16>(q, x, m, y, epi, a, b);
     }
     FH_FAIL(FH_ERR_UNSUPPORTED, "unsupported type %u", q->type);
 }
@@ -400,6 +401,7 @@ static fh_status qmm_check(const fh_qmatrix *q, const void *x, int m, const void
 extern "C" fh_status fh_qmatmul(const fh_qmatrix *q, const float *x_dev, int32_t m, float *y_dev) {
     FH_TRY(qmm_check(q, x_dev, m, y_dev));
     const int64_t mk = q->dev->opt_matmul_kernel;
+    if (q->type == FH_BF16 && mk != 1 && q->dev->opt_matvec_kernel != 1) return fh_launch_bf16_matmul(q, x_dev, 0, m, y_dev);
     // dense f16 / f32 weight rows (core/src/quantized/matmul/kernel.rs:132-193 routes them to the dense matmul) take
     // the matrix-core tiles as well once there are rows to fill them
     const bool dense = (q->type == FH_W_F16 || q->type == FH_W_F32) && q->k % 32 == 0;

@@ -1785,6 +1785,7 @@ static fh_status qmm_launch_dense(const fh_qmatrix *q, const _Float16 *xh, const
 fh_status fh_launch_qmatmul_tile(const fh_qmatrix *q, const void *x, int x_is_bf16, int m, float *y) {
     fh_device *dev = q->dev;
     const int64_t K = q->k;
+    if (q->type == FH_BF16) return fh_launch_bf16_matmul(q, x, x_is_bf16, m, y);
     if (fh_is_plain(q->type) && K % 32 != 0)
         FH_FAIL(FH_ERR_UNSUPPORTED, "type %u with k = %lld has no matrix-core matmul (it runs through fh_qmatmul)", q->type,
                 (long long)K);

@@ -1,0 +1,329 @@
+// Decode step kernels of the layer-list decoders (fh_step.h).
+#include "fh_step.h"
+
+static constexpr float FH_LOG2E = 1.4426950408889634f;
+
+__device__ __forceinline__ float dot8(const uint4 &w, const float *x, float acc) {
+    const float4 a = *(const float4 *)x, b = *(const float4 *)(x + 4);
+    acc = fmaf(fh_bf_lo(w.x), a.x, acc);
+    acc = fmaf(fh_bf_hi(w.x), a.y, acc);
+    acc = fmaf(fh_bf_lo(w.y), a.z, acc);
+    acc = fmaf(fh_bf_hi(w.y), a.w, acc);
+    acc = fmaf(fh_bf_lo(w.z), b.x, acc);
+    acc = fmaf(fh_bf_hi(w.z), b.y, acc);
+    acc = fmaf(fh_bf_lo(w.w), b.z, acc);
+    acc = fmaf(fh_bf_hi(w.w), b.w, acc);
+    return acc;
+}
+
+// One step of a recurrence: workgroup b takes 16 columns of one head's state, RPT rows per lane as in the prefill scan.
+template <int RPT>
+__device__ __forceinline__ void rec_step(const FhStep &st, int b, float *lds) {
+    const FhRecurrent &r = st.rec;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, rg = lane & 15;
+    const int ncb = (r.vdim + 15) / 16, h = b / ncb, cb = b % ncb, d = r.dim, rep = r.heads / r.kv_heads, kh = h / rep;
+    const int nq = r.kv_heads * d, channels = 2 * nq + r.heads * r.vdim, pos = *st.pos_dev;
+    const int col = cb * 16 + wave * 4 + (lane >> 4), i0 = rg * RPT;
+    const bool live = col < r.vdim;
+    const int c = live ? col : r.vdim - 1;
+    float *sp = st.rec_state.s + ((int64_t)h * r.vdim + c) * d;
+    float S[RPT];
+#pragma unroll
+    for (int i = 0; i < RPT; i++) S[i] = pos > 0 && i0 + i < d ? sp[i0 + i] : 0.f;
+    float *qk = lds, *vv = lds + 2 * d, *f = vv + 16; // [2 d], [16], [2]
+    float *slot = st.rec_state.conv + (int64_t)(pos % r.taps) * channels; // not among the rows the convolution reads
+    const bool keep = cb == 0 && h % rep == 0;        // one workgroup per key head stores its projections
+    for (int i = tid; i < 2 * d; i += 256) {
+        const int ch = i < d ? kh * d + i : nq + kh * d + i - d;
+        qk[i] = fh_rec_conv(r, ch, st.proj, 0, 0, pos, st.rec_state.conv, channels);
+        if (keep) slot[ch] = st.proj[i < d ? r.col_q + kh * d + i : r.col_k + kh * d + i - d];
+    }
+    if (tid < 16 && cb * 16 + tid < r.vdim) {
+        const int vc = h * r.vdim + cb * 16 + tid;
+        vv[tid] = fh_rec_conv(r, 2 * nq + vc, st.proj, 0, 0, pos, st.rec_state.conv, channels);
+        slot[2 * nq + vc] = st.proj[r.col_v + vc];
+    }
+    __syncthreads();
+    if (wave < 2) {
+        float g = 1.f;
+        if (r.delta) {
+            float ss = 0.f;
+            for (int i = lane; i < d; i += 64) ss = fmaf(qk[wave * d + i], qk[wave * d + i], ss);
+            g = 1.0f / sqrtf(fh_wave_sum(ss) + 1e-6f);
+        }
+        if (lane == 0) f[wave] = wave == 0 ? g * r.q_scale : g;
+    }
+    const float sp_ = fh_softplus_f(st.proj[r.col_a + h] + r.dt_bias[h]);
+    const float g = expf(-expf(r.a_log[h]) * sp_), be = r.delta ? fh_sigmoid_f(st.proj[r.col_b + h]) : sp_;
+    __syncthreads();
+    const float v = vv[live ? wave * 4 + (lane >> 4) : 0];
+    float k[RPT], dot = 0.f, o = 0.f;
+#pragma unroll
+    for (int i = 0; i < RPT; i++) {
+        k[i] = i0 + i < d ? qk[d + i0 + i] * f[1] : 0.f;
+        S[i] *= g;
+        dot = fmaf(S[i], k[i], dot);
+    }
+    const float u = r.delta ? be * (v - fh_row16_sum(dot)) : be * v;
+#pragma unroll
+    for (int i = 0; i < RPT; i++) {
+        S[i] = fmaf(k[i], u, S[i]);
+        o = fmaf(S[i], i0 + i < d ? qk[i0 + i] * f[0] : 0.f, o);
+        if (live && i0 + i < d) sp[i0 + i] = S[i];
+    }
+    o = fh_row16_sum(o);
+    if (rg == 0 && live) st.o[h * r.vdim + col] = o + (r.d_skip ? r.d_skip[h] * v : 0.f);
+}
+
+// Absorbed queries of latent attention: workgroup b < heads * chunks takes 128 latent dimensions of one head, the last one
+// appends this position's cache row.
+template <typename T>
+__device__ __forceinline__ void latent_step(const FhStep &st, T *ring, int cap, int b, float *lds) {
+    const FhLatent &a = st.lat;
+    const int tid = threadIdx.x, chunks = (a.r8 + 127) / 128, pos = *st.pos_dev, row = a.r8 + a.drp;
+    const float *ct = a.cos_t + (int64_t)pos * a.pairs, *sn = a.sin_t + (int64_t)pos * a.pairs;
+    if (b == a.heads * chunks) {
+        const float *p = st.proj + a.col_kv;
+        float ss = 0.f;
+        for (int c = tid; c < a.rank; c += 256) ss = fmaf(p[c], p[c], ss);
+        ss = fh_wave_sum(ss);
+        if ((tid & 63) == 0) lds[tid >> 6] = ss;
+        __syncthreads();
+        const float inv = 1.0f / sqrtf((lds[0] + lds[1] + lds[2] + lds[3]) / (float)a.rank + a.eps);
+        T *dst = ring + (int64_t)(pos % cap) * row;
+        for (int c = tid; c < row; c += 256) {
+            float v = 0.f;
+            if (c < a.rank) v = p[c] * inv * a.c_norm[c];
+            else if (c >= a.r8 && c - a.r8 < a.dr) {
+                const int i = c - a.r8, pr = i >> 1;
+                v = p[a.rank + i];
+                if (pr < a.pairs) {
+                    const float o = p[a.rank + (i ^ 1)];
+                    v = (i & 1) ? v * ct[pr] + o * sn[pr] : v * ct[pr] - o * sn[pr];
+                }
+            }
+            dst[c] = fh_to<T>(v);
+        }
+        return;
+    }
+    const int h = b / chunks, c0 = (b % chunks) * 128, sub = tid & 15, dg = tid >> 4, c = c0 + sub * 8;
+    const float sc = a.scale * FH_LOG2E;
+    const float *q = st.proj + a.col_q + h * (a.dn + a.dr);
+    float acc[8];
+#pragma unroll
+    for (int e = 0; e < 8; e++) acc[e] = 0.f;
+    if (c < a.rp)
+        for (int d = dg; d < a.dn; d += 16) {
+            const uint4 w = *(const uint4 *)(a.uk + (int64_t)(h * a.dnp + d) * a.rp + c);
+            const float x = q[d];
+            acc[0] = fmaf(fh_bf_lo(w.x), x, acc[0]);
+            acc[1] = fmaf(fh_bf_hi(w.x), x, acc[1]);
+            acc[2] = fmaf(fh_bf_lo(w.y), x, acc[2]);
+            acc[3] = fmaf(fh_bf_hi(w.y), x, acc[3]);
+            acc[4] = fmaf(fh_bf_lo(w.z), x, acc[4]);
+            acc[5] = fmaf(fh_bf_hi(w.z), x, acc[5]);
+            acc[6] = fmaf(fh_bf_lo(w.w), x, acc[6]);
+            acc[7] = fmaf(fh_bf_hi(w.w), x, acc[7]);
+        }
+#pragma unroll
+    for (int e = 0; e < 8; e++) lds[dg * 128 + sub * 8 + e] = acc[e];
+    __syncthreads();
+    float *dst = st.qa + (int64_t)h * row;
+    if (tid < 128 && c0 + tid < a.r8) {
+        float v = 0.f;
+#pragma unroll
+        for (int g = 0; g < 16; g++) v += lds[g * 128 + tid];
+        dst[c0 + tid] = v * sc;
+    }
+    if (c0 == 0)
+        for (int i = tid; i < a.drp; i += 256) {
+            const int pr = i >> 1;
+            float v = i < a.dr ? q[a.dn + i] : 0.f;
+            if (i < a.dr && pr < a.pairs) {
+                const float o = q[a.dn + (i ^ 1)];
+                v = (i & 1) ? v * ct[pr] + o * sn[pr] : v * ct[pr] - o * sn[pr];
+            }
+            dst[a.r8 + i] = v * sc;
+        }
+}
+
+// Gate and up products of the chosen experts: a workgroup takes 8 activations of one of them, two per wavefront.
+__device__ __forceinline__ void expert_step(const FhStep &st, int b, float *lds) {
+    const FhMoe &m = st.moe;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, tiles = (m.ff + 7) / 8, slot = b / tiles, tile = b % tiles;
+    int *who = (int *)(lds + st.kp);
+    if (wave == 0)
+        fh_moe_route(st.proj + m.col_z, m.experts, m.scale, slot + 1, [&](int n, int e, float w) {
+            if (n == slot && lane == 0) {
+                *who = e;
+                if (tile == 0) st.ids[slot] = e, st.wts[slot] = w;
+            }
+        });
+    for (int i = tid; i < st.kp; i += 256) lds[i] = st.hn[i];
+    __syncthreads();
+    const uint16_t *w = m.gate_up + (int64_t)*who * m.gu_stride;
+    const uint16_t *row[4];
+    const int p0 = tile * 8 + wave * 2;
+#pragma unroll
+    for (int i = 0; i < 2; i++) {
+        const int p = p0 + i < m.ff ? p0 + i : m.ff - 1;
+        row[2 * i] = w + (int64_t)(p / 16 * 32 + p % 16) * st.kp;
+        row[2 * i + 1] = row[2 * i] + (int64_t)16 * st.kp;
+    }
+    float acc[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int c = lane * 8; c < st.kp; c += 512) {
+        uint4 u[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) u[i] = *(const uint4 *)(row[i] + c);
+#pragma unroll
+        for (int i = 0; i < 4; i++) acc[i] = dot8(u[i], lds + c, acc[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) acc[i] = fh_wave_sum(acc[i]);
+    if (lane == 0)
+#pragma unroll
+        for (int i = 0; i < 2; i++)
+            if (p0 + i < m.ff) st.act[(int64_t)slot * m.ffp + p0 + i] = fh_silu_f(acc[2 * i]) * acc[2 * i + 1];
+}
+
+template <int RPT>
+__global__ __launch_bounds__(256) void k_step_recurrent(FhStep st, int n_mix) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    if ((int)blockIdx.x < n_mix) rec_step<RPT>(st, blockIdx.x, lds);
+    else expert_step(st, (int)blockIdx.x - n_mix, lds);
+}
+template <typename T>
+__global__ __launch_bounds__(256) void k_step_latent(FhStep st, T *ring, int cap, int n_mix) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    if ((int)blockIdx.x < n_mix) latent_step<T>(st, ring, cap, blockIdx.x, lds);
+    else expert_step(st, (int)blockIdx.x - n_mix, lds);
+}
+
+fh_status fh_step_middle(fh_device *dev, int dtype, const FhStep &st, fh_kvcache *cache) {
+    const FhMoe &m = st.moe;
+    const int n_exp = m.experts ? m.top * ((m.ff + 7) / 8) : 0;
+    size_t lds = m.experts ? (size_t)(st.kp + 4) * 4 : 0;
+    if (st.kind == FH_MIX_RECURRENT) {
+        const int n_mix = st.rec.heads * ((st.rec.vdim + 15) / 16), rpt = (st.rec.dim + 15) / 16;
+        const size_t need = (size_t)(2 * st.rec.dim + 32) * 4;
+        lds = lds > need ? lds : need;
+        const void *fn = rpt <= 2 ? (const void *)k_step_recurrent<2> : rpt <= 4 ? (const void *)k_step_recurrent<4>
+                         : rpt <= 8 ? (const void *)k_step_recurrent<8> : (const void *)k_step_recurrent<16>;
+        FH_REQUIRE(rpt <= 16, "recurrent state of %d rows (at most 256)", st.rec.dim);
+        if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, fn, lds));
+        const dim3 grid((unsigned)(n_mix + n_exp));
+        if (rpt <= 2) k_step_recurrent<2><<<grid, 256, lds, dev->stream>>>(st, n_mix);
+        else if (rpt <= 4) k_step_recurrent<4><<<grid, 256, lds, dev->stream>>>(st, n_mix);
+        else if (rpt <= 8) k_step_recurrent<8><<<grid, 256, lds, dev->stream>>>(st, n_mix);
+        else k_step_recurrent<16><<<grid, 256, lds, dev->stream>>>(st, n_mix);
+    } else {
+        const int n_mix = st.lat.heads * ((st.lat.r8 + 127) / 128) + 1;
+        const size_t need = (size_t)16 * 128 * 4;
+        lds = lds > need ? lds : need;
+        const dim3 grid((unsigned)(n_mix + n_exp));
+        if (lds > 48 * 1024)
+            FH_TRY(fh_kernel_lds(dev, dtype == FH_F32 ? (const void *)k_step_latent<float> : (const void *)k_step_latent<uint16_t>, lds));
+        if (dtype == FH_F32) k_step_latent<float><<<grid, 256, lds, dev->stream>>>(st, (float *)cache->k, cache->capacity, n_mix);
+        else k_step_latent<uint16_t><<<grid, 256, lds, dev->stream>>>(st, (uint16_t *)cache->k, cache->capacity, n_mix);
+    }
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+// ------------------------------------------------------------------------------ output launch
+// Every workgroup stages the inputs of all products once (the recurrent mixers' gate and norm are applied on the way),
+// then each wavefront adds ROWS rows of the residual stream.
+template <int ROWS>
+__global__ __launch_bounds__(256) void k_step_out(FhStep st) {
+    extern __shared__ __attribute__((aligned(16))) float in[]; // [kpo | top * ffp | sffp | norm groups]
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const FhMoe &m = st.moe;
+    const int n_e = m.experts ? m.top : 0, n_in = st.kpo + n_e * m.ffp + (m.sff ? m.sffp : 0);
+    float *ie = in + st.kpo, *is = ie + n_e * m.ffp, *ginv = in + n_in;
+    const int row0 = ((int)blockIdx.x * 4 + wave) * ROWS;
+    const uint16_t *wr[ROWS];
+    uint4 first[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) {
+        wr[r] = st.wo + (int64_t)(row0 + r < st.width ? row0 + r : st.width - 1) * st.kpo;
+        first[r] = lane * 8 < st.kpo ? *(const uint4 *)(wr[r] + lane * 8) : uint4{0, 0, 0, 0};
+    }
+    if (st.kind == FH_MIX_RECURRENT) {
+        const FhRecurrent &r = st.rec;
+        const float *gate = st.proj + r.col_g;
+        const int inner = r.heads * r.vdim, gl = inner / r.norm_groups;
+        for (int i = tid; i < st.kpo; i += 256) {
+            float v = i < inner ? st.o[i] : 0.f;
+            if (r.gate_first && i < inner) v *= fh_silu_f(gate[i]);
+            in[i] = v;
+        }
+        __syncthreads();
+        for (int g = wave; g < r.norm_groups; g += 4) {
+            float ss = 0.f;
+            for (int i = lane; i < gl; i += 64) ss = fmaf(in[g * gl + i], in[g * gl + i], ss);
+            ss = fh_wave_sum(ss);
+            if (lane == 0) ginv[g] = 1.0f / sqrtf(ss / (float)gl + r.eps);
+        }
+        __syncthreads();
+        for (int i = tid; i < inner; i += 256) {
+            float v = in[i] * ginv[i / gl] * r.norm[r.norm_len == inner ? i : i % r.norm_len];
+            if (!r.gate_first) v *= fh_silu_f(gate[i]);
+            in[i] = v;
+        }
+    } else {
+        const int inner = st.lat.heads * st.lat.dv;
+        for (int i = tid; i < st.kpo; i += 256) in[i] = i < inner ? st.o[i] : 0.f;
+    }
+    for (int j = 0; j < n_e; j++) {
+        const float w = st.wts[j];
+        for (int i = tid; i < m.ffp; i += 256) ie[j * m.ffp + i] = i < m.ff ? w * st.act[(int64_t)j * m.ffp + i] : 0.f;
+    }
+    if (m.sff)
+        for (int i = tid; i < m.sffp; i += 256) {
+            const int g = i / 16 * 32 + i % 16;
+            is[i] = fh_silu_f(st.s_gu[g]) * st.s_gu[g + 16];
+        }
+    __syncthreads();
+    float acc[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) acc[r] = 0.f;
+    if (lane * 8 < st.kpo)
+#pragma unroll
+        for (int r = 0; r < ROWS; r++) acc[r] = dot8(first[r], in + lane * 8, acc[r]);
+    auto sweep = [&](const uint16_t *w, int kp, const float *x, int c0) {
+#pragma unroll
+        for (int r = 0; r < ROWS; r++) wr[r] = w + (int64_t)(row0 + r < st.width ? row0 + r : st.width - 1) * kp;
+#pragma unroll 2
+        for (int c = c0 + lane * 8; c < kp; c += 512) {
+            uint4 u[ROWS];
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) u[r] = *(const uint4 *)(wr[r] + c);
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) acc[r] = dot8(u[r], x + c, acc[r]);
+        }
+    };
+    sweep(st.wo, st.kpo, in, 512);
+    for (int j = 0; j < n_e; j++) sweep(m.down + (int64_t)st.ids[j] * m.down_stride, m.ffp, ie + j * m.ffp, 0);
+    if (m.sff) sweep(m.s_down, m.sffp, is, 0);
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) acc[r] = fh_wave_sum(acc[r]);
+    if (lane == 0)
+#pragma unroll
+        for (int r = 0; r < ROWS; r++)
+            if (row0 + r < st.width) st.x[row0 + r] += acc[r];
+}
+
+fh_status fh_step_out(fh_device *dev, const FhStep &st) {
+    const FhMoe &m = st.moe;
+    const size_t lds = (size_t)(st.kpo + (m.experts ? m.top * m.ffp : 0) + (m.sff ? m.sffp : 0) +
+                                (st.kind == FH_MIX_RECURRENT ? st.rec.norm_groups : 0)) * 4;
+    FH_REQUIRE(lds <= 156 * 1024, "a decode step stages at most 156 KB of inputs (%zu bytes needed)", lds);
+    const int rows = st.width >= dev->compute_units * 8 ? 2 : 1;
+    const void *fn = rows == 2 ? (const void *)k_step_out<2> : (const void *)k_step_out<1>;
+    if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, fn, lds));
+    const dim3 grid((unsigned)((st.width + 4 * rows - 1) / (4 * rows)));
+    if (rows == 2) k_step_out<2><<<grid, 256, lds, dev->stream>>>(st);
+    else k_step_out<1><<<grid, 256, lds, dev->stream>>>(st);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}

@@ -9,10 +9,11 @@ import numpy as np
 
 from . import _lib, synth
 from ._lib import F16, F32, LlamaConfig, check
+from .decoder import Decoder
 from .fusor import Device
 
 
-class Model:
+class Model(Decoder):
     def __init__(self, device: Device, cfg: dict, kv_dtype: str = "f32", fuse_qkv: bool = True,
                  fuse_gate_up: bool = True, use_graph: bool = True):
         self.device, self.cfg = device, dict(cfg)
@@ -23,6 +24,9 @@ class Model:
         check(device._lib.fh_llama_create(device._h, C.byref(c), C.byref(h)))
         self._h = h
         self._final = False
+        d = C.c_void_p()
+        check(device._lib.fh_llama_decoder(h, C.byref(d)))
+        super().__init__(device, d, owned=False)
 
     def load_tensor(self, name: str, ggml_type: int, n: int, k: int, data: np.ndarray) -> None:
         a = np.ascontiguousarray(data)
@@ -81,43 +85,6 @@ class Model:
         check(self.device._lib.fh_llama_finalize(self._h))
         self._final = True
 
-    def reset(self) -> None:
-        check(self.device._lib.fh_llama_reset(self._h))
-
-    def forward(self, tokens, want_hidden: bool = False):
-        """Model::forward: logits of the last of `tokens` (raw/mod.rs:851-865)."""
-        t = np.ascontiguousarray(tokens, dtype=np.uint32).reshape(-1)
-        logits = np.empty(self.cfg["vocab"], np.float32)
-        hidden = np.empty(self.cfg["d_model"], np.float32)
-        check(self.device._lib.fh_llama_forward(self._h, t.ctypes.data_as(C.c_void_p), t.size,
-                                                logits.ctypes.data_as(C.c_void_p), hidden.ctypes.data_as(C.c_void_p)))
-        return (logits, hidden) if want_hidden else logits
-
-    def decode_greedy(self, first_token: int, steps: int):
-        """Greedy decode of `steps` tokens on the device; returns (token ids, device milliseconds)."""
-        out = np.empty(steps, np.uint32)
-        ms = C.c_float()
-        check(self.device._lib.fh_llama_decode_greedy(self._h, int(first_token), steps, out.ctypes.data_as(C.c_void_p),
-                                                      C.byref(ms)))
-        return out, ms.value
-
-    def decode_sampled(self, first_token: int, steps: int, params, randoms, previous_tokens=(), repetition_range: int = 64,
-                       mu: Optional[float] = None):
-        """Sampled decode of `steps` tokens with the token resident on the device (models/kalosm-llama/src/model/
-        inference.rs:38-173).  `params`: GpuStandardSamplerParams or GpuMirostat2SamplerParams (its `random` is
-        replaced by `randoms[step]`).  Returns (token ids, device milliseconds, mu after the last step)."""
-        out = np.empty(steps, np.uint32)
-        rnd = np.ascontiguousarray(randoms, np.float32)
-        assert rnd.size >= steps
-        prev = np.ascontiguousarray(previous_tokens, np.uint32)
-        ms, mu_c = C.c_float(), C.c_float(0.0 if mu is None else mu)
-        cp = params.to_c()
-        check(self.device._lib.fh_llama_decode_sampled(
-            self._h, int(first_token), steps, C.byref(cp), rnd.ctypes.data_as(C.c_void_p),
-            prev.ctypes.data_as(C.c_void_p) if prev.size else None, int(prev.size), int(repetition_range),
-            C.byref(mu_c), out.ctypes.data_as(C.c_void_p), C.byref(ms)))
-        return out, ms.value, mu_c.value
-
     def trace_text(self) -> str:
         """Lines traced by the last `forward` (device options trace_nan / trace_timing, or the reference's
         KALOSM_TRACE_LAYER_NAN / KALOSM_TRACE_FORWARD_TIMING / FUSOR_TRACE_GPU_KERNELS in the environment)."""
@@ -126,11 +93,6 @@ class Model:
         buf = C.create_string_buffer(n.value + 1)
         check(self.device._lib.fh_llama_trace_text(self._h, buf, n.value + 1, None))
         return buf.value.decode()
-
-    def weight_bytes(self) -> int:
-        b = C.c_uint64()
-        check(self.device._lib.fh_llama_weight_bytes(self._h, C.byref(b)))
-        return b.value
 
     def __del__(self):
         try:

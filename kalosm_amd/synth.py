@@ -10,7 +10,7 @@ from __future__ import annotations
 import numpy as np
 
 Q4_0, Q8_0, Q4_K, Q6_K = 2, 8, 12, 14
-W_F32, W_F16, Q5_0, Q5_K = 0, 1, 6, 13  # kept in the file's layout by the library (per-element kernels)
+W_F32, W_F16, Q5_0, Q5_K, W_BF16 = 0, 1, 6, 13, 30  # kept in the file's layout by the library (per-element kernels)
 BLOCK_ELEMS = {Q4_0: 32, Q8_0: 32, Q4_K: 256, Q6_K: 256, W_F32: 1, W_F16: 1, Q5_0: 32, Q5_K: 256}
 BLOCK_BYTES = {Q4_0: 18, Q8_0: 34, Q4_K: 144, Q6_K: 210, W_F32: 4, W_F16: 2, Q5_0: 22, Q5_K: 176}
 TYPE_NAMES = {Q4_0: "Q4_0", Q8_0: "Q8_0", Q4_K: "Q4_K", Q6_K: "Q6_K", W_F32: "F32", W_F16: "F16", Q5_0: "Q5_0",
@@ -122,12 +122,81 @@ def llama_tensor_specs(cfg: dict):
     return specs
 
 
+def _name_seed(name: str, seed: int) -> int:
+    h = 1469598103934665603
+    for ch in name.encode():
+        h = (h ^ ch) * 1099511628211 % (1 << 64)
+    return (h ^ (seed * 0x9E3779B97F4A7C15)) % (1 << 63)
+
+
 def llama_random_tensor(name: str, ty: int, n: int, k: int, seed: int, sigma: float) -> np.ndarray:
     """Deterministic per-tensor content: the seed is mixed with a hash of the tensor name."""
-    h = np.uint64(1469598103934665603)
-    for ch in name.encode():
-        h = np.uint64((int(h) ^ ch) * 1099511628211 % (1 << 64))
-    s = (int(h) ^ (seed * 0x9E3779B97F4A7C15)) % (1 << 63)
+    s = _name_seed(name, seed)
     if ty == 0:
         return (1.0 + 0.1 * np.random.default_rng(s).standard_normal(n)).astype(np.float32)
     return random_weight(ty, n, k, s, sigma)
+
+
+# ---------------------------------------------------------------------------------------------
+# Layer-list decoders (kalosm_amd.hybrid): tensor names and shapes from a configuration, random bf16 weights.
+def hybrid_tensor_specs(cfg: dict):
+    """[(name, n, k)]; k is 0 for vectors."""
+    D, V = cfg["width"], cfg["vocab"]
+    specs = [("embed", V, D), ("final.norm", D, 0), ("head", V, D)]
+    for i, layer in enumerate(cfg["layers"]):
+        p, c = f"l{i}.", layer["mixer"]
+        specs.append((p + "norm1", D, 0))
+        m = p + "mix."
+        if layer["type"] == "latent_attention":
+            H, dn, dr, dv, R = c["heads"], c["dim"], c["rot_dim"], c["vdim"], c["kv_rank"]
+            inner = H * dv
+            specs += [(m + "q", H * (dn + dr), D), (m + "dkv", R + dr, D), (m + "dkv.norm", R, 0), (m + "uk", H * dn, R),
+                      (m + "uv", H * dv, R), (m + "sink", H, 0)]
+        elif layer["type"] == "delta":
+            H, nq, taps = c["heads"], c["kv_heads"] * c["dim"], c["conv"]
+            inner = H * c["vdim"]
+            specs += [(m + "q", nq, D), (m + "q.conv", nq, taps), (m + "k", nq, D), (m + "k.conv", nq, taps), (m + "v", inner, D),
+                      (m + "v.conv", inner, taps), (m + "b", H, D), (m + "A_log", H, 0), (m + "norm", c["vdim"], 0),
+                      (m + "a", H, D), (m + "dt_bias", H, 0), (m + "g", inner, D)]
+        else:
+            H, gn, taps = c["heads"], c["groups"] * c["state"], c["conv"]
+            inner = H * c["vdim"]
+            specs += [(m + "in", 2 * inner + 2 * gn + H, D), (m + "conv", inner + 2 * gn, taps), (m + "conv.b", inner + 2 * gn, 0),
+                      (m + "dt_bias", H, 0), (m + "A_log", H, 0), (m + "D", H, 0), (m + "norm", inner, 0)]
+        specs.append((m + "o", D, inner))
+        mlp = layer.get("mlp")
+        if mlp:
+            f = p + "mlp."
+            parts = [(f"e{e}", mlp["expert"]["ff"]) for e in range(mlp["router"]["experts"])]
+            if mlp.get("shared"):
+                parts.append(("shared", mlp["shared"]["ff"]))
+            for n, ff in parts:
+                specs += [(f + n + ".gate", ff, D), (f + n + ".up", ff, D), (f + n + ".down", D, ff)]
+            specs.append((f + "router", mlp["router"]["experts"], D))
+    return specs
+
+
+def hybrid_random_tensor(name: str, n: int, k: int, seed: int) -> np.ndarray:
+    """Deterministic bf16 bit patterns: rows of matrices with a norm near one, decays and step sizes spread over useful
+    ranges, norm weights away from their neutral value."""
+    rng = np.random.default_rng(_name_seed(name, seed))
+    last = name.rsplit(".", 1)[-1]
+    if last == "A_log":
+        x = rng.uniform(-3.0, 1.0, n)
+    elif last == "dt_bias":
+        x = rng.uniform(-3.0, 0.5, n)
+    elif last in ("norm1",) or name == "final.norm":
+        x = 0.2 * rng.standard_normal(n)
+    elif last in ("norm", "D"):
+        x = 1.0 + 0.2 * rng.standard_normal(n)
+    elif last in ("sink", "b") and k == 0:
+        x = 0.5 * rng.standard_normal(n)
+    elif last == "conv":
+        x = rng.standard_normal((n, k)) / np.sqrt(k)
+    elif name == "embed":
+        x = rng.standard_normal((n, k), np.float32)
+    else:
+        x = rng.standard_normal((n, k), np.float32) * np.float32(1.0 / np.sqrt(k))
+        if last == "router":
+            x = x * 2.0
+    return to_bf16_bits(np.asarray(x, np.float32).reshape(-1))
