@@ -221,6 +221,8 @@ extern "C" fh_status fh_set_option(fh_device *dev, const char *key, int64_t valu
     else if (!strcmp(key, "attn_heads")) dev->opt_attn_heads = value;
     else if (!strcmp(key, "down_tiles")) dev->opt_down_tiles = value;
     else if (!strcmp(key, "deterministic")) dev->opt_deterministic = value;
+    else if (!strcmp(key, "recurrent_kernel")) dev->opt_recurrent_kernel = value;
+    else if (!strcmp(key, "step_eager")) dev->opt_step_eager = value;
     else if (!strcmp(key, "trace_nan")) dev->opt_trace_nan = value;
     else if (!strcmp(key, "trace_timing")) dev->opt_trace_timing = value;
     else if (!strcmp(key, "trace_stderr")) dev->opt_trace_stderr = value;

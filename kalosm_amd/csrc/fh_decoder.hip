@@ -122,7 +122,7 @@ fh_status fh_decoder::decode_greedy(uint32_t first_token, int steps, uint32_t *o
     k_set_u32<<<1, 1, 0, s>>>((uint32_t *)step_dev, 0u);
     FH_HIP(hipGetLastError());
     int done = 0;
-    if (use_graph) {
+    if (use_graph && !dev->opt_step_eager) {
         // One eager step sizes every scratch buffer and sets kernel attributes; the capture then
         // records launches only.  The graph depends on the cache capacity (strides), so it is
         // rebuilt when the capacity changed since the last capture.
@@ -225,7 +225,7 @@ fh_status fh_decoder::decode_sampled(uint32_t first_token, int steps, const fh_s
     k_set_u32<<<1, 1, 0, s>>>((uint32_t *)step_dev, 0u);
     FH_HIP(hipGetLastError());
     int done = 0;
-    if (use_graph) {
+    if (use_graph && !dev->opt_step_eager) {
         // the captured step holds the sampler's parameters and the window size as kernel arguments
         fh_sampler_params want = *params;
         want.random = 0.f; // every step takes its number from randoms_host

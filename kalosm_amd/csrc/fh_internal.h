@@ -80,6 +80,8 @@ struct fh_device {
     int64_t opt_wo_acc = 0;          // 0: decode steps accumulate the output projection into the residual stream, 1: never
     int64_t opt_fuse_norm = 0;       // 0: decode steps fold rms_norm into the consuming matvec, 1: separate launches
     int64_t opt_deterministic = 0;   // 1: decode steps never accumulate k-split partial sums with float atomics (run-to-run bit-equal)
+    int64_t opt_recurrent_kernel = 0; // 0 auto, 1 token by token, 2 chunks of 64 tokens for every portion
+    int64_t opt_step_eager = 0;      // 1: decode loops launch their steps on the stream (kernel tracers), never a captured graph
     int64_t opt_trace_nan = 0;       // 1: fh_llama_forward probes the residual stream of every layer for NaN / inf
     int64_t opt_trace_timing = 0;    // 1: fh_llama_forward times its layer loop, 2: and every stage of every layer
     int64_t opt_trace_stderr = 0;    // 1: trace lines go to stderr as well as into the decoder's trace text

@@ -39,7 +39,7 @@ static inline int fh_latent_old(const FhLatent &a, int pos) { return a.window &&
 fh_status fh_latent_prefill(fh_device *dev, int dtype, const FhLatent &a, fh_kvcache *cache, const float *proj, int64_t ldp,
                             int s, int pos, const FhLatentWork &w, void *o, int kp);
 
-enum { FH_LATENT_MAX_SPLITS = 32 };
+enum { FH_LATENT_MAX_SPLITS = 64 };
 static inline size_t fh_latent_part_floats(const FhLatent &a) { return (size_t)a.heads * FH_LATENT_MAX_SPLITS * (a.r8 + 2); }
 // Decode step behind the absorbed queries qa [heads, fh_latent_row] (scaled to base-2 exponents): o [heads * dv]
 fh_status fh_latent_decode(fh_device *dev, int dtype, const FhLatent &a, const fh_kvcache *cache, const int *pos_dev,

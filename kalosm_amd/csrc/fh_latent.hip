@@ -434,58 +434,228 @@ __global__ __launch_bounds__(256) void k_latent_decode(FhLatent a, const T *__re
     }
 }
 
+// The same on the matrix cores, for bf16 caches: 16 heads are the rows of every product and a workgroup takes tiles of 64
+// keys.  Scores (16 heads x 64 keys) = qa . C^T, one key block of 16 per wavefront, qa as hi + lo; softmax through the
+// LDS, 16 lanes per head; sums (16 heads x rank) += P . C, P as hi + lo, a quarter of the rank per wavefront, the operand
+// of C with the keys along k by the transposing LDS load (ds_read_b64_tr_b16: a lane receives its column of four rows).
+typedef short fh_s4 __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ fh_bf8 lat_tr8(const uint16_t *p, int row_stride) { // rows k .. k + 3 and k + 16 .. k + 19
+    const fh_s4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) fh_s4 *)(uintptr_t)(uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void *)p);
+    const fh_s4 b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) fh_s4 *)(uintptr_t)(uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void *)(p + 16 * row_stride));
+    fh_bf8 r;
+    __builtin_memcpy(&r, &a, 8);
+    __builtin_memcpy((char *)&r + 8, &b, 8);
+    return r;
+}
+
+template <int NT> // 16-wide rank tiles of a wavefront: rank at most 64 NT
+__global__ __launch_bounds__(256) void k_latent_decode_mfma(FhLatent a, const uint16_t *__restrict__ ring, int cap,
+                                                            const int *__restrict__ pos_dev, const float *__restrict__ qa,
+                                                            float *__restrict__ part) {
+    extern __shared__ __attribute__((aligned(16))) char ld_lds[];
+    const int row = a.r8 + a.drp, steps = (row + 31) / 32, CS = steps * 32 + 8; // LDS row stride
+    uint16_t *sc = (uint16_t *)ld_lds, *sq = sc + 64 * CS, *sp = sq + 2 * 16 * CS; // cache tile, qa hi / lo, P hi / lo
+    constexpr int PS = 72, SS = 68;
+    float *s_s = (float *)(sp + 2 * 16 * PS), *s_r = s_s + 16 * SS; // scores, rescale factors
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, li = lane & 15, g = lane >> 4;
+    const int h0 = (int)blockIdx.y * 16, np = row / 8, npp = steps * 4;
+    const int n = *pos_dev + 1 < cap ? *pos_dev + 1 : cap;
+    const int per = ((n + (int)gridDim.x - 1) / (int)gridDim.x + 15) / 16 * 16;
+    const int k0 = (int)blockIdx.x * per, k1 = k0 + per < n ? k0 + per : n;
+    auto stage = [&](int k) { // pieces of eight elements; zeros behind the row and behind the last key
+        for (int i = tid; i < 64 * npp; i += 256) {
+            const int r = i / npp, c = i % npp;
+            uint4 v = uint4{0, 0, 0, 0};
+            if (k + r < k1 && c < np) v = *(const uint4 *)(ring + (int64_t)(k + r) * row + c * 8);
+            *(uint4 *)(sc + r * CS + c * 8) = v;
+        }
+    };
+    stage(k0);
+    for (int i = tid; i < 16 * npp; i += 256) {
+        const int r = i / npp, c = i % npp;
+        float v[8];
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] = 0.f;
+        if (h0 + r < a.heads && c < np) {
+            const float4 x = *(const float4 *)(qa + (int64_t)(h0 + r) * row + c * 8), y = *(const float4 *)(qa + (int64_t)(h0 + r) * row + c * 8 + 4);
+            v[0] = x.x, v[1] = x.y, v[2] = x.z, v[3] = x.w, v[4] = y.x, v[5] = y.y, v[6] = y.z, v[7] = y.w;
+        }
+        uint16_t hi[8], lo[8];
+#pragma unroll
+        for (int e = 0; e < 8; e++) hi[e] = fh_f32_bf(v[e]), lo[e] = fh_f32_bf(v[e] - fh_bf_f32(hi[e]));
+        __builtin_memcpy(sq + r * CS + c * 8, hi, 16);
+        __builtin_memcpy(sq + (16 + r) * CS + c * 8, lo, 16);
+    }
+    fh_f4 o[NT];
+#pragma unroll
+    for (int t = 0; t < NT; t++) o[t] = fh_f4{0.f, 0.f, 0.f, 0.f};
+    float mx = -INFINITY, den = 0.f; // of head tid / 16, the same in its 16 lanes
+    for (int k = k0; k < k1; k += 64) {
+        __syncthreads();
+        fh_f4 S = fh_f4{0.f, 0.f, 0.f, 0.f};
+        if (k + 16 * wave < k1)
+#pragma unroll 4
+            for (int x = 0; x < steps; x++) {
+                fh_bf8 c, h, l;
+                fh_frag_load(c, sc + (16 * wave + li) * CS + 32 * x + 8 * g);
+                fh_frag_load(h, sq + li * CS + 32 * x + 8 * g);
+                fh_frag_load(l, sq + (16 + li) * CS + 32 * x + 8 * g);
+                S = fh_mma32(h, c, S);
+                S = fh_mma32(l, c, S);
+            }
+#pragma unroll
+        for (int e = 0; e < 4; e++) s_s[(4 * g + e) * SS + 16 * wave + li] = k + 16 * wave + li < k1 ? S[e] : -INFINITY;
+        __syncthreads();
+        {
+            const int hr = tid >> 4, kq = (tid & 15) * 4; // head row and four keys
+            const float4 s4 = *(const float4 *)(s_s + hr * SS + kq);
+            float tm = fmaxf(fmaxf(s4.x, s4.y), fmaxf(s4.z, s4.w));
+#define FH_ROR(N_) tm = fmaxf(tm, __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(tm), 0x120 + N_, 0xF, 0xF, true)))
+            FH_ROR(8);
+            FH_ROR(4);
+            FH_ROR(2);
+            FH_ROR(1);
+#undef FH_ROR
+            const float mn = fmaxf(mx, tm), f = exp2f(mx - mn); // a tile has a live key, so mn is a number
+            const float p[4] = {exp2f(s4.x - mn), exp2f(s4.y - mn), exp2f(s4.z - mn), exp2f(s4.w - mn)};
+            den = den * f + fh_row16_sum((p[0] + p[1]) + (p[2] + p[3]));
+            mx = mn;
+            uint16_t hi[4], lo[4];
+#pragma unroll
+            for (int e = 0; e < 4; e++) hi[e] = fh_f32_bf(p[e]), lo[e] = fh_f32_bf(p[e] - fh_bf_f32(hi[e]));
+            __builtin_memcpy(sp + hr * PS + kq, hi, 8);
+            __builtin_memcpy(sp + (16 + hr) * PS + kq, lo, 8);
+            if ((tid & 15) == 0) s_r[hr] = f;
+        }
+        __syncthreads();
+        float f[4];
+#pragma unroll
+        for (int e = 0; e < 4; e++) f[e] = s_r[4 * g + e];
+#pragma unroll
+        for (int t = 0; t < NT; t++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) o[t][e] *= f[e];
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            if (k + 32 * u >= k1) break;
+            // k-slots of lane group g: keys 4 g .. + 3 and 16 + 4 g .. + 3, as the transposing load delivers them
+            fh_bf8 ph, pl;
+            __builtin_memcpy(&ph, sp + li * PS + 32 * u + 4 * g, 8);
+            __builtin_memcpy((char *)&ph + 8, sp + li * PS + 32 * u + 16 + 4 * g, 8);
+            __builtin_memcpy(&pl, sp + (16 + li) * PS + 32 * u + 4 * g, 8);
+            __builtin_memcpy((char *)&pl + 8, sp + (16 + li) * PS + 32 * u + 16 + 4 * g, 8);
+#pragma unroll
+            for (int t = 0; t < NT; t++) {
+                const int d = (wave * NT + t) * 16;
+                if (d < a.r8) { // columns behind the rank (the rotated key, zeros) are never stored
+                    const fh_bf8 c = lat_tr8(sc + (32 * u + 4 * g + (li >> 2)) * CS + d + (li & 3) * 4, CS);
+                    o[t] = fh_mma32(ph, c, o[t]);
+                    o[t] = fh_mma32(pl, c, o[t]);
+                }
+            }
+        }
+        __syncthreads();
+        if (k + 64 < k1) stage(k + 64);
+    }
+    const int st = a.r8 + 2;
+#pragma unroll
+    for (int t = 0; t < NT; t++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int h = h0 + 4 * g + e, d = (wave * NT + t) * 16 + li;
+            if (h < a.heads && d < a.r8) part[((int64_t)h * gridDim.x + blockIdx.x) * st + d] = o[t][e];
+        }
+    if ((tid & 15) == 0 && h0 + (tid >> 4) < a.heads) {
+        float *p = part + ((int64_t)(h0 + (tid >> 4)) * gridDim.x + blockIdx.x) * st + a.r8;
+        p[0] = mx, p[1] = den;
+    }
+}
+
 // Merge of the splits (with the sink) and the value projection: grid (heads, blocks of 32 values).
 __global__ __launch_bounds__(256) void k_latent_values(FhLatent a, const float *__restrict__ part, int splits, float *__restrict__ o) {
     extern __shared__ __attribute__((aligned(16))) float oc[]; // [rp]
+    __shared__ float fw[FH_LATENT_MAX_SPLITS];
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.x, st = a.r8 + 2;
     const float *p = part + (int64_t)h * splits * st;
-    const float z = a.sink ? a.sink[h] * FH_LOG2E : -INFINITY;
-    float mm = z, l = 0.f;
-    for (int i = 0; i < splits; i++) mm = fmaxf(mm, p[i * st + a.r8]);
-    for (int i = 0; i < splits; i++) {
-        const float m = p[i * st + a.r8];
-        l += m == -INFINITY ? 0.f : exp2f(m - mm) * p[i * st + a.r8 + 1];
+    uint4 w[8]; // the first 512 of k of this wavefront's rows, requested before the merge
+    const int r0 = (int)blockIdx.y * 32 + wave * 8;
+#pragma unroll
+    for (int i = 0; i < 8; i++) {
+        const int r = r0 + i < a.dv ? r0 + i : a.dv - 1;
+        w[i] = lane * 8 < a.rp ? *(const uint4 *)(a.uv + (int64_t)(h * a.dv + r) * a.rp + lane * 8) : uint4{0, 0, 0, 0};
     }
-    if (a.sink) l += exp2f(z - mm);
-    const float inv = 1.0f / l;
+    if (wave == 0) {
+        static_assert(FH_LATENT_MAX_SPLITS <= 64, "one split per lane");
+        const float z = a.sink ? a.sink[h] * FH_LOG2E : -INFINITY;
+        const float m = lane < splits ? p[lane * st + a.r8] : -INFINITY, l = lane < splits ? p[lane * st + a.r8 + 1] : 0.f;
+        float mm = fmaxf(m, z);
+#pragma unroll
+        for (int i = 32; i > 0; i >>= 1) mm = fmaxf(mm, __shfl_xor(mm, i, 64));
+        const float f = m == -INFINITY ? 0.f : exp2f(m - mm);
+        float d = fh_wave_sum(f * l);
+        if (a.sink) d += exp2f(z - mm);
+        if (lane < splits) fw[lane] = f / d;
+    }
+    __syncthreads();
     for (int x = tid; x < a.rp; x += 256) {
         float v = 0.f;
         if (x < a.r8)
-            for (int i = 0; i < splits; i++) {
-                const float m = p[i * st + a.r8];
-                if (m != -INFINITY) v = fmaf(exp2f(m - mm), p[i * st + x], v);
-            }
-        oc[x] = v * inv;
+#pragma unroll 8
+            for (int i = 0; i < splits; i++) v = fmaf(fw[i], fw[i] != 0.f ? p[i * st + x] : 0.f, v);
+        oc[x] = v;
     }
     __syncthreads();
-    for (int i = 0; i < 8; i++) {
-        const int r = (int)blockIdx.y * 32 + wave * 8 + i;
-        if (r >= a.dv) break;
-        const uint16_t *w = a.uv + (int64_t)(h * a.dv + r) * a.rp;
-        float acc = 0.f;
-        for (int c = lane * 8; c < a.rp; c += 512) {
-            const uint4 u = *(const uint4 *)(w + c);
-            const float4 x = *(const float4 *)(oc + c), y = *(const float4 *)(oc + c + 4);
-            acc = fmaf(fh_bf_lo(u.x), x.x, acc);
-            acc = fmaf(fh_bf_hi(u.x), x.y, acc);
-            acc = fmaf(fh_bf_lo(u.y), x.z, acc);
-            acc = fmaf(fh_bf_hi(u.y), x.w, acc);
-            acc = fmaf(fh_bf_lo(u.z), y.x, acc);
-            acc = fmaf(fh_bf_hi(u.z), y.y, acc);
-            acc = fmaf(fh_bf_lo(u.w), y.z, acc);
-            acc = fmaf(fh_bf_hi(u.w), y.w, acc);
+    float acc[8];
+#pragma unroll
+    for (int i = 0; i < 8; i++) acc[i] = 0.f;
+    for (int c = lane * 8; c < a.rp; c += 512) {
+        const float4 x = *(const float4 *)(oc + c), y = *(const float4 *)(oc + c + 4);
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            const int r = r0 + i < a.dv ? r0 + i : a.dv - 1;
+            const uint4 u = c < 512 ? w[i] : *(const uint4 *)(a.uv + (int64_t)(h * a.dv + r) * a.rp + c);
+            acc[i] = fmaf(fh_bf_lo(u.x), x.x, acc[i]);
+            acc[i] = fmaf(fh_bf_hi(u.x), x.y, acc[i]);
+            acc[i] = fmaf(fh_bf_lo(u.y), x.z, acc[i]);
+            acc[i] = fmaf(fh_bf_hi(u.y), x.w, acc[i]);
+            acc[i] = fmaf(fh_bf_lo(u.z), y.x, acc[i]);
+            acc[i] = fmaf(fh_bf_hi(u.z), y.y, acc[i]);
+            acc[i] = fmaf(fh_bf_lo(u.w), y.z, acc[i]);
+            acc[i] = fmaf(fh_bf_hi(u.w), y.w, acc[i]);
         }
-        acc = fh_wave_sum(acc);
-        if (lane == 0) o[h * a.dv + r] = acc;
     }
+#pragma unroll
+    for (int i = 0; i < 8; i++) acc[i] = fh_wave_sum(acc[i]);
+    if (lane == 0)
+#pragma unroll
+        for (int i = 0; i < 8; i++)
+            if (r0 + i < a.dv) o[h * a.dv + r0 + i] = acc[i];
 }
 
 template <typename T>
 static fh_status latent_decode_t(fh_device *dev, const FhLatent &a, const fh_kvcache *cache, const int *pos_dev, const float *qa,
                                  float *part, float *o) {
     const int row = fh_latent_row(a), hb = a.heads % 2 == 0 ? 2 : 1;
-    int splits = cache->capacity / 64;
+    int splits = cache->capacity / 32;
     splits = splits < 1 ? 1 : splits > FH_LATENT_MAX_SPLITS ? FH_LATENT_MAX_SPLITS : splits;
+    const int cs = (row + 31) / 32 * 32 + 8;
+    const size_t mlds = (size_t)(96 * cs + 32 * 72) * 2 + (16 * 68 + 16) * 4;
+    if (sizeof(T) == 2 && a.r8 <= 640 && mlds <= 156 * 1024 && dev->opt_attn_kernel != 1) {
+        const dim3 mgrid((unsigned)splits, (unsigned)((a.heads + 15) / 16));
+        const uint16_t *mring = (const uint16_t *)cache->k;
+#define FH_GO(NT_)                                                                                                  \
+    do {                                                                                                            \
+        if (mlds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)k_latent_decode_mfma<NT_>, mlds));            \
+        k_latent_decode_mfma<NT_><<<mgrid, 256, mlds, dev->stream>>>(a, mring, cache->capacity, pos_dev, qa, part); \
+    } while (0)
+        if (a.r8 <= 128) FH_GO(2);
+        else if (a.r8 <= 512) FH_GO(8);
+        else FH_GO(10);
+#undef FH_GO
+        k_latent_values<<<dim3((unsigned)a.heads, (unsigned)((a.dv + 31) / 32)), 256, (size_t)a.rp * 4, dev->stream>>>(a, part, splits, o);
+        FH_HIP(hipGetLastError());
+        return FH_OK;
+    }
     const dim3 grid((unsigned)splits, (unsigned)(a.heads / hb));
     const size_t lds = (size_t)4 * hb * (a.r8 + 2) * 4;
     const T *ring = (const T *)cache->k;

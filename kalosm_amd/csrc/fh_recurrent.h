@@ -21,6 +21,8 @@ struct FhRecurrent {
     float eps = 0.f, q_scale = 1.f;
 };
 static inline int fh_rec_channels(const FhRecurrent &r) { return 2 * r.kv_heads * r.dim + r.heads * r.vdim; }
+// rows of q and k in the work arrays of a portion: dim rounded up to a size the chunked form has, zeros in the padding
+static inline int fh_rec_dp(const FhRecurrent &r) { return r.dim <= 32 ? 32 : r.dim <= 64 ? 64 : r.dim <= 128 ? 128 : 256; }
 static inline int fh_rec_inner(const FhRecurrent &r) { return r.heads * r.vdim; }
 
 // State of one recurrent layer of one sequence.
@@ -31,11 +33,11 @@ struct FhRecState {
 
 // Work arrays of a prefill portion, rows of one token each.
 struct FhRecWork {
-    float *q, *k;     // [t, kv_heads * dim]
+    float *q, *k;     // [t, kv_heads * fh_rec_dp]
     float *v;         // [t, heads * vdim]
     float *beta, *la; // [t, heads]
     float *o;         // [t, heads * vdim]
-    float *chunk;     // scratch of the chunked form (fh_rec_chunk_floats), NULL: token by token only
+    float *chunk;     // scratch of the chunked form (fh_rec_chunk_floats)
 };
 size_t fh_rec_chunk_floats(const FhRecurrent &r, int s);
 // One portion of s tokens at position pos: proj rows [s, ldp] -> normed, gated activation rows y [s, kp].

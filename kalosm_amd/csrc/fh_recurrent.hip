@@ -1,11 +1,11 @@
-// Prefill of the gated linear recurrences (fh_recurrent.h): convolutions and gates of a portion, the recurrence token by
-// token, and the gated norm of its output.
+// Prefill of the gated linear recurrences (fh_recurrent.h): convolutions and gates of a portion, the recurrence in chunks
+// (matrix cores) or token by token, and the gated norm of its output.
 #include "fh_recurrent.h"
 
 // ------------------------------------------------------------------------------ inputs of the recurrence
 // One workgroup per token.
 __global__ __launch_bounds__(256) void k_rec_prep(FhRecurrent r, const float *__restrict__ proj, int64_t ldp, int pos,
-                                                  const float *__restrict__ ring, FhRecWork w) {
+                                                  const float *__restrict__ ring, FhRecWork w, int dp) {
     extern __shared__ float qk[]; // [2 * kv_heads * dim]
     const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
     const int nq = r.kv_heads * r.dim, inner = r.heads * r.vdim, channels = 2 * nq + inner;
@@ -30,8 +30,8 @@ __global__ __launch_bounds__(256) void k_rec_prep(FhRecurrent r, const float *__
             f = 1.0f / sqrtf(fh_wave_sum(ss) + 1e-6f);
         }
         if (h < r.kv_heads) f *= r.q_scale;
-        float *dst = (h < r.kv_heads ? w.q : w.k) + (int64_t)t * nq + (h % r.kv_heads) * r.dim;
-        for (int i = lane; i < r.dim; i += 64) dst[i] = x[i] * f;
+        float *dst = (h < r.kv_heads ? w.q : w.k) + ((int64_t)t * r.kv_heads + h % r.kv_heads) * dp;
+        for (int i = lane; i < dp; i += 64) dst[i] = i < r.dim ? x[i] * f : 0.f;
     }
 }
 
@@ -48,22 +48,22 @@ __global__ void k_rec_tail(FhRecurrent r, const float *__restrict__ proj, int64_
 // One wavefront per four columns of a head's state; the 16 lanes of a DPP row share a column, RPT consecutive rows each,
 // in registers for the whole portion.  The next token's operands are requested before the current one is worked on.
 template <int RPT>
-__global__ __launch_bounds__(64) void k_rec_scan(FhRecurrent r, FhRecWork w, float *__restrict__ state, int s, int first) {
+__global__ __launch_bounds__(64) void k_rec_scan(FhRecurrent r, FhRecWork w, float *__restrict__ state, int s, int first, int dp) {
     const int h = blockIdx.y, lane = threadIdx.x, rg = lane & 15, col = (int)blockIdx.x * 4 + (lane >> 4);
-    const int nq = r.kv_heads * r.dim, inner = r.heads * r.vdim, kh = h / (r.heads / r.kv_heads), i0 = rg * RPT;
+    const int nq = r.kv_heads * dp, inner = r.heads * r.vdim, kh = h / (r.heads / r.kv_heads), i0 = rg * RPT;
     const bool live = col < r.vdim;
     const int c = live ? col : r.vdim - 1;
     float *sp = state + ((int64_t)h * r.vdim + c) * r.dim;
     float S[RPT], kc[RPT], qc[RPT], kn[RPT], qn[RPT];
 #pragma unroll
     for (int i = 0; i < RPT; i++) S[i] = !first && i0 + i < r.dim ? sp[i0 + i] : 0.f;
-    const float *kp = w.k + kh * r.dim + i0, *qp = w.q + kh * r.dim + i0, *vp = w.v + h * r.vdim + c;
+    const float *kp = w.k + kh * dp + i0, *qp = w.q + kh * dp + i0, *vp = w.v + h * r.vdim + c;
     const float skip = r.d_skip ? r.d_skip[h] : 0.f;
     auto load = [&](int t, float *k, float *q, float &v, float &be, float &la) {
 #pragma unroll
         for (int i = 0; i < RPT; i++) {
-            k[i] = i0 + i < r.dim ? kp[(int64_t)t * nq + i] : 0.f;
-            q[i] = i0 + i < r.dim ? qp[(int64_t)t * nq + i] : 0.f;
+            k[i] = i0 + i < dp ? kp[(int64_t)t * nq + i] : 0.f;
+            q[i] = i0 + i < dp ? qp[(int64_t)t * nq + i] : 0.f;
         }
         v = vp[(int64_t)t * inner];
         be = w.beta[(int64_t)t * r.heads + h];
@@ -127,7 +127,274 @@ __global__ __launch_bounds__(256) void k_rec_out(FhRecurrent r, const float *__r
     for (int i = inner + tid; i < kp; i += 256) yr[i] = fh_to<T>(0.f);
 }
 
-size_t fh_rec_chunk_floats(const FhRecurrent &, int) { return 0; }
+// ------------------------------------------------------------------------------ in chunks of 64 tokens
+// With c_t the running sum of la inside a chunk and S the state before it:
+//   O = e^c Q S + M U,   M_ts = e^(c_t - c_s) q_t . k_s  (s <= t),   S <- e^c_63 S + sum_s e^(c_63 - c_s) k_s u_s^T
+//   state space: u_t = beta_t v_t
+//   delta rule:  (1 + L) U = beta V - beta e^c K S,   L_ts = beta_t e^(c_t - c_s) k_t . k_s  (s < t)
+// The first launch works on all chunks at once: M, K^T, and for the delta rule U0 = (1 + L)^-1 beta V and
+// W = (1 + L)^-1 beta e^c K by forward substitution, one column of [W | U0] per thread with the 64 rows in registers.
+// The second walks the chunks with 16 columns of a head's state per workgroup: U = U0 - W S.  All products are
+// v_mfma_f32_16x16x4_f32; a lane takes four neighbouring k of an operand row at a time, on both sides alike.
+struct RecChunks { // scratch of one portion
+    float *m, *w, *u0; // per (chunk, head): [64][64], [64][dp], [64][vp]
+    float *kt;         // per (chunk, key head): [dp][64]
+    int dp, vp, n;     // vp: vdim rounded up to 16, n: chunks
+};
+static RecChunks rec_chunks(const FhRecurrent &r, int s, float *p) {
+    RecChunks c{};
+    c.dp = fh_rec_dp(r), c.vp = (r.vdim + 15) / 16 * 16, c.n = (s + 63) / 64;
+    const size_t hc = (size_t)c.n * r.heads;
+    c.m = p, p += hc * 4096;
+    c.kt = p, p += (size_t)c.n * r.kv_heads * c.dp * 64;
+    if (r.delta) c.w = p, p += hc * 64 * c.dp, c.u0 = p;
+    return c;
+}
+size_t fh_rec_chunk_floats(const FhRecurrent &r, int s) {
+    const RecChunks c = rec_chunks(r, s, nullptr);
+    return (size_t)c.n * ((size_t)r.heads * (4096 + (r.delta ? 64 * (c.dp + c.vp) : 0)) + (size_t)r.kv_heads * c.dp * 64);
+}
+
+__device__ __forceinline__ fh_f4 mma4(const float4 &a, const float4 &b, fh_f4 c) { // 16 of k
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, c, 0, 0, 0);
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, c, 0, 0, 0);
+    c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, c, 0, 0, 0);
+    return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, c, 0, 0, 0);
+}
+// Running sum of la over the 64 tokens of a chunk (one wavefront; tokens past the end change nothing).
+__device__ __forceinline__ float rec_decay_sum(const FhRecWork &w, int t, int s, int heads, int h) {
+    float v = t < s ? w.la[(int64_t)t * heads + h] : 0.f;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+        const float u = __shfl_up(v, o, 64);
+        if ((int)(threadIdx.x & 63) >= o) v += u;
+    }
+    return v;
+}
+
+template <int DP, bool DELTA>
+__global__ __launch_bounds__(256) void k_rec_chunk_prep(FhRecurrent r, FhRecWork w, RecChunks c, int s) {
+    constexpr int LD = DP + 4, LL = 68;
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    float *sk = lds, *sq = sk + 64 * LD, *cs = sq + 64 * (LD > LL ? LD : LL), *be = cs + 64; // L takes the place of Q
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, li = lane & 15, g = lane >> 4;
+    const int ch = blockIdx.x, h = blockIdx.y, rep = r.heads / r.kv_heads, kh = h / rep, t0 = ch * 64;
+    for (int i = tid; i < 64 * DP / 4; i += 256) {
+        const int t = i / (DP / 4), x = i % (DP / 4) * 4;
+        const int64_t o = ((int64_t)(t0 + t) * r.kv_heads + kh) * DP + x;
+        const float4 z = make_float4(0.f, 0.f, 0.f, 0.f);
+        *(float4 *)(sk + t * LD + x) = t0 + t < s ? *(const float4 *)(w.k + o) : z;
+        *(float4 *)(sq + t * LD + x) = t0 + t < s ? *(const float4 *)(w.q + o) : z;
+    }
+    if (wave == 0) {
+        cs[lane] = rec_decay_sum(w, t0 + lane, s, r.heads, h);
+        be[lane] = t0 + lane < s ? w.beta[(int64_t)(t0 + lane) * r.heads + h] : 0.f;
+    }
+    __syncthreads();
+    const int64_t hc = (int64_t)ch * r.heads + h;
+    float *mo = c.m + hc * 4096;
+    fh_f4 kk[4];
+#pragma unroll
+    for (int b = 0; b < 4; b++) { // wavefront: rows 16 wave .. + 15 against the 16 tokens of block b <= wave
+        if (b > wave) break;
+        fh_f4 qk = fh_f4{0.f, 0.f, 0.f, 0.f};
+        kk[b] = qk;
+#pragma unroll
+        for (int x = 0; x < DP / 16; x++) {
+            const float4 kb = *(const float4 *)(sk + (16 * b + li) * LD + 16 * x + 4 * g);
+            qk = mma4(*(const float4 *)(sq + (16 * wave + li) * LD + 16 * x + 4 * g), kb, qk);
+            if (DELTA) kk[b] = mma4(*(const float4 *)(sk + (16 * wave + li) * LD + 16 * x + 4 * g), kb, kk[b]);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int t = 16 * wave + 4 * g + e, u = 16 * b + li;
+            mo[t * 64 + u] = u <= t ? expf(cs[t] - cs[u]) * qk[e] : 0.f;
+        }
+    }
+    if (h % rep == 0) {
+        float *kt = c.kt + ((int64_t)ch * r.kv_heads + kh) * DP * 64;
+        for (int i = tid; i < DP * 64; i += 256) kt[i] = sk[(i & 63) * LD + (i >> 6)];
+    }
+    if (!DELTA) return;
+    __syncthreads(); // Q has been read
+    float *sl = sq;
+#pragma unroll
+    for (int b = 0; b < 4; b++) {
+        if (b > wave) break;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int t = 16 * wave + 4 * g + e, u = 16 * b + li;
+            sl[t * LL + u] = u < t ? be[t] * expf(cs[t] - cs[u]) * kk[b][e] : 0.f;
+        }
+    }
+    __syncthreads();
+    for (int j = tid; j < DP + c.vp; j += 256) {
+        float x[64];
+        if (j < DP) {
+#pragma unroll
+            for (int t = 0; t < 64; t++) x[t] = be[t] * expf(cs[t]) * sk[t * LD + j];
+        } else {
+            const int col = j - DP;
+#pragma unroll
+            for (int t = 0; t < 64; t++)
+                x[t] = t0 + t < s && col < r.vdim ? be[t] * w.v[((int64_t)(t0 + t) * r.heads + h) * r.vdim + col] : 0.f;
+        }
+#pragma unroll
+        for (int t = 1; t < 64; t++) {
+            float a = x[t];
+#pragma unroll
+            for (int u = 0; u < (t + 3) / 4; u++) {
+                const float4 l = *(const float4 *)(sl + t * LL + 4 * u); // zeros from u = t on inside the diagonal block
+                a = fmaf(-l.x, x[4 * u], a);
+                if (4 * u + 1 < t) a = fmaf(-l.y, x[4 * u + 1], a);
+                if (4 * u + 2 < t) a = fmaf(-l.z, x[4 * u + 2], a);
+                if (4 * u + 3 < t) a = fmaf(-l.w, x[4 * u + 3], a);
+            }
+            x[t] = a;
+        }
+        float *dst = j < DP ? c.w + hc * 64 * DP + j : c.u0 + hc * 64 * c.vp + j - DP;
+        const int st = j < DP ? DP : c.vp;
+#pragma unroll
+        for (int t = 0; t < 64; t++) dst[t * st] = x[t];
+    }
+}
+
+// grid (blocks of 16 value columns, heads), four wavefronts.  Wavefront w works out rows 16 w .. + 15 of U and O and rows
+// DP / 4 w .. of the state; U and the state pass between the wavefronts through the LDS, one column per row.
+template <int DP, bool DELTA>
+__global__ __launch_bounds__(256, 1) void k_rec_chunk_scan(FhRecurrent r, FhRecWork w, RecChunks c, float *__restrict__ state, int s,
+                                                           int first) {
+    constexpr int ST = DP / 64 > 0 ? DP / 64 : 1, SL = DP + 4, UL = 68; // state tiles of a wavefront
+    constexpr int SW = DP / 16 / ST;                                    // wavefronts with state rows
+    __shared__ __attribute__((aligned(16))) float ss[16 * SL], su[16 * UL], sd[16 * UL], cs[2][64];
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, li = lane & 15, g = lane >> 4;
+    const int h = blockIdx.y, kh = h / (r.heads / r.kv_heads), col0 = (int)blockIdx.x * 16, col = col0 + li;
+    const bool live = col < r.vdim, owner = wave < SW;
+    float *sp = state + ((int64_t)h * r.vdim + (live ? col : r.vdim - 1)) * r.dim;
+    fh_f4 S[ST];
+#pragma unroll
+    for (int i = 0; i < ST; i++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int row = (wave * ST + i) * 16 + 4 * g + e;
+            S[i][e] = !first && live && owner && row < r.dim ? sp[row] : 0.f;
+        }
+    const float skip = r.d_skip ? r.d_skip[h] : 0.f;
+    struct Ops { // a lane's operands of one chunk
+        float4 w[DELTA ? DP / 16 : 1], q[DP / 16], m[4], kt[ST][4];
+        float u[4], v[4], la;
+    } o0, o1;
+    auto load = [&](Ops &o, int ch) {
+        const int64_t hc = (int64_t)ch * r.heads + h;
+        const int t = ch * 64 + 16 * wave + li, tq = t < s ? t : s - 1; // rows past the end are multiplied by zeros of M and decays
+        if (DELTA) {
+            const float *wp = c.w + (hc * 64 + 16 * wave + li) * DP + 4 * g;
+#pragma unroll
+            for (int x = 0; x < DP / 16; x++) o.w[x] = *(const float4 *)(wp + 16 * x);
+        }
+        const float *qp = w.q + ((int64_t)tq * r.kv_heads + kh) * DP + 4 * g;
+#pragma unroll
+        for (int x = 0; x < DP / 16; x++) o.q[x] = *(const float4 *)(qp + 16 * x);
+        const float *mp = c.m + hc * 4096 + (16 * wave + li) * 64 + 4 * g;
+#pragma unroll
+        for (int b = 0; b < 4; b++)
+            if (b <= wave) o.m[b] = *(const float4 *)(mp + 16 * b);
+        if (owner) {
+            const float *kp = c.kt + (((int64_t)ch * r.kv_heads + kh) * DP + wave * ST * 16 + li) * 64 + 4 * g;
+#pragma unroll
+            for (int i = 0; i < ST; i++)
+#pragma unroll
+                for (int b = 0; b < 4; b++) o.kt[i][b] = *(const float4 *)(kp + i * 1024 + 16 * b);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int row = 16 * wave + 4 * g + e, tt = ch * 64 + row;
+            const bool in = tt < s && live;
+            o.v[e] = in && (!DELTA || r.d_skip) ? w.v[((int64_t)tt * r.heads + h) * r.vdim + col] : 0.f;
+            o.u[e] = DELTA ? c.u0[(hc * 64 + row) * c.vp + col] : in ? o.v[e] * w.beta[(int64_t)tt * r.heads + h] : 0.f;
+        }
+        o.la = ch * 64 + lane < s ? w.la[(int64_t)(ch * 64 + lane) * r.heads + h] : 0.f;
+    };
+    auto step = [&](const Ops &o, int ch) {
+        float *c_ = cs[ch & 1];
+        if (wave == 0) {
+            float v = o.la;
+#pragma unroll
+            for (int d = 1; d < 64; d <<= 1) {
+                const float u = __shfl_up(v, d, 64);
+                if (lane >= d) v += u;
+            }
+            c_[lane] = v;
+        }
+        if (owner)
+#pragma unroll
+            for (int i = 0; i < ST; i++) *(fh_f4 *)(ss + li * SL + (wave * ST + i) * 16 + 4 * g) = S[i];
+        __syncthreads(); // state and decays are there; U of the chunk before has been read
+        fh_f4 ws = fh_f4{0.f, 0.f, 0.f, 0.f}, qs = ws;
+#pragma unroll
+        for (int x = 0; x < DP / 16; x++) {
+            const float4 b = *(const float4 *)(ss + li * SL + 16 * x + 4 * g);
+            if (DELTA) ws = mma4(o.w[x], b, ws);
+            qs = mma4(o.q[x], b, qs);
+        }
+        const float end = c_[63];
+        fh_f4 u, ud, out;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const float ct = c_[16 * wave + 4 * g + e];
+            u[e] = o.u[e] - ws[e];
+            ud[e] = expf(end - ct) * u[e];
+            out[e] = expf(ct) * qs[e];
+        }
+        *(fh_f4 *)(su + li * UL + 16 * wave + 4 * g) = u;
+        *(fh_f4 *)(sd + li * UL + 16 * wave + 4 * g) = ud;
+        __syncthreads();
+#pragma unroll
+        for (int b = 0; b < 4; b++)
+            if (b <= wave) out = mma4(o.m[b], *(const float4 *)(su + li * UL + 16 * b + 4 * g), out);
+        const float f = expf(end);
+        if (owner)
+#pragma unroll
+            for (int i = 0; i < ST; i++) {
+#pragma unroll
+                for (int e = 0; e < 4; e++) S[i][e] *= f;
+#pragma unroll
+                for (int b = 0; b < 4; b++) S[i] = mma4(o.kt[i][b], *(const float4 *)(sd + li * UL + 16 * b + 4 * g), S[i]);
+            }
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int tt = ch * 64 + 16 * wave + 4 * g + e;
+            if (tt < s && live) w.o[((int64_t)tt * r.heads + h) * r.vdim + col] = out[e] + skip * o.v[e];
+        }
+    };
+    load(o0, 0);
+    for (int ch = 0; ch < c.n; ch += 2) { // the next chunk's operands are requested before the current one is worked on
+        if (ch + 1 < c.n) load(o1, ch + 1);
+        step(o0, ch);
+        if (ch + 1 >= c.n) break;
+        if (ch + 2 < c.n) load(o0, ch + 2);
+        step(o1, ch + 1);
+    }
+#pragma unroll
+    for (int i = 0; i < ST; i++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int row = (wave * ST + i) * 16 + 4 * g + e;
+            if (live && owner && row < r.dim) sp[row] = S[i][e];
+        }
+}
+
+template <int DP, bool DELTA>
+static fh_status rec_chunked(fh_device *dev, const FhRecurrent &r, const FhRecWork &w, float *state, int s, bool first) {
+    const RecChunks c = rec_chunks(r, s, w.chunk);
+    const size_t lds = (size_t)(64 * (DP + 4) + 64 * (DP + 4 > 68 ? DP + 4 : 68) + 128) * 4;
+    auto prep = k_rec_chunk_prep<DP, DELTA>;
+    if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)prep, lds));
+    prep<<<dim3((unsigned)c.n, (unsigned)r.heads), 256, lds, dev->stream>>>(r, w, c, s);
+    k_rec_chunk_scan<DP, DELTA><<<dim3((unsigned)(c.vp / 16), (unsigned)r.heads), 256, 0, dev->stream>>>(r, w, c, state, s, first);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
 
 fh_status fh_recurrent_prefill(fh_device *dev, int dtype, const FhRecurrent &r, const FhRecState &st, const float *proj,
                                int64_t ldp, int s, int pos, const FhRecWork &w, void *y, int kp) {
@@ -136,15 +403,25 @@ fh_status fh_recurrent_prefill(fh_device *dev, int dtype, const FhRecurrent &r, 
     const size_t lds1 = (size_t)2 * nq * 4, lds2 = (size_t)inner * 4;
     FH_REQUIRE(lds1 <= 150 * 1024 && lds2 <= 150 * 1024, "recurrent layer of %d channels is too wide", channels);
     if (lds1 > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)k_rec_prep, lds1));
-    k_rec_prep<<<dim3((unsigned)s), 256, lds1, str>>>(r, proj, ldp, pos, st.conv, w);
+    const int dp = fh_rec_dp(r);
+    k_rec_prep<<<dim3((unsigned)s), 256, lds1, str>>>(r, proj, ldp, pos, st.conv, w, dp);
     const int ty = s < r.taps ? s : r.taps;
     k_rec_tail<<<dim3((unsigned)((channels + 255) / 256), (unsigned)ty), 256, 0, str>>>(r, proj, ldp, s, pos, st.conv);
     const dim3 sg((unsigned)((r.vdim + 3) / 4), (unsigned)r.heads);
     const int rpt = (r.dim + 15) / 16;
-    if (rpt <= 2) k_rec_scan<2><<<sg, 64, 0, str>>>(r, w, st.s, s, pos == 0);
-    else if (rpt <= 4) k_rec_scan<4><<<sg, 64, 0, str>>>(r, w, st.s, s, pos == 0);
-    else if (rpt <= 8) k_rec_scan<8><<<sg, 64, 0, str>>>(r, w, st.s, s, pos == 0);
-    else if (rpt <= 16) k_rec_scan<16><<<sg, 64, 0, str>>>(r, w, st.s, s, pos == 0);
+    const int64_t kernel = dev->opt_recurrent_kernel;
+    if (kernel == 2 || (kernel == 0 && s >= 24)) {
+        const bool f = pos == 0;
+        switch (dp) {
+        case 32: FH_TRY(r.delta ? (rec_chunked<32, true>(dev, r, w, st.s, s, f)) : (rec_chunked<32, false>(dev, r, w, st.s, s, f))); break;
+        case 64: FH_TRY(r.delta ? (rec_chunked<64, true>(dev, r, w, st.s, s, f)) : (rec_chunked<64, false>(dev, r, w, st.s, s, f))); break;
+        case 128: FH_TRY(r.delta ? (rec_chunked<128, true>(dev, r, w, st.s, s, f)) : (rec_chunked<128, false>(dev, r, w, st.s, s, f))); break;
+        default: FH_TRY(r.delta ? (rec_chunked<256, true>(dev, r, w, st.s, s, f)) : (rec_chunked<256, false>(dev, r, w, st.s, s, f))); break;
+        }
+    } else if (rpt <= 2) k_rec_scan<2><<<sg, 64, 0, str>>>(r, w, st.s, s, pos == 0, dp);
+    else if (rpt <= 4) k_rec_scan<4><<<sg, 64, 0, str>>>(r, w, st.s, s, pos == 0, dp);
+    else if (rpt <= 8) k_rec_scan<8><<<sg, 64, 0, str>>>(r, w, st.s, s, pos == 0, dp);
+    else if (rpt <= 16) k_rec_scan<16><<<sg, 64, 0, str>>>(r, w, st.s, s, pos == 0, dp);
     else FH_FAIL(FH_ERR_UNSUPPORTED, "recurrent state of %d rows (at most 256)", r.dim);
     if (dtype == FH_F32) {
         if (lds2 > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)k_rec_out<float>, lds2));

@@ -231,99 +231,101 @@ fh_status fh_step_middle(fh_device *dev, int dtype, const FhStep &st, fh_kvcache
 }
 
 // ------------------------------------------------------------------------------ output launch
-// Every workgroup stages the inputs of all products once (the recurrent mixers' gate and norm are applied on the way),
-// then each wavefront adds ROWS rows of the residual stream.
-template <int ROWS>
-__global__ __launch_bounds__(256) void k_step_out(FhStep st) {
-    extern __shared__ __attribute__((aligned(16))) float in[]; // [kpo | top * ffp | sffp | norm groups]
+// One wavefront per row of the residual stream, eight rows per workgroup.  A row's weights - of the output projection, of
+// the chosen experts and of the expert of every token - are one list of pieces of 512; a table in the LDS says where each
+// piece lies.  The first pieces are requested before the inputs are staged (the recurrent mixers' gate and norm are
+// applied on the way into the LDS), later ones while earlier ones are multiplied.
+struct OutPiece { const uint16_t *w; int kp, len, in; };
+enum { FH_OUT_AHEAD = 8 };
+
+__global__ __launch_bounds__(512) void k_step_out(FhStep st, int n_pieces) {
+    extern __shared__ __attribute__((aligned(16))) float in[]; // [kpo | top * ffp | sffp | norm groups | pieces]
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
     const FhMoe &m = st.moe;
-    const int n_e = m.experts ? m.top : 0, n_in = st.kpo + n_e * m.ffp + (m.sff ? m.sffp : 0);
+    const int n_e = m.experts ? m.top : 0, n_s = m.sff ? m.sffp : 0, n_in = st.kpo + n_e * m.ffp + n_s;
+    const int n_g = st.kind == FH_MIX_RECURRENT ? (st.rec.norm_groups + 3) / 4 * 4 : 0;
     float *ie = in + st.kpo, *is = ie + n_e * m.ffp, *ginv = in + n_in;
-    const int row0 = ((int)blockIdx.x * 4 + wave) * ROWS;
-    const uint16_t *wr[ROWS];
-    uint4 first[ROWS];
-#pragma unroll
-    for (int r = 0; r < ROWS; r++) {
-        wr[r] = st.wo + (int64_t)(row0 + r < st.width ? row0 + r : st.width - 1) * st.kpo;
-        first[r] = lane * 8 < st.kpo ? *(const uint4 *)(wr[r] + lane * 8) : uint4{0, 0, 0, 0};
+    OutPiece *pt = (OutPiece *)(ginv + n_g);
+    const int po = (st.kpo + 511) / 512, pe = (m.ffp + 511) / 512;
+    for (int i = tid; i < n_pieces; i += 512) {
+        OutPiece p;
+        int k;
+        if (i < po) k = i * 512, p.w = st.wo + k, p.kp = st.kpo, p.in = k;
+        else if (i < po + n_e * pe) {
+            const int j = (i - po) / pe;
+            k = (i - po) % pe * 512;
+            p.w = m.down + (int64_t)st.ids[j] * m.down_stride + k, p.kp = m.ffp, p.in = st.kpo + j * m.ffp + k;
+        } else k = (i - po - n_e * pe) * 512, p.w = m.s_down + k, p.kp = m.sffp, p.in = st.kpo + n_e * m.ffp + k;
+        p.len = p.kp - k;
+        pt[i] = p;
     }
+    __syncthreads();
+    const int row = (int)blockIdx.x * 8 + wave, r = row < st.width ? row : st.width - 1;
+    uint4 u[FH_OUT_AHEAD];
+    auto fetch = [&](int i) -> uint4 {
+        if (i >= n_pieces) return uint4{0, 0, 0, 0};
+        const OutPiece p = pt[i];
+        return lane * 8 < p.len ? *(const uint4 *)(p.w + (int64_t)r * p.kp + lane * 8) : uint4{0, 0, 0, 0};
+    };
+#pragma unroll
+    for (int i = 0; i < FH_OUT_AHEAD; i++) u[i] = fetch(i);
     if (st.kind == FH_MIX_RECURRENT) {
-        const FhRecurrent &r = st.rec;
-        const float *gate = st.proj + r.col_g;
-        const int inner = r.heads * r.vdim, gl = inner / r.norm_groups;
-        for (int i = tid; i < st.kpo; i += 256) {
+        const FhRecurrent &rc = st.rec;
+        const float *gate = st.proj + rc.col_g;
+        const int inner = rc.heads * rc.vdim, gl = inner / rc.norm_groups;
+        for (int i = tid; i < st.kpo; i += 512) {
             float v = i < inner ? st.o[i] : 0.f;
-            if (r.gate_first && i < inner) v *= fh_silu_f(gate[i]);
+            if (rc.gate_first && i < inner) v *= fh_silu_f(gate[i]);
             in[i] = v;
         }
         __syncthreads();
-        for (int g = wave; g < r.norm_groups; g += 4) {
+        for (int g = wave; g < rc.norm_groups; g += 8) {
             float ss = 0.f;
             for (int i = lane; i < gl; i += 64) ss = fmaf(in[g * gl + i], in[g * gl + i], ss);
             ss = fh_wave_sum(ss);
-            if (lane == 0) ginv[g] = 1.0f / sqrtf(ss / (float)gl + r.eps);
+            if (lane == 0) ginv[g] = 1.0f / sqrtf(ss / (float)gl + rc.eps);
         }
         __syncthreads();
-        for (int i = tid; i < inner; i += 256) {
-            float v = in[i] * ginv[i / gl] * r.norm[r.norm_len == inner ? i : i % r.norm_len];
-            if (!r.gate_first) v *= fh_silu_f(gate[i]);
+        for (int i = tid; i < inner; i += 512) {
+            float v = in[i] * ginv[i / gl] * rc.norm[rc.norm_len == inner ? i : i % rc.norm_len];
+            if (!rc.gate_first) v *= fh_silu_f(gate[i]);
             in[i] = v;
         }
     } else {
         const int inner = st.lat.heads * st.lat.dv;
-        for (int i = tid; i < st.kpo; i += 256) in[i] = i < inner ? st.o[i] : 0.f;
+        for (int i = tid; i < st.kpo; i += 512) in[i] = i < inner ? st.o[i] : 0.f;
     }
     for (int j = 0; j < n_e; j++) {
         const float w = st.wts[j];
-        for (int i = tid; i < m.ffp; i += 256) ie[j * m.ffp + i] = i < m.ff ? w * st.act[(int64_t)j * m.ffp + i] : 0.f;
+        for (int i = tid; i < m.ffp; i += 512) ie[j * m.ffp + i] = i < m.ff ? w * st.act[(int64_t)j * m.ffp + i] : 0.f;
     }
-    if (m.sff)
-        for (int i = tid; i < m.sffp; i += 256) {
-            const int g = i / 16 * 32 + i % 16;
-            is[i] = fh_silu_f(st.s_gu[g]) * st.s_gu[g + 16];
-        }
+    for (int i = tid; i < n_s; i += 512) {
+        const int g = i / 16 * 32 + i % 16;
+        is[i] = fh_silu_f(st.s_gu[g]) * st.s_gu[g + 16];
+    }
     __syncthreads();
-    float acc[ROWS];
+    float acc = 0.f;
+    for (int b = 0; b < n_pieces; b += FH_OUT_AHEAD) {
 #pragma unroll
-    for (int r = 0; r < ROWS; r++) acc[r] = 0.f;
-    if (lane * 8 < st.kpo)
-#pragma unroll
-        for (int r = 0; r < ROWS; r++) acc[r] = dot8(first[r], in + lane * 8, acc[r]);
-    auto sweep = [&](const uint16_t *w, int kp, const float *x, int c0) {
-#pragma unroll
-        for (int r = 0; r < ROWS; r++) wr[r] = w + (int64_t)(row0 + r < st.width ? row0 + r : st.width - 1) * kp;
-#pragma unroll 2
-        for (int c = c0 + lane * 8; c < kp; c += 512) {
-            uint4 u[ROWS];
-#pragma unroll
-            for (int r = 0; r < ROWS; r++) u[r] = *(const uint4 *)(wr[r] + c);
-#pragma unroll
-            for (int r = 0; r < ROWS; r++) acc[r] = dot8(u[r], x + c, acc[r]);
+        for (int i = 0; i < FH_OUT_AHEAD; i++) {
+            const uint4 w = u[i];
+            u[i] = fetch(b + i + FH_OUT_AHEAD);
+            if (b + i < n_pieces && lane * 8 < pt[b + i].len) acc = dot8(w, in + pt[b + i].in + lane * 8, acc);
         }
-    };
-    sweep(st.wo, st.kpo, in, 512);
-    for (int j = 0; j < n_e; j++) sweep(m.down + (int64_t)st.ids[j] * m.down_stride, m.ffp, ie + j * m.ffp, 0);
-    if (m.sff) sweep(m.s_down, m.sffp, is, 0);
-#pragma unroll
-    for (int r = 0; r < ROWS; r++) acc[r] = fh_wave_sum(acc[r]);
-    if (lane == 0)
-#pragma unroll
-        for (int r = 0; r < ROWS; r++)
-            if (row0 + r < st.width) st.x[row0 + r] += acc[r];
+    }
+    acc = fh_wave_sum(acc);
+    if (lane == 0 && row < st.width) st.x[row] += acc;
 }
 
 fh_status fh_step_out(fh_device *dev, const FhStep &st) {
     const FhMoe &m = st.moe;
-    const size_t lds = (size_t)(st.kpo + (m.experts ? m.top * m.ffp : 0) + (m.sff ? m.sffp : 0) +
-                                (st.kind == FH_MIX_RECURRENT ? st.rec.norm_groups : 0)) * 4;
+    const int n_e = m.experts ? m.top : 0, n_s = m.sff ? m.sffp : 0;
+    const int pieces = (st.kpo + 511) / 512 + n_e * ((m.ffp + 511) / 512) + (n_s + 511) / 512;
+    const size_t lds = (size_t)(st.kpo + n_e * m.ffp + n_s + (st.kind == FH_MIX_RECURRENT ? (st.rec.norm_groups + 3) / 4 * 4 : 0)) * 4 +
+                       (size_t)pieces * sizeof(OutPiece);
     FH_REQUIRE(lds <= 156 * 1024, "a decode step stages at most 156 KB of inputs (%zu bytes needed)", lds);
-    const int rows = st.width >= dev->compute_units * 8 ? 2 : 1;
-    const void *fn = rows == 2 ? (const void *)k_step_out<2> : (const void *)k_step_out<1>;
-    if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, fn, lds));
-    const dim3 grid((unsigned)((st.width + 4 * rows - 1) / (4 * rows)));
-    if (rows == 2) k_step_out<2><<<grid, 256, lds, dev->stream>>>(st);
-    else k_step_out<1><<<grid, 256, lds, dev->stream>>>(st);
+    if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)k_step_out, lds));
+    k_step_out<<<dim3((unsigned)((st.width + 7) / 8)), 512, lds, dev->stream>>>(st, pieces);
     FH_HIP(hipGetLastError());
     return FH_OK;
 }
