@@ -325,16 +325,26 @@ __global__ __launch_bounds__(256) void k_matvec_norm(const float *__restrict__ x
 #pragma unroll
     for (int r = 0; r < ROWS; r++) cur[r] = in0 ? *(const uint4 *)wr[r] : uint4{0, 0, 0, 0};
     float ss = 0.f;
-    for (int i = tid; i < kp; i += 256) {
-        const float v = i < k ? x[i] : 0.f;
-        ss = fmaf(v, v, ss);
-        xs[i] = v;
+    if ((k & 3) == 0) {
+#pragma unroll 4
+        for (int i = tid * 4; i < kp; i += 1024) {
+            const float4 v = i < k ? *(const float4 *)(x + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+            ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+            *(float4 *)(xs + i) = v;
+        }
+    } else {
+        for (int i = tid; i < kp; i += 256) {
+            const float v = i < k ? x[i] : 0.f;
+            ss = fmaf(v, v, ss);
+            xs[i] = v;
+        }
     }
     if (nw) {
         ss = fh_wave_sum(ss);
         if (lane == 0) red[wave] = ss;
         __syncthreads();
         const float inv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)k + eps);
+#pragma unroll 4
         for (int i = tid; i < k; i += 256) xs[i] = xs[i] * inv * nw[i];
     }
     __syncthreads();

@@ -463,29 +463,47 @@ __global__ __launch_bounds__(256) void k_latent_decode_mfma(FhLatent a, const ui
     const int per = ((n + (int)gridDim.x - 1) / (int)gridDim.x + 15) / 16 * 16;
     const int k0 = (int)blockIdx.x * per, k1 = k0 + per < n ? k0 + per : n;
     auto stage = [&](int k) { // pieces of eight elements; zeros behind the row and behind the last key
-        for (int i = tid; i < 64 * npp; i += 256) {
-            const int r = i / npp, c = i % npp;
-            uint4 v = uint4{0, 0, 0, 0};
-            if (k + r < k1 && c < np) v = *(const uint4 *)(ring + (int64_t)(k + r) * row + c * 8);
-            *(uint4 *)(sc + r * CS + c * 8) = v;
+        for (int b = tid; b < 64 * npp; b += 256 * 9) { // nine requests on their way at a time
+            uint4 v[9];
+#pragma unroll
+            for (int j = 0; j < 9; j++) {
+                const int i = b + 256 * j, r = i / npp, c = i % npp;
+                v[j] = uint4{0, 0, 0, 0};
+                if (i < 64 * npp && k + r < k1 && c < np) v[j] = *(const uint4 *)(ring + (int64_t)(k + r) * row + c * 8);
+            }
+#pragma unroll
+            for (int j = 0; j < 9; j++) {
+                const int i = b + 256 * j, r = i / npp, c = i % npp;
+                if (i < 64 * npp) *(uint4 *)(sc + r * CS + c * 8) = v[j];
+            }
         }
     };
-    stage(k0);
-    for (int i = tid; i < 16 * npp; i += 256) {
-        const int r = i / npp, c = i % npp;
-        float v[8];
+    for (int b = tid; b < 16 * npp; b += 256 * 5) {
+        float v[5][8];
 #pragma unroll
-        for (int e = 0; e < 8; e++) v[e] = 0.f;
-        if (h0 + r < a.heads && c < np) {
-            const float4 x = *(const float4 *)(qa + (int64_t)(h0 + r) * row + c * 8), y = *(const float4 *)(qa + (int64_t)(h0 + r) * row + c * 8 + 4);
-            v[0] = x.x, v[1] = x.y, v[2] = x.z, v[3] = x.w, v[4] = y.x, v[5] = y.y, v[6] = y.z, v[7] = y.w;
+        for (int j = 0; j < 5; j++) {
+            const int i = b + 256 * j, r = i / npp, c = i % npp;
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[j][e] = 0.f;
+            if (i < 16 * npp && h0 + r < a.heads && c < np) {
+                const float4 x = *(const float4 *)(qa + (int64_t)(h0 + r) * row + c * 8), y = *(const float4 *)(qa + (int64_t)(h0 + r) * row + c * 8 + 4);
+                v[j][0] = x.x, v[j][1] = x.y, v[j][2] = x.z, v[j][3] = x.w, v[j][4] = y.x, v[j][5] = y.y, v[j][6] = y.z, v[j][7] = y.w;
+            }
         }
-        uint16_t hi[8], lo[8];
+        if (b == tid) stage(k0);
 #pragma unroll
-        for (int e = 0; e < 8; e++) hi[e] = fh_f32_bf(v[e]), lo[e] = fh_f32_bf(v[e] - fh_bf_f32(hi[e]));
-        __builtin_memcpy(sq + r * CS + c * 8, hi, 16);
-        __builtin_memcpy(sq + (16 + r) * CS + c * 8, lo, 16);
+        for (int j = 0; j < 5; j++) {
+            const int i = b + 256 * j, r = i / npp, c = i % npp;
+            uint16_t hi[8], lo[8];
+#pragma unroll
+            for (int e = 0; e < 8; e++) hi[e] = fh_f32_bf(v[j][e]), lo[e] = fh_f32_bf(v[j][e] - fh_bf_f32(hi[e]));
+            if (i < 16 * npp) {
+                __builtin_memcpy(sq + r * CS + c * 8, hi, 16);
+                __builtin_memcpy(sq + (16 + r) * CS + c * 8, lo, 16);
+            }
+        }
     }
+    if (tid >= 16 * npp) stage(k0); // a thread without query pieces
     fh_f4 o[NT];
 #pragma unroll
     for (int t = 0; t < NT; t++) o[t] = fh_f4{0.f, 0.f, 0.f, 0.f};
@@ -494,7 +512,6 @@ __global__ __launch_bounds__(256) void k_latent_decode_mfma(FhLatent a, const ui
         __syncthreads();
         fh_f4 S = fh_f4{0.f, 0.f, 0.f, 0.f};
         if (k + 16 * wave < k1)
-#pragma unroll 4
             for (int x = 0; x < steps; x++) {
                 fh_bf8 c, h, l;
                 fh_frag_load(c, sc + (16 * wave + li) * CS + 32 * x + 8 * g);
@@ -584,6 +601,11 @@ __global__ __launch_bounds__(256) void k_latent_values(FhLatent a, const float *
         const int r = r0 + i < a.dv ? r0 + i : a.dv - 1;
         w[i] = lane * 8 < a.rp ? *(const uint4 *)(a.uv + (int64_t)(h * a.dv + r) * a.rp + lane * 8) : uint4{0, 0, 0, 0};
     }
+    // this thread's two columns of the first 32 splits (an empty split holds zeros)
+    auto two = [&](int i, int x) { return i < splits && x < a.r8 ? *(const float2 *)(p + (int64_t)i * st + x) : make_float2(0.f, 0.f); };
+    float2 y[32];
+#pragma unroll
+    for (int i = 0; i < 32; i++) y[i] = two(i, tid * 2);
     if (wave == 0) {
         static_assert(FH_LATENT_MAX_SPLITS <= 64, "one split per lane");
         const float z = a.sink ? a.sink[h] * FH_LOG2E : -INFINITY;
@@ -594,15 +616,19 @@ __global__ __launch_bounds__(256) void k_latent_values(FhLatent a, const float *
         const float f = m == -INFINITY ? 0.f : exp2f(m - mm);
         float d = fh_wave_sum(f * l);
         if (a.sink) d += exp2f(z - mm);
-        if (lane < splits) fw[lane] = f / d;
+        fw[lane] = lane < splits ? f / d : 0.f;
     }
     __syncthreads();
-    for (int x = tid; x < a.rp; x += 256) {
-        float v = 0.f;
-        if (x < a.r8)
-#pragma unroll 8
-            for (int i = 0; i < splits; i++) v = fmaf(fw[i], fw[i] != 0.f ? p[i * st + x] : 0.f, v);
-        oc[x] = v;
+    for (int x = tid * 2; x < a.rp; x += 512) {
+        float2 v = make_float2(0.f, 0.f);
+        for (int i0 = 0; i0 < splits; i0 += 32) {
+            if (i0 || x >= 512)
+#pragma unroll
+                for (int i = 0; i < 32; i++) y[i] = two(i0 + i, x);
+#pragma unroll
+            for (int i = 0; i < 32; i++) v.x = fmaf(fw[i0 + i], y[i].x, v.x), v.y = fmaf(fw[i0 + i], y[i].y, v.y);
+        }
+        *(float2 *)(oc + x) = v;
     }
     __syncthreads();
     float acc[8];

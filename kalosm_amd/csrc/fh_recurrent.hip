@@ -268,7 +268,11 @@ __global__ __launch_bounds__(256, 1) void k_rec_chunk_scan(FhRecurrent r, FhRecW
     constexpr int SW = DP / 16 / ST;                                    // wavefronts with state rows
     __shared__ __attribute__((aligned(16))) float ss[16 * SL], su[16 * UL], sd[16 * UL], cs[2][64];
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, li = lane & 15, g = lane >> 4;
-    const int h = blockIdx.y, kh = h / (r.heads / r.kv_heads), col0 = (int)blockIdx.x * 16, col = col0 + li;
+    // The column blocks of a head read the same operands: they go to one of the eight dies, whose L2 then serves all but one
+    // (workgroups are dealt to the dies in turn).
+    const int ncb = c.vp / 16, lin = blockIdx.x, full = r.heads / 8 * 8 * ncb;
+    const int h = lin < full ? lin % 8 + lin / (8 * ncb) * 8 : lin / ncb, cb = lin < full ? lin / 8 % ncb : lin % ncb;
+    const int kh = h / (r.heads / r.kv_heads), col = cb * 16 + li;
     const bool live = col < r.vdim, owner = wave < SW;
     float *sp = state + ((int64_t)h * r.vdim + (live ? col : r.vdim - 1)) * r.dim;
     fh_f4 S[ST];
@@ -284,6 +288,8 @@ __global__ __launch_bounds__(256, 1) void k_rec_chunk_scan(FhRecurrent r, FhRecW
         float4 w[DELTA ? DP / 16 : 1], q[DP / 16], m[4], kt[ST][4];
         float u[4], v[4], la;
     } o0, o1;
+    // No branches around the requests: the number in flight is then known at compile time, so that waiting for one chunk's
+    // operands does not wait for the next one's.  Places outside the portion read a valid address instead.
     auto load = [&](Ops &o, int ch) {
         const int64_t hc = (int64_t)ch * r.heads + h;
         const int t = ch * 64 + 16 * wave + li, tq = t < s ? t : s - 1; // rows past the end are multiplied by zeros of M and decays
@@ -297,28 +303,27 @@ __global__ __launch_bounds__(256, 1) void k_rec_chunk_scan(FhRecurrent r, FhRecW
         for (int x = 0; x < DP / 16; x++) o.q[x] = *(const float4 *)(qp + 16 * x);
         const float *mp = c.m + hc * 4096 + (16 * wave + li) * 64 + 4 * g;
 #pragma unroll
-        for (int b = 0; b < 4; b++)
-            if (b <= wave) o.m[b] = *(const float4 *)(mp + 16 * b);
-        if (owner) {
-            const float *kp = c.kt + (((int64_t)ch * r.kv_heads + kh) * DP + wave * ST * 16 + li) * 64 + 4 * g;
+        for (int b = 0; b < 4; b++) o.m[b] = *(const float4 *)(mp + 16 * b); // blocks behind the diagonal are never used
+        const float *kp = c.kt + (((int64_t)ch * r.kv_heads + kh) * DP + (owner ? wave : 0) * ST * 16 + li) * 64 + 4 * g;
 #pragma unroll
-            for (int i = 0; i < ST; i++)
+        for (int i = 0; i < ST; i++)
 #pragma unroll
-                for (int b = 0; b < 4; b++) o.kt[i][b] = *(const float4 *)(kp + i * 1024 + 16 * b);
-        }
+            for (int b = 0; b < 4; b++) o.kt[i][b] = *(const float4 *)(kp + i * 1024 + 16 * b);
 #pragma unroll
         for (int e = 0; e < 4; e++) {
-            const int row = 16 * wave + 4 * g + e, tt = ch * 64 + row;
-            const bool in = tt < s && live;
-            o.v[e] = in && (!DELTA || r.d_skip) ? w.v[((int64_t)tt * r.heads + h) * r.vdim + col] : 0.f;
-            o.u[e] = DELTA ? c.u0[(hc * 64 + row) * c.vp + col] : in ? o.v[e] * w.beta[(int64_t)tt * r.heads + h] : 0.f;
+            const int row = 16 * wave + 4 * g + e, tt = ch * 64 + row < s ? ch * 64 + row : s - 1;
+            if (DELTA) o.u[e] = c.u0[(hc * 64 + row) * c.vp + col];
+            else {
+                o.v[e] = w.v[((int64_t)tt * r.heads + h) * r.vdim + (live ? col : r.vdim - 1)];
+                o.u[e] = w.beta[(int64_t)tt * r.heads + h];
+            }
         }
-        o.la = ch * 64 + lane < s ? w.la[(int64_t)(ch * 64 + lane) * r.heads + h] : 0.f;
+        o.la = w.la[(int64_t)(ch * 64 + lane < s ? ch * 64 + lane : s - 1) * r.heads + h];
     };
     auto step = [&](const Ops &o, int ch) {
         float *c_ = cs[ch & 1];
         if (wave == 0) {
-            float v = o.la;
+            float v = ch * 64 + lane < s ? o.la : 0.f;
 #pragma unroll
             for (int d = 1; d < 64; d <<= 1) {
                 const float u = __shfl_up(v, d, 64);
@@ -342,7 +347,7 @@ __global__ __launch_bounds__(256, 1) void k_rec_chunk_scan(FhRecurrent r, FhRecW
 #pragma unroll
         for (int e = 0; e < 4; e++) {
             const float ct = c_[16 * wave + 4 * g + e];
-            u[e] = o.u[e] - ws[e];
+            u[e] = DELTA ? o.u[e] - ws[e] : ch * 64 + 16 * wave + 4 * g + e < s ? o.u[e] * o.v[e] : 0.f;
             ud[e] = expf(end - ct) * u[e];
             out[e] = expf(ct) * qs[e];
         }
@@ -364,15 +369,15 @@ __global__ __launch_bounds__(256, 1) void k_rec_chunk_scan(FhRecurrent r, FhRecW
 #pragma unroll
         for (int e = 0; e < 4; e++) {
             const int tt = ch * 64 + 16 * wave + 4 * g + e;
-            if (tt < s && live) w.o[((int64_t)tt * r.heads + h) * r.vdim + col] = out[e] + skip * o.v[e];
+            if (tt < s && live) w.o[((int64_t)tt * r.heads + h) * r.vdim + col] = DELTA ? out[e] : out[e] + skip * o.v[e];
         }
     };
     load(o0, 0);
     for (int ch = 0; ch < c.n; ch += 2) { // the next chunk's operands are requested before the current one is worked on
-        if (ch + 1 < c.n) load(o1, ch + 1);
+        load(o1, ch + 1 < c.n ? ch + 1 : ch);
         step(o0, ch);
         if (ch + 1 >= c.n) break;
-        if (ch + 2 < c.n) load(o0, ch + 2);
+        load(o0, ch + 2 < c.n ? ch + 2 : ch);
         step(o1, ch + 1);
     }
 #pragma unroll
@@ -391,7 +396,7 @@ static fh_status rec_chunked(fh_device *dev, const FhRecurrent &r, const FhRecWo
     auto prep = k_rec_chunk_prep<DP, DELTA>;
     if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)prep, lds));
     prep<<<dim3((unsigned)c.n, (unsigned)r.heads), 256, lds, dev->stream>>>(r, w, c, s);
-    k_rec_chunk_scan<DP, DELTA><<<dim3((unsigned)(c.vp / 16), (unsigned)r.heads), 256, 0, dev->stream>>>(r, w, c, state, s, first);
+    k_rec_chunk_scan<DP, DELTA><<<dim3((unsigned)(c.vp / 16 * r.heads)), 256, 0, dev->stream>>>(r, w, c, state, s, first);
     FH_HIP(hipGetLastError());
     return FH_OK;
 }

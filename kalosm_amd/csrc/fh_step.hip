@@ -159,7 +159,7 @@ __device__ __forceinline__ void expert_step(const FhStep &st, int b, float *lds)
                 if (tile == 0) st.ids[slot] = e, st.wts[slot] = w;
             }
         });
-    for (int i = tid; i < st.kp; i += 256) lds[i] = st.hn[i];
+    for (int i = tid * 4; i < st.kp; i += 1024) *(float4 *)(lds + i) = *(const float4 *)(st.hn + i);
     __syncthreads();
     const uint16_t *w = m.gate_up + (int64_t)*who * m.gu_stride;
     const uint16_t *row[4];
@@ -295,9 +295,13 @@ __global__ __launch_bounds__(512) void k_step_out(FhStep st, int n_pieces) {
         const int inner = st.lat.heads * st.lat.dv;
         for (int i = tid; i < st.kpo; i += 512) in[i] = i < inner ? st.o[i] : 0.f;
     }
-    for (int j = 0; j < n_e; j++) {
+#pragma unroll 4
+    for (int i = tid * 4; i < n_e * m.ffp; i += 2048) {
+        const int j = i / m.ffp, c = i % m.ffp;
         const float w = st.wts[j];
-        for (int i = tid; i < m.ffp; i += 512) ie[j * m.ffp + i] = i < m.ff ? w * st.act[(int64_t)j * m.ffp + i] : 0.f;
+        const float4 v = *(const float4 *)(st.act + i);
+        *(float4 *)(ie + i) = make_float4(c < m.ff ? w * v.x : 0.f, c + 1 < m.ff ? w * v.y : 0.f, c + 2 < m.ff ? w * v.z : 0.f,
+                                          c + 3 < m.ff ? w * v.w : 0.f);
     }
     for (int i = tid; i < n_s; i += 512) {
         const int g = i / 16 * 32 + i % 16;
