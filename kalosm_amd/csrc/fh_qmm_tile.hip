@@ -1504,9 +1504,11 @@ __global__ __launch_bounds__(512) void k_qmm_tile2q(QView q, const _Float16 *__r
     stage(0, w0);
     fetch_w(2, w0);
     auto step = [&](int ks, WSlab &wn1) { // wn1: the weights of step ks + 1
-        // The activation pieces of buffer ks & 1 were requested a step ago, before the last five weight loads: all but
-        // those have to be back.  Then the barrier: buffer ks & 1 is complete; the other one is no longer read.
-        asm volatile("s_waitcnt vmcnt(5)" ::: "memory");
+        // The activation pieces of buffer ks & 1 were requested a step ago, before the last weight loads: all but those have
+        // to be back.  They are four at least (the fifth, the block's d, is dropped by the compiler for the steps that do
+        // not use it), so no more than four may still be on their way.  Then the barrier: buffer ks & 1 is complete; the
+        // other one is no longer read.
+        asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
         __syncthreads();
         fetch_x(ks + 1);
         const _Float16 *buf = smem + (ks & 1) * BUF;
