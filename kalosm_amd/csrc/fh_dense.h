@@ -88,9 +88,8 @@ struct FhGemm {
     int n = 0, kp = 0, m = 0;    // n: weight rows of a group
     const FhTile *tiles = nullptr; // grouped: device table and its fill count
     const int *n_tiles = nullptr;
-    int max_tiles = 0;
+    int max_tiles = 0, tile_rows = 64; // rows an entry may cover: 64, or 128 with bf16 activations
 };
-int fh_gemm_tile_rows(int dtype); // rows one entry of FhGemm::tiles may cover
 fh_status fh_gemm(fh_device *dev, int dtype, int epi, const FhGemm &g);
 
 // y[seg][row] = W_seg[row, :] . n(x), n(x) = x / rms(x) * w (w NULL: x as it is).  norm_out (optional) receives n(x).

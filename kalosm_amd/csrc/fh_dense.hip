@@ -224,12 +224,11 @@ __global__ __launch_bounds__(256) void k_gemm_f32(FhGemm g) {
     }
 }
 
-int fh_gemm_tile_rows(int dtype) { (void)dtype; return 64; }
-
 fh_status fh_gemm(fh_device *dev, int dtype, int epi, const FhGemm &g) {
     FH_REQUIRE(g.w && g.x && g.y && g.n > 0 && g.kp > 0 && g.kp % 64 == 0, "bad product");
     FH_REQUIRE(g.tiles ? g.max_tiles > 0 && g.n_tiles : g.m > 0, "product without rows");
     FH_REQUIRE(epi != FH_GEMM_SWIGLU || g.n % 32 == 0, "gate and up rows come in groups of 16");
+    FH_REQUIRE(!g.tiles || g.tile_rows == 64 || (g.tile_rows == 128 && dtype != FH_F32), "row tiles of %d", g.tile_rows);
     FH_REQUIRE(epi != FH_GEMM_ACT_T || !g.tiles, "a grouped product has no transposed form");
     hipStream_t s = dev->stream;
 #define FH_GEMM_EPI(K_, GRID_)                                              \
@@ -249,7 +248,7 @@ fh_status fh_gemm(fh_device *dev, int dtype, int epi, const FhGemm &g) {
     } else {
         const int tn = (g.n + 127) / 128;
         // small row tiles where the large ones would leave compute units without work
-        const bool big = !g.tiles && (int64_t)tn * ((g.m + 127) / 128) >= dev->compute_units;
+        const bool big = g.tiles ? g.tile_rows == 128 : (int64_t)tn * ((g.m + 127) / 128) >= dev->compute_units;
         const int ty = g.tiles ? g.max_tiles : big ? (g.m + 127) / 128 : (g.m + 63) / 64;
         FH_REQUIRE(ty <= 65535, "too many rows for one launch");
         const dim3 grid((unsigned)tn, (unsigned)ty);

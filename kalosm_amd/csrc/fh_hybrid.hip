@@ -433,7 +433,7 @@ fh_status Hybrid::ensure_steps(int s) {
     for (const Layer &l : layer) {
         np = std::max(np, l.np), kpo = std::max(kpo, l.kpo), inner = std::max(inner, l.inner);
         top = std::max(top, l.moe.experts ? l.moe.top : 0), ffp = std::max(ffp, l.moe.ffp), sffp = std::max(sffp, l.moe.sffp);
-        if (l.moe.experts) tiles = std::max(tiles, fh_moe_max_tiles(l.moe, s, fh_gemm_tile_rows(dtype)));
+        if (l.moe.experts) tiles = std::max(tiles, fh_moe_max_tiles(l.moe, s, 64));
         if (l.kind == FH_MIX_RECURRENT) {
             nq = std::max(nq, l.rec.kv_heads * fh_rec_dp(l.rec)), heads = std::max(heads, l.rec.heads);
             chunk = std::max(chunk, fh_rec_chunk_floats(l.rec, s));

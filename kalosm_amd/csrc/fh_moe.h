@@ -28,6 +28,10 @@ struct FhMoeWork {
     void *s_act;    // [t, sffp]
     float *s_y;     // [t, width]
 };
+// rows per tile: the larger ones where an expert has rows to fill them on average
+static inline int fh_moe_tile_rows(const FhMoe &m, int dtype, int s) {
+    return dtype != FH_F32 && (int64_t)s * m.top >= (int64_t)m.experts * 96 ? 128 : 64;
+}
 static inline int fh_moe_max_tiles(const FhMoe &m, int s, int tile_rows) { return s * m.top / tile_rows + m.experts; }
 // x [s, width] += mix [s, width] + the feed-forward of the activation rows h [s, kp]
 fh_status fh_moe_prefill(fh_device *dev, int dtype, const FhMoe &m, const void *h, int kp, const float *proj, int64_t ldp,

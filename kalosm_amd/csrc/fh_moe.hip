@@ -66,7 +66,7 @@ fh_status fh_moe_prefill(fh_device *dev, int dtype, const FhMoe &m, const void *
                          int s, int width, const FhMoeWork &w, const float *mix, float *x) {
     hipStream_t str = dev->stream;
     if (m.experts) {
-        const int tr = fh_gemm_tile_rows(dtype);
+        const int tr = fh_moe_tile_rows(m, dtype, s);
         k_moe_route<<<dim3((unsigned)((s + 3) / 4)), 256, 0, str>>>(m, proj, ldp, s, w.ids, w.wts);
         k_moe_sort<<<dim3(1), 1024, 0, str>>>(m, w.ids, s, tr, w.src, w.inv, w.tiles, w.n_tiles);
         FH_HIP(hipGetLastError());
@@ -74,6 +74,7 @@ fh_status fh_moe_prefill(fh_device *dev, int dtype, const FhMoe &m, const void *
         g.tiles = w.tiles;
         g.n_tiles = w.n_tiles;
         g.max_tiles = fh_moe_max_tiles(m, s, tr);
+        g.tile_rows = tr;
         g.w = m.gate_up, g.w_group = m.gu_stride, g.n = 2 * m.ffp, g.kp = kp;
         g.x = h, g.gather = w.src, g.y = w.act, g.ldy = m.ffp;
         FH_TRY(fh_gemm(dev, dtype, FH_GEMM_SWIGLU, g));
