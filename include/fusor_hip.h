@@ -50,7 +50,8 @@ enum {
 
 /* GgmlType ids, fusor-ml/gguf/src/lib.rs:35-50.  Q4_0, Q8_0, Q4_K and Q6_K weights are re-laid-out for the
  * matrix-core kernels; Q5_0, Q5_K and dense F32 (0) / F16 (1) weights keep the file's layout and run through
- * the per-element kernels (every fh_qmatrix_* call, fh_embed_rows, fh_qmatmul, fh_qmatmul_add2 / _swiglu). */
+ * the per-element kernels (every fh_qmatrix_* call, fh_embed_rows, fh_qmatmul, fh_qmatmul_add2 / _swiglu).  Dense BF16
+ * rows are padded and have kernels of their own (no k restriction; f32 activations are multiplied in f32). */
 enum { FH_Q4_0 = 2, FH_Q5_0 = 6, FH_Q8_0 = 8, FH_Q4_K = 12, FH_Q5_K = 13, FH_Q6_K = 14, FH_BF16 = 30 };
 
 /* MaskKind, fusor-ml/fusor/src/composite/flash_attention.rs:12-24 */
@@ -200,6 +201,9 @@ typedef struct {
     float factor, high_freq_factor, low_freq_factor;
     int32_t original_max_position_embeddings;
 } fh_rope_scaling;
+fh_status fh_rope_tables_scaled(fh_device *dev, int32_t head_dim, int32_t ctx, float theta,
+                                const fh_rope_scaling *scaling, const float *freq_weight_host,
+                                float *cos_dev, float *sin_dev);
 /* YaRN scaling of `dims` rotated dimensions: rotations that turn at least `fast` times within `original` positions keep
  * their frequency, those that turn at most `slow` times are slowed down by `factor`, a ramp over the pair index joins
  * them, and cos and sin carry the factor 0.1 ln(factor) + 1.  scaling NULL: plain frequencies base^(-2i/dims).  The
@@ -209,9 +213,6 @@ typedef struct {
 } fh_yarn_scaling;
 fh_status fh_rope_tables_yarn(fh_device *dev, int32_t dims, int32_t ctx, double base, const fh_yarn_scaling *scaling,
                               float *cos_dev, float *sin_dev);
-fh_status fh_rope_tables_scaled(fh_device *dev, int32_t head_dim, int32_t ctx, float theta,
-                                const fh_rope_scaling *scaling, const float *freq_weight_host,
-                                float *cos_dev, float *sin_dev);
 /* RopeCache::forward{,_interleaved}(&q, &k, start_pos), rope.rs:284-329.  q is [b, hq, s, d] and
  * k is [b, hk, s, d] as VIEWS: element (b, h, t, c) of q lives at q_dev[b*q_sb + h*q_sh + t*q_st + c]
  * (strides in elements), likewise k.  Outputs are contiguous [b, h, s, d].  One launch rotates both. */

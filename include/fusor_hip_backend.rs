@@ -483,3 +483,53 @@ impl HipLlama {
         check(unsafe { sys::fh_llama_reset(self.raw) })
     }
 }
+
+// ------------------------------------------------------------------------------------------ other decoders
+/// A decoder that comes as a folder with `config.json` and `model.safetensors` (architecture by name in the configuration).
+pub struct HipDecoder {
+    dev: HipDevice,
+    raw: *mut sys::FhDecoder,
+    pub vocab: usize,
+}
+unsafe impl Send for HipDecoder {}
+impl Drop for HipDecoder {
+    fn drop(&mut self) {
+        let _g = self.dev.lock();
+        unsafe { sys::fh_decoder_destroy(self.raw) };
+    }
+}
+impl HipDecoder {
+    /// `dtype`: `sys::FH_F32` or `sys::FH_DECODER_BF16`.
+    pub fn open(dev: &HipDevice, folder: &Path, dtype: i32, context: usize) -> Result<Self> {
+        let path = CString::new(folder.to_string_lossy().as_bytes()).map_err(|_| HipError {
+            status: sys::FH_ERR_INVALID,
+            message: "folder name with a NUL byte".into(),
+        })?;
+        let (mut raw, mut vocab) = (ptr::null_mut(), 0i32);
+        {
+            let _g = dev.lock();
+            check(unsafe { sys::fh_decoder_open(dev.raw(), path.as_ptr(), dtype, context as i32, &mut raw) })?;
+            unsafe { sys::fh_decoder_info(raw, &mut vocab, ptr::null_mut(), ptr::null_mut(), ptr::null_mut(), ptr::null_mut()) };
+        }
+        Ok(HipDecoder { dev: dev.clone(), raw, vocab: vocab as usize })
+    }
+    pub fn reset(&mut self) -> Result<()> {
+        let _g = self.dev.lock();
+        check(unsafe { sys::fh_decoder_reset(self.raw) })
+    }
+    /// Logits of the last of `tokens` at the current position.
+    pub fn forward(&mut self, tokens: &[u32]) -> Result<Vec<f32>> {
+        let mut logits = vec![0f32; self.vocab];
+        let _g = self.dev.lock();
+        check(unsafe {
+            sys::fh_decoder_forward(self.raw, tokens.as_ptr(), tokens.len() as i32, ptr::null(), 0, logits.as_mut_ptr(), ptr::null_mut())
+        })?;
+        Ok(logits)
+    }
+    pub fn decode_greedy(&mut self, first_token: u32, steps: usize) -> Result<Vec<u32>> {
+        let mut out = vec![0u32; steps];
+        let _g = self.dev.lock();
+        check(unsafe { sys::fh_decoder_decode_greedy(self.raw, first_token, steps as i32, out.as_mut_ptr(), ptr::null_mut()) })?;
+        Ok(out)
+    }
+}

@@ -1,6 +1,6 @@
 // Decoders whose configuration lists their layers one by one: each layer has a mixer (latent attention, gated delta rule
 // or state space, with sizes of its own) and, optionally, a mixture-of-experts feed-forward.  Registered designs:
-//   Fidasun   parallel residual (mixer and feed-forward read one norm), norms with weights stored around zero, sinks
+//   Fidasun   parallel residual (one norm feeds mixer and feed-forward), norm weights as distances from one, sinks
 // Weights are dense bf16 (safetensors).  Prefill portions run on the matrix cores (fh_dense.hip), one token through the
 // fused step kernels (fh_step.hip); both use the same caches.
 #include "fh_decoder.h"
@@ -18,7 +18,7 @@ namespace {
 // What a design fixes for all of its models.
 struct Design {
     const char *name;
-    bool norm_about_zero; // stored norm weights are distances from one (the layer norms and the final one)
+    bool norm_one_plus; // layer and final norm weights are distances from one
     bool sink;            // attention heads have a learned sink
 };
 const Design DESIGNS[] = {{"Fidasun", true, true}};
@@ -192,7 +192,7 @@ fh_status Hybrid::init(const FhJson &j) {
     n_layers = (int)ls->items.size();
     kpd = (int)fh_pad64(d_model);
     layer.resize(n_layers);
-    const float one = design->norm_about_zero ? 1.f : 0.f;
+    const float one = design->norm_one_plus ? 1.f : 0.f;
     FH_TRY(matrix(vocab, d_model, &embd));
     FH_TRY(matrix(vocab, d_model, &out));
     slot_rows("embed", embd, 0, vocab, d_model);
@@ -213,7 +213,7 @@ fh_status Hybrid::init_layer(int i, const FhJson &j) {
     const FhJson *type = j.find("type"), *c;
     FH_REQUIRE(type && type->is_string(), "configuration: layer %d has no type", i);
     FH_TRY(get_object(j, "mixer", &c));
-    FH_TRY(slot_vector(base + "norm1", &l.norm, d_model, 0, design->norm_about_zero ? 1.f : 0.f));
+    FH_TRY(slot_vector(base + "norm1", &l.norm, d_model, 0, design->norm_one_plus ? 1.f : 0.f));
     // the routed experts' logits are the last columns of the projection row
     int experts = 0;
     const FhJson *mlp = j.find("mlp");

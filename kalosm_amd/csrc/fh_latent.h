@@ -1,9 +1,9 @@
-// Attention over a low-rank latent: what is cached per position is one latent vector c (RMS normed) and one rotated key
-// part shared by all heads; keys and values are linear in c.
+// Attention over a low-rank latent.  A position caches its RMS-normed latent vector c and a rotated key fragment kr that
+// all heads use; the heads' keys and values are linear maps of c.
 //   score(i, j) = (q_h . W_uk,h c_j + qr_h . kr_j) * scale,   out_h = W_uv,h sum_j p_ij c_j
 // Prefill expands keys and values of the visible positions and runs a tiled attention over them; a decode step moves
 // W_uk to the query and W_uv behind the sum, so that it reads the cached rows only.
-// A window of n lets a position see itself and the n - 1 before it; a sink adds exp(sink_h) to the denominator.
+// With a window w, key j is visible to query i while 0 <= i - j < w; a sink adds exp(sink_h) to a head's denominator.
 // Scores, weights and sums are f32; in bf16 serving the operands of the prefill products are bf16, the weights p of the
 // second product as two terms (hi + lo).
 //

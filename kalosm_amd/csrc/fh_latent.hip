@@ -453,7 +453,7 @@ __global__ __launch_bounds__(256) void k_latent_decode_mfma(FhLatent a, const ui
                                                             const int *__restrict__ pos_dev, const float *__restrict__ qa,
                                                             float *__restrict__ part) {
     extern __shared__ __attribute__((aligned(16))) char ld_lds[];
-    const int row = a.r8 + a.drp, steps = (row + 31) / 32, CS = steps * 32 + 8; // LDS row stride
+    const int row = a.r8 + a.drp, steps = (row + 95) / 96 * 3, CS = steps * 32 + 8; // steps of 32 (threes of them), LDS row stride
     uint16_t *sc = (uint16_t *)ld_lds, *sq = sc + 64 * CS, *sp = sq + 2 * 16 * CS; // cache tile, qa hi / lo, P hi / lo
     constexpr int PS = 72, SS = 68;
     float *s_s = (float *)(sp + 2 * 16 * PS), *s_r = s_s + 16 * SS; // scores, rescale factors
@@ -462,48 +462,50 @@ __global__ __launch_bounds__(256) void k_latent_decode_mfma(FhLatent a, const ui
     const int n = *pos_dev + 1 < cap ? *pos_dev + 1 : cap;
     const int per = ((n + (int)gridDim.x - 1) / (int)gridDim.x + 15) / 16 * 16;
     const int k0 = (int)blockIdx.x * per, k1 = k0 + per < n ? k0 + per : n;
-    auto stage = [&](int k) { // pieces of eight elements; zeros behind the row and behind the last key
-        for (int b = tid; b < 64 * npp; b += 256 * 9) { // nine requests on their way at a time
+    auto stage = [&](int k) { // pieces of eight elements, four threads per row; zeros behind the row and behind the last key
+        const int r = tid >> 2;
+        const bool in = k + r < k1;
+        const uint16_t *src = ring + (int64_t)(in ? k + r : 0) * row;
+        for (int c0 = tid & 3; c0 < npp; c0 += 36) { // nine requests on their way at a time
             uint4 v[9];
 #pragma unroll
-            for (int j = 0; j < 9; j++) {
-                const int i = b + 256 * j, r = i / npp, c = i % npp;
-                v[j] = uint4{0, 0, 0, 0};
-                if (i < 64 * npp && k + r < k1 && c < np) v[j] = *(const uint4 *)(ring + (int64_t)(k + r) * row + c * 8);
-            }
+            for (int j = 0; j < 9; j++) v[j] = in && c0 + 4 * j < np ? *(const uint4 *)(src + (c0 + 4 * j) * 8) : uint4{0, 0, 0, 0};
 #pragma unroll
-            for (int j = 0; j < 9; j++) {
-                const int i = b + 256 * j, r = i / npp, c = i % npp;
-                if (i < 64 * npp) *(uint4 *)(sc + r * CS + c * 8) = v[j];
-            }
+            for (int j = 0; j < 9; j++)
+                if (c0 + 4 * j < npp) *(uint4 *)(sc + r * CS + (c0 + 4 * j) * 8) = v[j];
         }
     };
-    for (int b = tid; b < 16 * npp; b += 256 * 5) {
-        float v[5][8];
+    {
+        const int r = tid >> 4;
+        const float *src = qa + (int64_t)(h0 + r < a.heads ? h0 + r : 0) * row;
+        float4 x[5], y[5];
+        auto get = [&](int c0) {
 #pragma unroll
-        for (int j = 0; j < 5; j++) {
-            const int i = b + 256 * j, r = i / npp, c = i % npp;
-#pragma unroll
-            for (int e = 0; e < 8; e++) v[j][e] = 0.f;
-            if (i < 16 * npp && h0 + r < a.heads && c < np) {
-                const float4 x = *(const float4 *)(qa + (int64_t)(h0 + r) * row + c * 8), y = *(const float4 *)(qa + (int64_t)(h0 + r) * row + c * 8 + 4);
-                v[j][0] = x.x, v[j][1] = x.y, v[j][2] = x.z, v[j][3] = x.w, v[j][4] = y.x, v[j][5] = y.y, v[j][6] = y.z, v[j][7] = y.w;
+            for (int j = 0; j < 5; j++) {
+                const int c = c0 + 16 * j;
+                const bool in = c < np && h0 + r < a.heads;
+                x[j] = in ? *(const float4 *)(src + c * 8) : make_float4(0.f, 0.f, 0.f, 0.f);
+                y[j] = in ? *(const float4 *)(src + c * 8 + 4) : make_float4(0.f, 0.f, 0.f, 0.f);
             }
-        }
-        if (b == tid) stage(k0);
+        };
+        get(tid & 15);
+        stage(k0);
+        for (int c0 = tid & 15; c0 < npp; c0 += 80) {
+            if (c0 >= 80) get(c0);
 #pragma unroll
-        for (int j = 0; j < 5; j++) {
-            const int i = b + 256 * j, r = i / npp, c = i % npp;
-            uint16_t hi[8], lo[8];
+            for (int j = 0; j < 5; j++) {
+                const int c = c0 + 16 * j;
+                const float v[8] = {x[j].x, x[j].y, x[j].z, x[j].w, y[j].x, y[j].y, y[j].z, y[j].w};
+                uint16_t hi[8], lo[8];
 #pragma unroll
-            for (int e = 0; e < 8; e++) hi[e] = fh_f32_bf(v[j][e]), lo[e] = fh_f32_bf(v[j][e] - fh_bf_f32(hi[e]));
-            if (i < 16 * npp) {
-                __builtin_memcpy(sq + r * CS + c * 8, hi, 16);
-                __builtin_memcpy(sq + (16 + r) * CS + c * 8, lo, 16);
+                for (int e = 0; e < 8; e++) hi[e] = fh_f32_bf(v[e]), lo[e] = fh_f32_bf(v[e] - fh_bf_f32(hi[e]));
+                if (c < npp) {
+                    __builtin_memcpy(sq + r * CS + c * 8, hi, 16);
+                    __builtin_memcpy(sq + (16 + r) * CS + c * 8, lo, 16);
+                }
             }
         }
     }
-    if (tid >= 16 * npp) stage(k0); // a thread without query pieces
     fh_f4 o[NT];
 #pragma unroll
     for (int t = 0; t < NT; t++) o[t] = fh_f4{0.f, 0.f, 0.f, 0.f};
@@ -512,13 +514,16 @@ __global__ __launch_bounds__(256) void k_latent_decode_mfma(FhLatent a, const ui
         __syncthreads();
         fh_f4 S = fh_f4{0.f, 0.f, 0.f, 0.f};
         if (k + 16 * wave < k1)
-            for (int x = 0; x < steps; x++) {
-                fh_bf8 c, h, l;
-                fh_frag_load(c, sc + (16 * wave + li) * CS + 32 * x + 8 * g);
-                fh_frag_load(h, sq + li * CS + 32 * x + 8 * g);
-                fh_frag_load(l, sq + (16 + li) * CS + 32 * x + 8 * g);
-                S = fh_mma32(h, c, S);
-                S = fh_mma32(l, c, S);
+            for (int x = 0; x < steps; x += 3) {
+                fh_bf8 c[3], h[3], l[3];
+#pragma unroll
+                for (int j = 0; j < 3; j++) {
+                    fh_frag_load(c[j], sc + (16 * wave + li) * CS + 32 * (x + j) + 8 * g);
+                    fh_frag_load(h[j], sq + li * CS + 32 * (x + j) + 8 * g);
+                    fh_frag_load(l[j], sq + (16 + li) * CS + 32 * (x + j) + 8 * g);
+                }
+#pragma unroll
+                for (int j = 0; j < 3; j++) S = fh_mma32(h[j], c[j], S), S = fh_mma32(l[j], c[j], S);
             }
 #pragma unroll
         for (int e = 0; e < 4; e++) s_s[(4 * g + e) * SS + 16 * wave + li] = k + 16 * wave + li < k1 ? S[e] : -INFINITY;
@@ -589,11 +594,14 @@ __global__ __launch_bounds__(256) void k_latent_decode_mfma(FhLatent a, const ui
 }
 
 // Merge of the splits (with the sink) and the value projection: grid (heads, blocks of 32 values).
-__global__ __launch_bounds__(256) void k_latent_values(FhLatent a, const float *__restrict__ part, int splits, float *__restrict__ o) {
+__global__ __launch_bounds__(256) void k_latent_values(FhLatent a, const float *__restrict__ part, int splits, float *__restrict__ o,
+                                                       const int *__restrict__ pos_dev, int cap) {
     extern __shared__ __attribute__((aligned(16))) float oc[]; // [rp]
     __shared__ float fw[FH_LATENT_MAX_SPLITS];
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, h = blockIdx.x, st = a.r8 + 2;
     const float *p = part + (int64_t)h * splits * st;
+    const int n = *pos_dev + 1 < cap ? *pos_dev + 1 : cap, per = ((n + splits - 1) / splits + 15) / 16 * 16;
+    const int live = (n + per - 1) / per; // splits that had keys
     uint4 w[8]; // the first 512 of k of this wavefront's rows, requested before the merge
     const int r0 = (int)blockIdx.y * 32 + wave * 8;
 #pragma unroll
@@ -601,27 +609,27 @@ __global__ __launch_bounds__(256) void k_latent_values(FhLatent a, const float *
         const int r = r0 + i < a.dv ? r0 + i : a.dv - 1;
         w[i] = lane * 8 < a.rp ? *(const uint4 *)(a.uv + (int64_t)(h * a.dv + r) * a.rp + lane * 8) : uint4{0, 0, 0, 0};
     }
-    // this thread's two columns of the first 32 splits (an empty split holds zeros)
-    auto two = [&](int i, int x) { return i < splits && x < a.r8 ? *(const float2 *)(p + (int64_t)i * st + x) : make_float2(0.f, 0.f); };
+    // this thread's two columns of the first 32 splits with keys
+    auto two = [&](int i, int x) { return i < live && x < a.r8 ? *(const float2 *)(p + (int64_t)i * st + x) : make_float2(0.f, 0.f); };
     float2 y[32];
 #pragma unroll
     for (int i = 0; i < 32; i++) y[i] = two(i, tid * 2);
     if (wave == 0) {
         static_assert(FH_LATENT_MAX_SPLITS <= 64, "one split per lane");
         const float z = a.sink ? a.sink[h] * FH_LOG2E : -INFINITY;
-        const float m = lane < splits ? p[lane * st + a.r8] : -INFINITY, l = lane < splits ? p[lane * st + a.r8 + 1] : 0.f;
+        const float m = lane < live ? p[lane * st + a.r8] : -INFINITY, l = lane < live ? p[lane * st + a.r8 + 1] : 0.f;
         float mm = fmaxf(m, z);
 #pragma unroll
         for (int i = 32; i > 0; i >>= 1) mm = fmaxf(mm, __shfl_xor(mm, i, 64));
         const float f = m == -INFINITY ? 0.f : exp2f(m - mm);
         float d = fh_wave_sum(f * l);
         if (a.sink) d += exp2f(z - mm);
-        fw[lane] = lane < splits ? f / d : 0.f;
+        fw[lane] = lane < live ? f / d : 0.f;
     }
     __syncthreads();
     for (int x = tid * 2; x < a.rp; x += 512) {
         float2 v = make_float2(0.f, 0.f);
-        for (int i0 = 0; i0 < splits; i0 += 32) {
+        for (int i0 = 0; i0 < live; i0 += 32) {
             if (i0 || x >= 512)
 #pragma unroll
                 for (int i = 0; i < 32; i++) y[i] = two(i0 + i, x);
@@ -664,7 +672,7 @@ static fh_status latent_decode_t(fh_device *dev, const FhLatent &a, const fh_kvc
     const int row = fh_latent_row(a), hb = a.heads % 2 == 0 ? 2 : 1;
     int splits = cache->capacity / 32;
     splits = splits < 1 ? 1 : splits > FH_LATENT_MAX_SPLITS ? FH_LATENT_MAX_SPLITS : splits;
-    const int cs = (row + 31) / 32 * 32 + 8;
+    const int cs = (row + 95) / 96 * 96 + 8;
     const size_t mlds = (size_t)(96 * cs + 32 * 72) * 2 + (16 * 68 + 16) * 4;
     if (sizeof(T) == 2 && a.r8 <= 640 && mlds <= 156 * 1024 && dev->opt_attn_kernel != 1) {
         const dim3 mgrid((unsigned)splits, (unsigned)((a.heads + 15) / 16));
@@ -678,7 +686,7 @@ static fh_status latent_decode_t(fh_device *dev, const FhLatent &a, const fh_kvc
         else if (a.r8 <= 512) FH_GO(8);
         else FH_GO(10);
 #undef FH_GO
-        k_latent_values<<<dim3((unsigned)a.heads, (unsigned)((a.dv + 31) / 32)), 256, (size_t)a.rp * 4, dev->stream>>>(a, part, splits, o);
+        k_latent_values<<<dim3((unsigned)a.heads, (unsigned)((a.dv + 31) / 32)), 256, (size_t)a.rp * 4, dev->stream>>>(a, part, splits, o, pos_dev, cache->capacity);
         FH_HIP(hipGetLastError());
         return FH_OK;
     }
@@ -698,7 +706,7 @@ static fh_status latent_decode_t(fh_device *dev, const FhLatent &a, const fh_kvc
     else if (row <= 1152) FH_GO(9);
     else FH_FAIL(FH_ERR_UNSUPPORTED, "latent rows of %d elements (at most 1152)", row);
 #undef FH_GO
-    k_latent_values<<<dim3((unsigned)a.heads, (unsigned)((a.dv + 31) / 32)), 256, (size_t)a.rp * 4, dev->stream>>>(a, part, splits, o);
+    k_latent_values<<<dim3((unsigned)a.heads, (unsigned)((a.dv + 31) / 32)), 256, (size_t)a.rp * 4, dev->stream>>>(a, part, splits, o, pos_dev, cache->capacity);
     FH_HIP(hipGetLastError());
     return FH_OK;
 }

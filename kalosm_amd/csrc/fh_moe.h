@@ -1,5 +1,5 @@
-// Mixture-of-experts feed-forward: softmax router, the `top` best experts of every token with their plain scores times
-// a factor as weights, and an optional expert that runs for every token.  Expert weights are stacked: gate | up rows in
+// Mixture-of-experts feed-forward: softmax router, the `top` best experts of a token weighted by scale times their score,
+// and optionally one more expert that is always on.  Expert weights are stacked: gate | up rows in
 // alternating groups of 16, [experts][2 ffp][kp], and down [experts][dp][ffp], with ffp = ff rounded up to 64 (zero rows)
 // and dp = the width rounded up to 16.
 #pragma once
@@ -12,7 +12,7 @@ struct FhMoe {
     int col_z = 0;                               // router logits in a projection row
     const uint16_t *gate_up = nullptr, *down = nullptr;
     int64_t gu_stride = 0, down_stride = 0;      // elements per expert
-    int sff = 0, sffp = 0;                       // the expert of every token (0: none)
+    int sff = 0, sffp = 0;                       // the always-on expert (0: none)
     const uint16_t *s_gate_up = nullptr, *s_down = nullptr;
 };
 // Work arrays of a prefill portion.

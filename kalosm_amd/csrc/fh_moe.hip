@@ -46,7 +46,7 @@ __global__ __launch_bounds__(1024) void k_moe_sort(FhMoe m, const int *__restric
     }
 }
 
-// x += mix + sum of the token's weighted expert rows + the row of the expert of every token
+// x += mix + the token's weighted expert rows + its row of the always-on expert
 __global__ __launch_bounds__(256) void k_moe_combine(FhMoe m, const float *__restrict__ mix, const float *__restrict__ y,
                                                      const float *__restrict__ sy, const int *__restrict__ inv,
                                                      const float *__restrict__ wts, int width, float *__restrict__ x) {

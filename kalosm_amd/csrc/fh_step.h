@@ -22,7 +22,7 @@ struct FhStep {
     float *act = nullptr;        // [top, ffp] expert activations
     int *ids = nullptr;          // [top]
     float *wts = nullptr;        // [top]
-    const float *s_gu = nullptr; // gate and up products of the expert of every token [2 sffp]
+    const float *s_gu = nullptr; // gate and up products of the always-on expert [2 sffp]
     const uint16_t *wo = nullptr; // [width, kpo]
     int kpo = 0, width = 0;
     float *x = nullptr;          // residual stream

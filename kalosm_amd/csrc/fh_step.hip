@@ -232,7 +232,7 @@ fh_status fh_step_middle(fh_device *dev, int dtype, const FhStep &st, fh_kvcache
 
 // ------------------------------------------------------------------------------ output launch
 // One wavefront per row of the residual stream, eight rows per workgroup.  A row's weights - of the output projection, of
-// the chosen experts and of the expert of every token - are one list of pieces of 512; a table in the LDS says where each
+// the chosen experts and of the always-on one - are one list of pieces of 512; a table in the LDS says where each
 // piece lies.  The first pieces are requested before the inputs are staged (the recurrent mixers' gate and norm are
 // applied on the way into the LDS), later ones while earlier ones are multiplied.
 struct OutPiece { const uint16_t *w; int kp, len, in; };

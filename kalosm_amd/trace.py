@@ -1,5 +1,5 @@
-"""Replays a trace through a decoder: steps of given token ids come in as JSON lines, the logits at the wanted places go
-out as files of little-endian 32-bit floats.  One sequence at a time; a step runs only the tokens it brings."""
+"""Replays recorded token ids through a decoder: steps come in as JSON lines, the logits of the places a step names leave as
+little-endian f32 files.  Sequences are replayed one after the other, each continuing on the decoder's caches."""
 from __future__ import annotations
 
 import json

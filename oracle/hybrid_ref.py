@@ -24,7 +24,7 @@ def rms(x, eps):
     return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + eps)
 
 
-def norm_about_zero(x, w, eps):
+def norm_one_plus(x, w, eps):
     """RMS norm whose weight is stored as its distance from one."""
     return rms(x, eps) * (1.0 + w)
 
@@ -64,7 +64,7 @@ def rotate_interleaved(x, positions, freq, amp, angle32=True):
 
 # ---------------------------------------------------------------- latent attention
 def sink_softmax(scores, visible, sink):
-    """Softmax over the visible keys of each row; exp(sink) joins the denominator and nothing else."""
+    """Softmax over the visible keys of each row with exp(sink) added to the denominator."""
     z = np.where(visible, scores, -np.inf)
     m = np.maximum(z.max(axis=-1, keepdims=True), sink)
     e = np.exp(z - m)
@@ -99,7 +99,7 @@ def latent_attention(h, w, c, eps, dtype=np.float64):
 
 # ---------------------------------------------------------------- recurrent mixers
 def short_conv(x, taps_w, bias=None):
-    """Causal convolution per channel, x [t, ch], taps_w [ch, taps]: the last column meets the current token."""
+    """Depthwise causal convolution, x [t, ch], taps_w [ch, taps] with the oldest tap first."""
     T, K = x.shape[0], taps_w.shape[1]
     out = np.zeros_like(x)
     for t in range(T):
@@ -115,8 +115,7 @@ def unit(x):
 
 
 def gated_delta(q, k, v, g, beta):
-    """One head: q, k [t, d], v [t, e], g, beta [t].  The state decays, the key's old value is taken out of what is
-    written, and the read sees the write."""
+    """One head: q, k [t, d], v [t, e], g, beta [t].  Decay, correct the value stored under the key by beta, read."""
     S = np.zeros((q.shape[1], v.shape[1]), q.dtype)
     out = np.zeros_like(v)
     for t in range(len(q)):
@@ -183,7 +182,7 @@ def expert(h, gate, up, down):
 
 
 def route(z, top, scale):
-    """Chosen experts (largest softmax score first) and their weights: the plain scores times `scale`."""
+    """The `top` experts by softmax score, best first, and scale times those scores."""
     e = np.exp(z - z.max())
     s = e / e.sum()
     idx = np.argsort(-s, kind="stable")[:top]
@@ -217,10 +216,10 @@ def forward(cfg, weights, tokens, dtype=np.float64):
     layers = []
     for i, lc in enumerate(cfg["layers"]):
         L = _under(W, f"l{i}.")
-        h = norm_about_zero(x, L["norm1"], eps)
+        h = norm_one_plus(x, L["norm1"], eps)
         y = MIXERS[lc["type"]](h, _under(L, "mix."), lc["mixer"], eps, dtype)
         if lc.get("mlp"):
             y = y + moe(h, _under(L, "mlp."), lc["mlp"])
         x = x + y
         layers.append(x)
-    return norm_about_zero(x, W["final.norm"], eps) @ W["head"].T, np.stack(layers)
+    return norm_one_plus(x, W["final.norm"], eps) @ W["head"].T, np.stack(layers)

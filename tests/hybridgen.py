@@ -55,14 +55,14 @@ CONFIGS = {
                     with_mlp(delta(1, 1, 16, 16, 1), moe(2, 1, 8, 0)), with_mlp(mamba2(1, 16, 16, 1, 1, 1), moe(3, 3, 16, 8))],
                    width=64, vocab=40),
     # no window: the cache grows
-    "full": config([with_mlp(latent(window=0, heads=2, dim=32, rot_dim=16, vdim=32, kv_rank=64), moe(8, 2, 64, 64)),
-                    with_mlp(mamba2(4, 32, 32, 1, 4, 4), moe(8, 2, 64, 64))], width=128, vocab=96),
+    "full": config([with_mlp(latent(window=0, heads=2, dim=40, rot_dim=24, vdim=48, kv_rank=56), moe(8, 2, 64, 64)),
+                    with_mlp(mamba2(4, 40, 48, 1, 4, 4), moe(8, 2, 64, 64))], width=128, vocab=96),
     # head sizes of large models: the widest operand shapes of every kernel
-    "large": config([with_mlp(latent(heads=2, dim=128, rot_dim=64, vdim=128, kv_rank=512, window=70), moe(4, 2, 96, 96)),
-                     with_mlp(delta(4, 2, 128, 128, 4), moe(4, 2, 96, 96)), with_mlp(mamba2(4, 64, 128, 2, 2, 4), None),
+    "large": config([with_mlp(latent(heads=2, dim=128, rot_dim=64, vdim=128, kv_rank=512, window=70), moe(4, 2, 112, 80)),
+                     with_mlp(delta(4, 2, 128, 128, 4), moe(4, 2, 112, 80)), with_mlp(mamba2(4, 64, 128, 2, 2, 4), None),
                      with_mlp(delta(2, 1, 200, 72, 4), None)], width=256, vocab=200),
     # values wider than one block of the attention kernel, latent rows beyond 640
-    "wide": config([with_mlp(latent(heads=3, dim=96, rot_dim=32, vdim=160, kv_rank=640, window=40), None)], width=128, vocab=64),
+    "wide": config([with_mlp(latent(heads=3, dim=96, rot_dim=32, vdim=160, kv_rank=640, window=37), None)], width=128, vocab=64),
 }
 
 

@@ -174,7 +174,7 @@ def test_sink_sizes(dev, sink):
 @pytest.mark.parametrize("a_log,dt", [(-12.0, 0.0), (3.0, 2.0)])
 def test_decays_near_one_and_near_zero(dev, mixer, a_log, dt):
     """A state that forgets nothing over a long prompt, and one that forgets at once."""
-    cfg = G.config([G.with_mlp(G.delta(2, 1, 32, 32, 4) if mixer == "delta" else G.mamba2(2, 32, 32, 1, 1, 4), None)], 128, 64)
+    cfg = G.config([G.with_mlp(G.delta(2, 1, 32, 24, 5) if mixer == "delta" else G.mamba2(2, 40, 32, 1, 2, 3), None)], 128, 64)
     w = G.weights(cfg)
     w["l0.mix.A_log"] = np.full_like(w["l0.mix.A_log"], a_log)
     w["l0.mix.dt_bias"] = np.full_like(w["l0.mix.dt_bias"], dt)
