@@ -62,6 +62,19 @@ def rotate_interleaved(x, positions, freq, amp, angle32=True):
     return out
 
 
+def rotated_halves(x, positions, freq):
+    """x [..., t, d]: of the first n = 2 len(freq) dimensions, i and i + n / 2 form a pair, turned by position * freq_i."""
+    p = np.asarray(positions, np.float32)
+    a = (p[:, None] * freq[None, :].astype(np.float32)).astype(np.float64)
+    c, s = np.cos(a), np.sin(a)
+    out = x.copy()
+    n = len(freq)
+    u, v = x[..., :n], x[..., n:2 * n]
+    out[..., :n] = u * c - v * s
+    out[..., n:2 * n] = v * c + u * s
+    return out
+
+
 # ---------------------------------------------------------------- latent attention
 def sink_softmax(scores, visible, sink):
     """Softmax over the visible keys of each row with exp(sink) added to the denominator."""
@@ -173,7 +186,96 @@ def mamba2(h, w, c, eps, dtype=np.float64):
     return y @ w["o"].T
 
 
-MIXERS = {"latent_attention": latent_attention, "delta": delta, "mamba2": mamba2}
+# ---------------------------------------------------------------- grouped-query attention with kept first tokens
+def kept_window(T, size, keep):
+    """visible[i, j]: j not after i, and less than `size` positions behind it or among the first `keep`."""
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    return (j <= i) & ((i - j < size) | (j < keep))
+
+
+def grouped_attention(h, w, c, eps, dtype=np.float64):
+    """h [t, width] -> [t, width].  w: q, k, v, q.norm, k.norm, o and (optional) sink."""
+    T = h.shape[0]
+    H, G, d, dv = c["heads"], c["kv_heads"], c["dim"], c["vdim"]
+    freq, _ = yarn_frequencies(c["rot"]["base"], c["rot"]["dims"])
+    pos = np.arange(T)
+    q = rms((h @ w["q"].T).reshape(T, H, d), eps) * w["q.norm"]
+    k = rms((h @ w["k"].T).reshape(T, G, d), eps) * w["k.norm"]
+    v = (h @ w["v"].T).reshape(T, G, dv)
+    m = c.get("mask")
+    visible = kept_window(T, m["size"], m.get("keep_first", 0)) if m else kept_window(T, T, 0)
+    out = np.zeros((T, H, dv), dtype)
+    for n in range(H):
+        g = n // (H // G)
+        s = rotate_interleaved(q[:, n], pos, freq, 1.0) @ rotate_interleaved(k[:, g], pos, freq, 1.0).T * c["scale"]
+        out[:, n] = sink_softmax(s, visible, w["sink"][n] if "sink" in w else -np.inf) @ v[:, g]
+    return out.reshape(T, H * dv) @ w["o"].T
+
+
+# ---------------------------------------------------------------- recurrences without a short convolution
+def fixed_decay(q, k, v, decay):
+    """One head: the state forgets by a constant factor per token."""
+    S = np.zeros((q.shape[1], v.shape[1]), q.dtype)
+    out = np.zeros_like(v)
+    for t in range(len(q)):
+        S = decay * S + np.outer(k[t], v[t])
+        out[t] = S.T @ q[t]
+    return out
+
+
+def retention(h, w, c, eps, dtype=np.float64):
+    T = h.shape[0]
+    H, d, dv = c["heads"], c["dim"], c["vdim"]
+    freq, _ = yarn_frequencies(c["rot"]["base"], c["rot"]["dims"])
+    q, k, v = ((h @ w[n].T).reshape(T, H, -1) for n in ("q", "k", "v"))
+    o = np.zeros((T, H, dv), dtype)
+    for n in range(H):
+        qr, kr = (rotated_halves(x[:, n], np.arange(T), freq) for x in (q, k))
+        o[:, n] = fixed_decay(qr, kr * d ** -0.5, v[:, n], c["decay"][n])
+    return (rms(o, eps).reshape(T, H * dv) * silu(h @ w["g"].T)) @ w["o"].T
+
+
+def channel_decay(r, k, v, g, u):
+    """One head: r, k, g [t, d], v [t, e], u [d].  Every key channel forgets at its own rate; the current token's own
+    contribution is read with the bonus u before it joins the state."""
+    S = np.zeros((r.shape[1], v.shape[1]), r.dtype)
+    out = np.zeros_like(v)
+    for t in range(len(r)):
+        kv = np.outer(k[t], v[t])
+        out[t] = (S + u[:, None] * kv).T @ r[t]
+        S = g[t][:, None] * S + kv
+    return out
+
+
+def shifted(h, mu):
+    """Every channel moved by mu towards the previous token's (zeros ahead of the first)."""
+    prev = np.concatenate([np.zeros_like(h[:1]), h[:-1]])
+    return h + (prev - h) * mu
+
+
+def time_mixing(h, w, c, eps, dtype=np.float64):
+    """w: r, k, v, g, w1, w2, w0, u, norm, o and mu.r ... mu.w."""
+    T = h.shape[0]
+    H, d = c["heads"], c["dim"]
+    r, k, v = ((shifted(h, w["mu." + n]) @ w[n].T).reshape(T, H, d) for n in ("r", "k", "v"))
+    gate = silu(shifted(h, w["mu.g"]) @ w["g"].T)
+    z = np.tanh(shifted(h, w["mu.w"]) @ w["w1"].T) @ w["w2"].T + w["w0"]
+    g = np.exp(-np.exp(z)).reshape(T, H, d)
+    o = np.zeros((T, H, d), dtype)
+    for n in range(H):
+        o[:, n] = channel_decay(r[:, n], k[:, n], v[:, n], g[:, n], w["u"][n])
+    return (rms(o, eps).reshape(T, H * d) * w["norm"] * gate) @ w["o"].T
+
+
+def side_by_side(h, w, c, eps, dtype=np.float64):
+    """Attention and time mixing on the same input, added with their scales."""
+    left = grouped_attention(h, _under(w, "left."), c["left"], eps, dtype)
+    right = time_mixing(h, _under(w, "right."), c["right"], eps, dtype)
+    return c["left_scale"] * left + c["right_scale"] * right
+
+
+MIXERS = {"latent_attention": latent_attention, "delta": delta, "mamba2": mamba2, "retention": retention,
+          "parallel": side_by_side}
 
 
 # ---------------------------------------------------------------- feed-forward
@@ -202,24 +304,42 @@ def moe(h, w, c):
     return out
 
 
+def dense(h, w, c):
+    """Two matrices with the square of relu between them."""
+    return np.square(np.maximum(h @ w["up"].T, 0.0)) @ w["down"].T
+
+
 # ---------------------------------------------------------------- model
 def _under(weights, prefix):
     n = len(prefix)
     return {k[n:]: v for k, v in weights.items() if k.startswith(prefix)}
 
 
+def parallel_residual_layer(x, L, lc, eps, dtype):
+    """One norm feeds mixer and feed-forward."""
+    h = norm_one_plus(x, L["norm1"], eps)
+    y = MIXERS[lc["type"]](h, _under(L, "mix."), lc["mixer"], eps, dtype)
+    return x + (y + moe(h, _under(L, "mlp."), lc["mlp"]) if lc.get("mlp") else y)
+
+
+def output_norm_layer(x, L, lc, eps, dtype):
+    """Mixer and feed-forward read the residual stream as it is; what they give is normed before it is added."""
+    x = x + rms(MIXERS[lc["type"]](x, _under(L, "mix."), lc["mixer"], eps, dtype), eps) * L["norm1"]
+    return x + rms(dense(x, _under(L, "mlp."), lc["mlp"]), eps) * L["norm2"] if lc.get("mlp") else x
+
+
 def forward(cfg, weights, tokens, dtype=np.float64):
     """Logits of every position [t, vocab] and the residual stream after every layer [layers, t, width]."""
     W = {k: np.asarray(v, dtype) for k, v in weights.items()}
     eps = cfg["norm"]["eps"]
+    zovovik = cfg["architecture"] == "Zovovik"
+    layer = output_norm_layer if zovovik else parallel_residual_layer
     x = W["embed"][np.asarray(tokens)]
+    if zovovik:
+        x = x + W["pos"][:len(x)]
     layers = []
     for i, lc in enumerate(cfg["layers"]):
-        L = _under(W, f"l{i}.")
-        h = norm_one_plus(x, L["norm1"], eps)
-        y = MIXERS[lc["type"]](h, _under(L, "mix."), lc["mixer"], eps, dtype)
-        if lc.get("mlp"):
-            y = y + moe(h, _under(L, "mlp."), lc["mlp"])
-        x = x + y
+        x = layer(x, _under(W, f"l{i}."), lc, eps, dtype)
         layers.append(x)
-    return norm_one_plus(x, W["final.norm"], eps) @ W["head"].T, np.stack(layers)
+    h = rms(x, eps) * W["final.norm"] if zovovik else norm_one_plus(x, W["final.norm"], eps)
+    return h @ W["head"].T, np.stack(layers)
