@@ -76,7 +76,8 @@ enum {
     FH_GEMM_F32 = 0,        // y f32 [m, ldy]
     FH_GEMM_ACT = 1,        // y in the activation type [m, ldy]
     FH_GEMM_ACT_T = 2,      // y in the activation type, transposed: [n, ldy], ldy >= m
-    FH_GEMM_SWIGLU = 3      // weight rows in alternating groups of 16 (gate, up): y = silu(gate) * up, activation type [m, ldy]
+    FH_GEMM_SWIGLU = 3,     // weight rows in alternating groups of 16 (gate, up): y = silu(gate) * up, activation type [m, ldy]
+    FH_GEMM_RELU2 = 4       // y = max(x, 0)^2, activation type [m, ldy]
 };
 struct FhGemm {
     const uint16_t *w = nullptr; // [n, kp]
@@ -99,3 +100,56 @@ fh_status fh_matvec_norm(fh_device *dev, const float *x, int k, const float *w, 
 // f32 rows -> activation rows of stride kp: plain copy, or RMS norm with weight w (w NULL: copy)
 fh_status fh_rows_to_act(fh_device *dev, int dtype, const float *x, int64_t ldx, int rows, int k, const float *w, float eps,
                          void *y, int kp);
+
+// The row table of a product whose `groups` groups have s rows each, group after group (FhGemm::tiles, n_tiles).
+static inline int fh_group_tile_rows(const fh_device *dev, int dtype, int groups, int s, int n) {
+    return dtype != FH_F32 && (int64_t)groups * ((s + 127) / 128) * ((n + 127) / 128) >= dev->compute_units ? 128 : 64;
+}
+fh_status fh_group_tiles(fh_device *dev, int groups, int s, int tile_rows, FhTile *tiles, int *n_tiles);
+
+// ---------------------------------------------------------------- residual streams that are normed at a sublayer's end
+// x_out = x + y / rms(y) * w per row, and (act not NULL) x_out as activation rows of stride kp; x_out may be x.
+fh_status fh_add_normed(fh_device *dev, int dtype, const float *x, const float *y, int rows, int k, const float *w, float eps,
+                        float *x_out, void *act, int kp);
+// x[t] = table row ids[t] + pos row (pos + t, or *pos_dev for one token); pos_table NULL: without.  Also activation rows.
+fh_status fh_embed_at(fh_device *dev, int dtype, const fh_qmatrix *table, const fh_qmatrix *pos_table, const uint32_t *ids, int s,
+                      int pos, const int *pos_dev, float *x, void *act, int kp);
+
+// Token shift: mixture n of token t is x_t + (x_(t-1) - x_t) * mu_n.  The row ahead of the portion is kept in a state of two
+// rows (position p in row p % 2; nothing is read at position 0).
+enum { FH_SHIFT_MAX = 6 };
+struct FhShift {
+    int n = 0;
+    const float *mu[FH_SHIFT_MAX] = {};
+    void *y[FH_SHIFT_MAX] = {};   // [s, kp]
+    int f32[FH_SHIFT_MAX] = {};   // rows in f32 whatever the activation type
+};
+// y = tanh(W x) in 32 bits, W [n, kp] for a small n: x [rows, kp] f32, y [rows, ldy] f32 with zeros from n on.
+fh_status fh_low_rank_tanh(fh_device *dev, const float *x, int kp, int rows, const uint16_t *w, int n, float *y, int ldy);
+fh_status fh_token_shift(fh_device *dev, int dtype, const FhShift &m, const float *x, int s, int k, int pos, float *state, int kp);
+
+// Decode: x' = x + y / rms(y) * w (y NULL: x), then up to FH_MV_MAX matrices on mixtures of x' (mu NULL: x' itself).  One
+// workgroup stores x' (x_out, not x) and, with a state, the row of this position.
+enum { FH_MV_ACT_NONE = 0, FH_MV_ACT_RELU2 = 1, FH_MV_ACT_TANH = 2, FH_MV_MAX = 6 };
+struct FhMvMix { const uint16_t *w; const float *mu; float *y; int n, act; };
+struct FhMvAdd {
+    const float *x = nullptr, *y = nullptr, *w = nullptr;
+    float eps = 0.f;
+    float *x_out = nullptr;
+    float *state = nullptr;       // [2][k]
+    const int *pos_dev = nullptr;
+};
+fh_status fh_matvec_mix(fh_device *dev, const FhMvAdd &in, int k, const FhMvMix *segs, int n_segs);
+
+#ifdef __HIPCC__
+// Dimension i of a head after rotation: pairs (2i, 2i + 1), or (i, i + pairs) with `halves`, of the first 2 pairs dimensions;
+// at(i) gives dimension i before it, ct / st the row of the position.
+template <typename F>
+__device__ __forceinline__ float fh_rotated(F at, int i, int pairs, int halves, const float *ct, const float *st) {
+    const float v = at(i);
+    if (i >= 2 * pairs) return v;
+    if (halves) return i < pairs ? v * ct[i] - at(i + pairs) * st[i] : v * ct[i - pairs] + at(i - pairs) * st[i - pairs];
+    const int p = i >> 1;
+    return i & 1 ? v * ct[p] + at(i - 1) * st[p] : v * ct[p] - at(i + 1) * st[p];
+}
+#endif

@@ -45,6 +45,12 @@ __device__ __forceinline__ void gemm_store(void *y, int64_t ldy, int m_row, int 
     }
 }
 
+__device__ __forceinline__ fh_f4 relu2(fh_f4 v) {
+#pragma unroll
+    for (int e = 0; e < 4; e++) v[e] = fmaxf(v[e], 0.f) * fmaxf(v[e], 0.f);
+    return v;
+}
+
 __device__ __forceinline__ int gemm_sw(int row) { return (row >> 1) & 7; }
 
 template <int BM, int EPI>
@@ -139,6 +145,8 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(FhGemm g) {
 #pragma unroll
                 for (int r = 0; r < 4; r++) v[r] = fh_silu_f(acc[a][b][r]) * acc[a + 1 < FN ? a + 1 : a][b][r];
                 gemm_store<FH_GEMM_ACT, uint16_t>(g.y, g.ldy, mb + li, nb / 2 + gq * 4, v, m_end, g.n / 2);
+            } else if (EPI == FH_GEMM_RELU2) {
+                gemm_store<FH_GEMM_ACT, uint16_t>(g.y, g.ldy, mb + li, nb + gq * 4, relu2(acc[a][b]), m_end, g.n);
             } else if (EPI == FH_GEMM_ACT_T) {
                 gemm_store<EPI, uint16_t>(g.y, g.ldy, mb + gq * 4, nb + li, acc[a][b], m_end, g.n);
             } else {
@@ -218,6 +226,7 @@ __global__ __launch_bounds__(256) void k_gemm_f32(FhGemm g) {
             for (int a = 0; a < 2; a++) {
                 const int nb = n0 + wn * 32 + a * 16;
                 if (EPI == FH_GEMM_ACT_T) gemm_store<EPI, float>(g.y, g.ldy, mb + gq * 4, nb + li, acc[a][b], m_end, g.n);
+                else if (EPI == FH_GEMM_RELU2) gemm_store<FH_GEMM_ACT, float>(g.y, g.ldy, mb + li, nb + gq * 4, relu2(acc[a][b]), m_end, g.n);
                 else gemm_store<EPI, float>(g.y, g.ldy, mb + li, nb + gq * 4, acc[a][b], m_end, g.n);
             }
         }
@@ -236,6 +245,7 @@ fh_status fh_gemm(fh_device *dev, int dtype, int epi, const FhGemm &g) {
     case FH_GEMM_F32: K_(FH_GEMM_F32)<<<GRID_, 256, 0, s>>>(g); break;      \
     case FH_GEMM_ACT: K_(FH_GEMM_ACT)<<<GRID_, 256, 0, s>>>(g); break;      \
     case FH_GEMM_ACT_T: K_(FH_GEMM_ACT_T)<<<GRID_, 256, 0, s>>>(g); break;  \
+    case FH_GEMM_RELU2: K_(FH_GEMM_RELU2)<<<GRID_, 256, 0, s>>>(g); break;  \
     default: K_(FH_GEMM_SWIGLU)<<<GRID_, 256, 0, s>>>(g); break;            \
     }
     if (dtype == FH_F32) {
@@ -401,6 +411,247 @@ fh_status fh_matvec_norm(fh_device *dev, const float *x, int k, const float *w, 
     if (rows == 4) k_matvec_norm<4><<<dim3((unsigned)tiles), 256, lds, dev->stream>>>(x, k, kp, w, eps, ms, norm_out);
     else if (rows == 2) k_matvec_norm<2><<<dim3((unsigned)tiles), 256, lds, dev->stream>>>(x, k, kp, w, eps, ms, norm_out);
     else k_matvec_norm<1><<<dim3((unsigned)tiles), 256, lds, dev->stream>>>(x, k, kp, w, eps, ms, norm_out);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+// ------------------------------------------------------------------------------ residual streams normed at a sublayer's end
+__global__ void k_group_tiles(int groups, int s, int tile_rows, FhTile *tiles, int *n_tiles) {
+    const int per = (s + tile_rows - 1) / tile_rows;
+    for (int i = threadIdx.x; i < groups * per; i += blockDim.x) {
+        const int g = i / per, r = i % per * tile_rows;
+        tiles[i] = FhTile{g, g * s + r, s - r < tile_rows ? s - r : tile_rows, 0};
+    }
+    if (threadIdx.x == 0) *n_tiles = groups * per;
+}
+
+fh_status fh_group_tiles(fh_device *dev, int groups, int s, int tile_rows, FhTile *tiles, int *n_tiles) {
+    k_group_tiles<<<1, 256, 0, dev->stream>>>(groups, s, tile_rows, tiles, n_tiles);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_add_normed(const float *__restrict__ x, const float *__restrict__ y, int k,
+                                                    const float *__restrict__ w, float eps, float *__restrict__ x_out,
+                                                    T *__restrict__ act, int kp) {
+    __shared__ float red[4];
+    const int64_t row = (int64_t)blockIdx.x * k;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < k; i += 256) ss = fmaf(y[row + i], y[row + i], ss);
+    ss = fh_wave_sum(ss);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+    __syncthreads();
+    const float inv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)k + eps);
+    for (int i = threadIdx.x; i < kp; i += 256) {
+        float v = 0.f;
+        if (i < k) x_out[row + i] = v = x[row + i] + y[row + i] * inv * w[i];
+        if (act) act[(int64_t)blockIdx.x * kp + i] = fh_to<T>(v);
+    }
+}
+
+fh_status fh_add_normed(fh_device *dev, int dtype, const float *x, const float *y, int rows, int k, const float *w, float eps,
+                        float *x_out, void *act, int kp) {
+    const dim3 grid((unsigned)rows);
+    if (dtype == FH_F32) k_add_normed<float><<<grid, 256, 0, dev->stream>>>(x, y, k, w, eps, x_out, (float *)act, kp);
+    else k_add_normed<uint16_t><<<grid, 256, 0, dev->stream>>>(x, y, k, w, eps, x_out, (uint16_t *)act, kp);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_embed_at(const uint16_t *__restrict__ table, int n, const uint16_t *__restrict__ pos_table,
+                                                  int positions, const uint32_t *__restrict__ ids, int pos,
+                                                  const int *__restrict__ pos_dev, int k, float *__restrict__ x, T *__restrict__ act, int kp) {
+    const int t = blockIdx.y, c = (int)blockIdx.x * 256 + threadIdx.x;
+    if (c >= kp) return;
+    const uint32_t id = ids[t];
+    int p = (pos_dev ? *pos_dev : pos) + t;
+    p = p < positions ? p : positions - 1; // the host refuses positions behind the table
+    float v = 0.f;
+    if (c < k) {
+        v = fh_bf_f32(table[(int64_t)(id < (uint32_t)n ? id : 0) * kp + c]);
+        if (pos_table) v += fh_bf_f32(pos_table[(int64_t)p * kp + c]);
+        x[(int64_t)t * k + c] = v;
+    }
+    if (act) act[(int64_t)t * kp + c] = fh_to<T>(v);
+}
+
+fh_status fh_embed_at(fh_device *dev, int dtype, const fh_qmatrix *table, const fh_qmatrix *pos_table, const uint32_t *ids, int s,
+                      int pos, const int *pos_dev, float *x, void *act, int kp) {
+    FH_REQUIRE(table->type == FH_BF16 && table->recs == kp && (!pos_table || (pos_table->type == FH_BF16 && pos_table->recs == kp)),
+               "embedding tables are bf16 rows of one stride");
+    const dim3 grid((unsigned)((kp + 255) / 256), (unsigned)s);
+    const uint16_t *tb = (const uint16_t *)table->data, *pt = pos_table ? (const uint16_t *)pos_table->data : nullptr;
+    const int n = (int)table->n, np = pos_table ? (int)pos_table->n : 1 << 30, k = (int)table->k;
+    if (dtype == FH_F32) k_embed_at<float><<<grid, 256, 0, dev->stream>>>(tb, n, pt, np, ids, pos, pos_dev, k, x, (float *)act, kp);
+    else k_embed_at<uint16_t><<<grid, 256, 0, dev->stream>>>(tb, n, pt, np, ids, pos, pos_dev, k, x, (uint16_t *)act, kp);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_token_shift(FhShift m, const float *__restrict__ x, int k, int pos,
+                                                     const float *__restrict__ state, int kp) {
+    const int t = blockIdx.y, c = (int)blockIdx.x * 256 + threadIdx.x;
+    if (c >= kp) return;
+    float v = 0.f, d = 0.f;
+    if (c < k) {
+        v = x[(int64_t)t * k + c];
+        d = (t > 0 ? x[(int64_t)(t - 1) * k + c] : pos > 0 ? state[((pos - 1) & 1) * k + c] : 0.f) - v;
+    }
+#pragma unroll
+    for (int n = 0; n < FH_SHIFT_MAX; n++) {
+        if (n >= m.n) break;
+        const float y = c < k ? fmaf(d, m.mu[n][c], v) : 0.f;
+        const int64_t o = (int64_t)t * kp + c;
+        if (m.f32[n]) ((float *)m.y[n])[o] = y;
+        else ((T *)m.y[n])[o] = fh_to<T>(y);
+    }
+}
+
+fh_status fh_token_shift(fh_device *dev, int dtype, const FhShift &m, const float *x, int s, int k, int pos, float *state, int kp) {
+    const dim3 grid((unsigned)((kp + 255) / 256), (unsigned)s);
+    if (dtype == FH_F32) k_token_shift<float><<<grid, 256, 0, dev->stream>>>(m, x, k, pos, state, kp);
+    else k_token_shift<uint16_t><<<grid, 256, 0, dev->stream>>>(m, x, k, pos, state, kp);
+    FH_HIP(hipGetLastError());
+    // after every reader of the old rows
+    return fh_copy(dev, state + (int64_t)((pos + s - 1) & 1) * k, x + (int64_t)(s - 1) * k, (size_t)k * 4);
+}
+
+// A workgroup takes 16 rows of x and 16 of W; its four wavefronts share out k.  True f32 products on the widened weights.
+__global__ __launch_bounds__(256) void k_low_rank_tanh(const float *__restrict__ x, int kp, int rows, const uint16_t *__restrict__ w, int n,
+                                                       float *__restrict__ y, int ldy) {
+    __shared__ float red[4][256];
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, li = lane & 15, g = lane >> 4, m0 = (int)blockIdx.x * 16, n0 = (int)blockIdx.y * 16;
+    const float *xp = x + (int64_t)(m0 + li < rows ? m0 + li : rows - 1) * kp + 8 * g;
+    const uint16_t *wp = w + (int64_t)(n0 + li < n ? n0 + li : n - 1) * kp + 8 * g;
+    fh_f4 acc = fh_f4{0.f, 0.f, 0.f, 0.f};
+    for (int k = 32 * wave; k < kp; k += 128) {
+        const uint4 u = *(const uint4 *)(wp + k);
+        const fh_f8 fw = {{fh_bf_lo(u.x), fh_bf_hi(u.x), fh_bf_lo(u.y), fh_bf_hi(u.y), fh_bf_lo(u.z), fh_bf_hi(u.z), fh_bf_lo(u.w), fh_bf_hi(u.w)}};
+        fh_f8 fx;
+        fh_frag_load(fx, xp + k);
+        acc = fh_mma32(fw, fx, acc); // a lane: W rows 4 g .. + 3 of x row li
+    }
+#pragma unroll
+    for (int e = 0; e < 4; e++) red[wave][lane * 4 + e] = acc[e];
+    __syncthreads();
+    const int r = m0 + (tid >> 2) % 16, c = n0 + 4 * (tid >> 6) + (tid & 3); // lane tid / 4, element tid % 4
+    const float v = (red[0][tid] + red[1][tid]) + (red[2][tid] + red[3][tid]);
+    if (r < rows && c < ldy) y[(int64_t)r * ldy + c] = c < n ? tanhf(v) : 0.f;
+}
+
+fh_status fh_low_rank_tanh(fh_device *dev, const float *x, int kp, int rows, const uint16_t *w, int n, float *y, int ldy) {
+    FH_REQUIRE(n > 0 && ldy >= n && kp % 64 == 0, "bad low-rank product");
+    k_low_rank_tanh<<<dim3((unsigned)((rows + 15) / 16), (unsigned)((ldy + 15) / 16)), 256, 0, dev->stream>>>(x, kp, rows, w, n, y, ldy);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+// As k_matvec_norm, with a workgroup of eight wavefronts: the input is worked out once per workgroup into the LDS.
+struct MvMixes { FhMvMix s[FH_MV_MAX]; int tiles[FH_MV_MAX]; int n; };
+
+template <int ROWS>
+__global__ __launch_bounds__(512) void k_matvec_mix(FhMvAdd in, int k, int kp, MvMixes segs) {
+    extern __shared__ __attribute__((aligned(16))) float xs[]; // [kp]
+    __shared__ float red[8];
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    int tile = blockIdx.x, si = 0;
+    while (si + 1 < segs.n && tile >= segs.tiles[si]) tile -= segs.tiles[si++];
+    const FhMvMix seg = segs.s[si];
+    const int row0 = (tile * 8 + wave) * ROWS;
+    const uint16_t *wr[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) wr[r] = seg.w + (int64_t)(row0 + r < seg.n ? row0 + r : seg.n - 1) * kp + lane * 8;
+    uint4 cur[ROWS]; // the first weights are requested before the input is worked out
+    const bool in0 = lane * 8 < kp;
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) cur[r] = in0 ? *(const uint4 *)wr[r] : uint4{0, 0, 0, 0};
+    float inv = 0.f;
+    if (in.y) {
+        float ss = 0.f;
+        for (int i = tid; i < k; i += 512) ss = fmaf(in.y[i], in.y[i], ss);
+        ss = fh_wave_sum(ss);
+        if (lane == 0) red[wave] = ss;
+        __syncthreads();
+        inv = 1.0f / sqrtf((((red[0] + red[1]) + (red[2] + red[3])) + ((red[4] + red[5]) + (red[6] + red[7]))) / (float)k + in.eps);
+    }
+    const int pos = in.state ? *in.pos_dev : 0;
+    const float *before = in.state + ((pos - 1) & 1) * k;
+    float *here = in.state + (pos & 1) * k;
+    for (int i = tid; i < kp; i += 512) {
+        float v = 0.f;
+        if (i < k) {
+            v = in.x[i];
+            if (in.y) v += in.y[i] * inv * in.w[i];
+            if (blockIdx.x == 0) {
+                if (in.x_out) in.x_out[i] = v;
+                if (in.state) here[i] = v;
+            }
+            if (seg.mu) v = fmaf((pos > 0 ? before[i] : 0.f) - v, seg.mu[i], v);
+        }
+        xs[i] = v;
+    }
+    __syncthreads();
+    float acc[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) acc[r] = 0.f;
+    for (int c = lane * 8; c < kp; c += 512) {
+        uint4 nxt[ROWS];
+        const bool more = c + 512 < kp;
+#pragma unroll
+        for (int r = 0; r < ROWS; r++) nxt[r] = more ? *(const uint4 *)(wr[r] + (c - lane * 8) + 512) : uint4{0, 0, 0, 0};
+        const float4 a = *(const float4 *)(xs + c), b = *(const float4 *)(xs + c + 4);
+#pragma unroll
+        for (int r = 0; r < ROWS; r++) {
+            acc[r] = fmaf(fh_bf_lo(cur[r].x), a.x, acc[r]);
+            acc[r] = fmaf(fh_bf_hi(cur[r].x), a.y, acc[r]);
+            acc[r] = fmaf(fh_bf_lo(cur[r].y), a.z, acc[r]);
+            acc[r] = fmaf(fh_bf_hi(cur[r].y), a.w, acc[r]);
+            acc[r] = fmaf(fh_bf_lo(cur[r].z), b.x, acc[r]);
+            acc[r] = fmaf(fh_bf_hi(cur[r].z), b.y, acc[r]);
+            acc[r] = fmaf(fh_bf_lo(cur[r].w), b.z, acc[r]);
+            acc[r] = fmaf(fh_bf_hi(cur[r].w), b.w, acc[r]);
+            cur[r] = nxt[r];
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) acc[r] = fh_wave_sum(acc[r]);
+    if (lane == 0)
+#pragma unroll
+        for (int r = 0; r < ROWS; r++)
+            if (row0 + r < seg.n) {
+                float v = acc[r];
+                if (seg.act == FH_MV_ACT_RELU2) v = fmaxf(v, 0.f) * fmaxf(v, 0.f);
+                else if (seg.act == FH_MV_ACT_TANH) v = tanhf(v);
+                seg.y[row0 + r] = v;
+            }
+}
+
+fh_status fh_matvec_mix(fh_device *dev, const FhMvAdd &in, int k, const FhMvMix *segs, int n_segs) {
+    FH_REQUIRE(n_segs >= 1 && n_segs <= FH_MV_MAX, "1 to %d matrices per launch", FH_MV_MAX);
+    FH_REQUIRE(in.x && in.x != in.x_out && (!in.y || in.w) && (!in.state || in.pos_dev), "bad input of a decode product");
+    const int kp = (int)fh_pad64(k);
+    MvMixes ms{};
+    int64_t total = 0;
+    for (int i = 0; i < n_segs; i++) total += segs[i].n;
+    const int rows = total >= (int64_t)dev->compute_units * 8 * 4 ? 4 : total >= (int64_t)dev->compute_units * 8 * 2 ? 2 : 1;
+    int tiles = 0;
+    ms.n = n_segs;
+    for (int i = 0; i < n_segs; i++) {
+        ms.s[i] = segs[i];
+        ms.tiles[i] = (segs[i].n + 8 * rows - 1) / (8 * rows);
+        tiles += ms.tiles[i];
+    }
+    const size_t lds = (size_t)kp * 4;
+    FH_REQUIRE(lds <= 120 * 1024, "k = %d too long for the matvec", k);
+    const void *fn = rows == 4 ? (const void *)k_matvec_mix<4> : rows == 2 ? (const void *)k_matvec_mix<2> : (const void *)k_matvec_mix<1>;
+    if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, fn, lds));
+    const dim3 grid((unsigned)tiles);
+    if (rows == 4) k_matvec_mix<4><<<grid, 512, lds, dev->stream>>>(in, k, kp, ms);
+    else if (rows == 2) k_matvec_mix<2><<<grid, 512, lds, dev->stream>>>(in, k, kp, ms);
+    else k_matvec_mix<1><<<grid, 512, lds, dev->stream>>>(in, k, kp, ms);
     FH_HIP(hipGetLastError());
     return FH_OK;
 }

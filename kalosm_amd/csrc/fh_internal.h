@@ -178,9 +178,11 @@ static inline int fh_rec_blocks(uint32_t t) {   // blocks per record (per row)
 }
 static inline int fh_rec_bytes(uint32_t t) { return 16 * fh_rec_blocks(t) * fh_block_bytes(t); }
 
-// An FH_BF16 matrix of zeros, and n rows of k values into it (interleave: row r goes to row0 + 32 (r / 16) + r % 16).
+// An FH_BF16 matrix of zeros, and n rows of k values into it, from column col0 on (interleave, whole rows only: row r goes to
+// row0 + 32 (r / 16) + r % 16).
 fh_status fh_qmatrix_alloc_bf16(fh_device *dev, int64_t n, int64_t k, fh_qmatrix **out);
-fh_status fh_qmatrix_put_bf16(fh_qmatrix *q, int64_t row0, int64_t n, int64_t k, const void *bytes, bool interleave);
+fh_status fh_qmatrix_put_bf16(fh_qmatrix *q, int64_t row0, int64_t n, int64_t k, const void *bytes, bool interleave,
+                              int64_t col0 = 0);
 
 // A plain-data view passed to kernels by value.
 struct QView {
@@ -241,7 +243,12 @@ struct fh_kvcache {
 size_t fh_dtype_size(int dtype);
 fh_status fh_kvcache_reserve(fh_kvcache *c, int required);
 // One layer of `row` elements per position (FH_F32, or 2 for bf16), a ring of at most max_len rows, no V plane.
+// keep > 0: positions below it stay in the row of their number and the ring is made of the rows behind them
+// (fh_ring_row), max_len rows altogether.
 fh_status fh_kvcache_create_ring(fh_device *dev, int row, int max_len, int dtype, fh_kvcache **out);
+// Row of position p of a ring of cap rows whose first `keep` are not part of the ring.  While the cache still grows
+// (cap below its final size) no position is behind its capacity, and the row is p.
+__host__ __device__ static inline int fh_ring_row(int p, int cap, int keep) { return p < cap ? p : keep + (p - keep) % (cap - keep); }
 // dense bf16 rows (fh_dense.hip): x f32 [m, k]
 fh_status fh_launch_bf16_matmul(const fh_qmatrix *q, const void *x, int x_is_bf16, int m, float *y);
 // append reading the write position from c->len_dev (graph friendly), s == 1

@@ -11,6 +11,7 @@
 // padded with zeros to multiples of 8.
 #pragma once
 #include "fh_recurrent.h"
+#include "fh_window_attn.h"
 
 struct FhLatent {
     int heads = 0, dn = 0, dr = 0, dv = 0, rank = 0;

@@ -225,12 +225,13 @@ fh_status fh_qmatrix_alloc_bf16(fh_device *dev, int64_t n, int64_t k, fh_qmatrix
     return FH_OK;
 }
 
-fh_status fh_qmatrix_put_bf16(fh_qmatrix *q, int64_t row0, int64_t n, int64_t k, const void *bytes, bool interleave) {
-    FH_REQUIRE(q && q->type == FH_BF16 && k == q->k && bytes && n > 0, "bad rows for a bf16 matrix");
+fh_status fh_qmatrix_put_bf16(fh_qmatrix *q, int64_t row0, int64_t n, int64_t k, const void *bytes, bool interleave, int64_t col0) {
+    FH_REQUIRE(q && q->type == FH_BF16 && bytes && n > 0, "bad rows for a bf16 matrix");
+    FH_REQUIRE(interleave ? k == q->k && col0 == 0 : col0 >= 0 && k > 0 && col0 + k <= q->k, "columns %lld .. of %lld", (long long)col0, (long long)q->k);
     const int64_t ld = q->recs, last = interleave ? row0 + 32 * ((n - 1) / 16) + (n - 1) % 16 : row0 + n - 1;
     FH_REQUIRE(row0 >= 0 && last < q->n, "rows %lld .. %lld of %lld", (long long)row0, (long long)last, (long long)q->n);
     hipStream_t s = q->dev->stream;
-    uint8_t *dst = q->data + (size_t)row0 * ld * 2;
+    uint8_t *dst = q->data + ((size_t)row0 * ld + (size_t)col0) * 2;
     if (!interleave) {
         FH_HIP(hipMemcpy2DAsync(dst, (size_t)ld * 2, bytes, (size_t)k * 2, (size_t)k * 2, (size_t)n, hipMemcpyHostToDevice, s));
     } else {

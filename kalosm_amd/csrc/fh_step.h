@@ -3,6 +3,7 @@
 // experts' gate and up products - and the output launch, which adds every down-stream product of the layer into the
 // residual stream:  x += W_o . mix + sum_j w_j D_(e_j) . a_j + D_s . a_s.
 #pragma once
+#include "fh_gqa.h"
 #include "fh_latent.h"
 #include "fh_moe.h"
 
@@ -29,3 +30,22 @@ struct FhStep {
 };
 fh_status fh_step_middle(fh_device *dev, int dtype, const FhStep &st, fh_kvcache *cache);
 fh_status fh_step_out(fh_device *dev, const FhStep &st);
+
+// A layer whose sublayers are normed at their end keeps them apart, each a chain of its own:
+//   projections (fh_matvec_mix: the sublayer before is normed and added on the way in) - fh_step_mixers: attention over parts
+//   of the cache beside the recurrence's step - fh_step_mix_out: merge of the parts, norm and gate of the recurrence -
+//   output projection (fh_matvec_mix) - feed-forward (twice fh_matvec_mix)
+// `act` is the input of the output projection: the attention's heads * vdim values padded to kpl with zeros, then the
+// recurrence's.
+struct FhMixStep {
+    int attn = 0, rec = 0;       // which mixers there are
+    FhGqa gqa;
+    FhRecurrent r;
+    FhRecState state;
+    const float *proj = nullptr; // this token's projection row
+    const int *pos_dev = nullptr;
+    float *part = nullptr, *o = nullptr, *act = nullptr;
+    int kpl = 0;
+};
+fh_status fh_step_mixers(fh_device *dev, int dtype, const FhMixStep &st, fh_kvcache *cache);
+fh_status fh_step_mix_out(fh_device *dev, const FhMixStep &st, const fh_kvcache *cache);

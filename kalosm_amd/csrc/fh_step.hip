@@ -46,7 +46,7 @@ __device__ __forceinline__ void rec_step(const FhStep &st, int b, float *lds) {
     __syncthreads();
     if (wave < 2) {
         float g = 1.f;
-        if (r.delta) {
+        if (r.delta()) {
             float ss = 0.f;
             for (int i = lane; i < d; i += 64) ss = fmaf(qk[wave * d + i], qk[wave * d + i], ss);
             g = 1.0f / sqrtf(fh_wave_sum(ss) + 1e-6f);
@@ -54,7 +54,7 @@ __device__ __forceinline__ void rec_step(const FhStep &st, int b, float *lds) {
         if (lane == 0) f[wave] = wave == 0 ? g * r.q_scale : g;
     }
     const float sp_ = fh_softplus_f(st.proj[r.col_a + h] + r.dt_bias[h]);
-    const float g = expf(-expf(r.a_log[h]) * sp_), be = r.delta ? fh_sigmoid_f(st.proj[r.col_b + h]) : sp_;
+    const float g = expf(-expf(r.a_log[h]) * sp_), be = r.delta() ? fh_sigmoid_f(st.proj[r.col_b + h]) : sp_;
     __syncthreads();
     const float v = vv[live ? wave * 4 + (lane >> 4) : 0];
     float k[RPT], dot = 0.f, o = 0.f;
@@ -64,7 +64,7 @@ __device__ __forceinline__ void rec_step(const FhStep &st, int b, float *lds) {
         S[i] *= g;
         dot = fmaf(S[i], k[i], dot);
     }
-    const float u = r.delta ? be * (v - fh_row16_sum(dot)) : be * v;
+    const float u = r.delta() ? be * (v - fh_row16_sum(dot)) : be * v;
 #pragma unroll
     for (int i = 0; i < RPT; i++) {
         S[i] = fmaf(k[i], u, S[i]);
@@ -330,6 +330,126 @@ fh_status fh_step_out(fh_device *dev, const FhStep &st) {
     FH_REQUIRE(lds <= 156 * 1024, "a decode step stages at most 156 KB of inputs (%zu bytes needed)", lds);
     if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)k_step_out, lds));
     k_step_out<<<dim3((unsigned)((st.width + 7) / 8)), 512, lds, dev->stream>>>(st, pieces);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+// ------------------------------------------------------------------------------ mixers of sublayers normed at their end
+// One step of a recurrence without a short convolution: workgroup b takes 16 columns of one head's state.
+template <int RPT>
+__device__ __forceinline__ void linear_step(const FhMixStep &st, int pos, int b, float *lds) {
+    const FhRecurrent &r = st.r;
+    const int tid = threadIdx.x, lane = tid & 63, rg = lane & 15, d = r.dim;
+    const int ncb = (r.vdim + 15) / 16, h = b / ncb, col = b % ncb * 16 + (tid >> 4), i0 = rg * RPT;
+    const bool live = col < r.vdim;
+    float *sp = st.state.s + ((int64_t)h * r.vdim + (live ? col : r.vdim - 1)) * d;
+    float S[RPT];
+#pragma unroll
+    for (int i = 0; i < RPT; i++) S[i] = pos > 0 && i0 + i < d ? sp[i0 + i] : 0.f;
+    const float *q = st.proj + r.col_q + h * d, *k = st.proj + r.col_k + h * d;
+    const float v = st.proj[r.col_v + h * r.vdim + (live ? col : r.vdim - 1)];
+    float o = 0.f;
+    if (r.kind == FH_REC_CHANNEL) {
+        float *g = lds, *t1 = lds + 256; // [d], [rp]
+        for (int i = tid; i < r.rp; i += 256) t1[i] = i < r.rank ? st.proj[r.col_a + i] : 0.f;
+        __syncthreads();
+        for (int c = tid >> 4; c < d; c += 16) {
+            float z = 0.f;
+            for (int i = rg * 8; i < r.rp; i += 128) z = dot8(*(const uint4 *)(r.w2 + (int64_t)(h * d + c) * r.rp + i), t1 + i, z);
+            z = fh_row16_sum(z);
+            if (rg == 0) g[c] = expf(fh_rec_la(z + r.w0[h * d + c]));
+        }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < RPT; i++)
+            if (i0 + i < d) {
+                const float kv = k[i0 + i] * v;
+                o = fmaf(fmaf(r.bonus[h * d + i0 + i], kv, S[i]), q[i0 + i], o);
+                S[i] = fmaf(S[i], g[i0 + i], kv);
+            }
+    } else {
+        const float g = expf(r.log_decay[h]), *ct = r.cos_t + (int64_t)pos * r.pairs, *sn = r.sin_t + (int64_t)pos * r.pairs;
+        float *qk = lds; // [2 d]
+        for (int i = tid; i < 2 * d; i += 256) {
+            const float *x = i < d ? q : k;
+            qk[i] = fh_rotated([&](int j) { return x[j]; }, i < d ? i : i - d, r.pairs, r.halves, ct, sn) * (i < d ? r.q_scale : r.k_scale);
+        }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < RPT; i++)
+            if (i0 + i < d) {
+                S[i] = fmaf(qk[d + i0 + i], v, S[i] * g);
+                o = fmaf(S[i], qk[i0 + i], o);
+            }
+    }
+    o = fh_row16_sum(o);
+#pragma unroll
+    for (int i = 0; i < RPT; i++)
+        if (live && i0 + i < d) sp[i0 + i] = S[i];
+    if (rg == 0 && live) st.o[h * r.vdim + col] = o;
+}
+
+template <typename T, int NP, int RPT>
+__global__ __launch_bounds__(256) void k_step_mixers(FhMixStep st, T *ring, int cap, int splits, int n_attn) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const int pos = *st.pos_dev;
+    if ((int)blockIdx.x < n_attn) fh_gqa_step<T, NP>(st.gqa, st.proj, ring, cap, pos, splits, blockIdx.x, st.part, lds);
+    else linear_step<RPT>(st, pos, (int)blockIdx.x - n_attn, lds);
+}
+
+template <typename T, int NP>
+static fh_status step_mixers_t(fh_device *dev, const FhMixStep &st, fh_kvcache *cache) {
+    const int splits = st.attn ? fh_gqa_splits(cache) : 1, n_attn = st.attn ? fh_gqa_blocks(st.gqa, splits) : 0;
+    const int n_rec = st.rec ? st.r.heads * ((st.r.vdim + 15) / 16) : 0, rpt = st.rec ? (st.r.dim + 15) / 16 : 1;
+    size_t lds = st.attn ? fh_gqa_lds(st.gqa) : 0;
+    const size_t need = !st.rec ? 0 : (size_t)(st.r.kind == FH_REC_CHANNEL ? 256 + st.r.rp : 2 * st.r.dim) * 4;
+    lds = lds > need ? lds : need;
+    FH_REQUIRE(lds <= 60 * 1024 && rpt <= 16, "mixers too wide for a decode step (%zu bytes of LDS)", lds);
+    const dim3 grid((unsigned)(n_attn + n_rec));
+    T *ring = cache ? (T *)cache->k : nullptr;
+    const int cap = cache ? cache->capacity : 1;
+    if (rpt <= 2) k_step_mixers<T, NP, 2><<<grid, 256, lds, dev->stream>>>(st, ring, cap, splits, n_attn);
+    else if (rpt <= 4) k_step_mixers<T, NP, 4><<<grid, 256, lds, dev->stream>>>(st, ring, cap, splits, n_attn);
+    else if (rpt <= 8) k_step_mixers<T, NP, 8><<<grid, 256, lds, dev->stream>>>(st, ring, cap, splits, n_attn);
+    else k_step_mixers<T, NP, 16><<<grid, 256, lds, dev->stream>>>(st, ring, cap, splits, n_attn);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
+fh_status fh_step_mixers(fh_device *dev, int dtype, const FhMixStep &st, fh_kvcache *cache) {
+    FH_REQUIRE(!st.attn || (cache && st.gqa.dnp <= 256 && st.gqa.dvp <= 256), "attention heads of a decode step have at most 256 dimensions");
+    const bool one = !st.attn || (st.gqa.dnp <= 128 && st.gqa.dvp <= 128);
+    if (dtype == FH_F32) return one ? step_mixers_t<float, 1>(dev, st, cache) : step_mixers_t<float, 2>(dev, st, cache);
+    return one ? step_mixers_t<uint16_t, 1>(dev, st, cache) : step_mixers_t<uint16_t, 2>(dev, st, cache);
+}
+
+// One wavefront per attention head, then one per norm group of the recurrence.
+__global__ __launch_bounds__(64) void k_step_mix_out(FhMixStep st, int splits) {
+    const int lane = threadIdx.x, na = st.attn ? st.gqa.heads : 0, b = blockIdx.x;
+    if (b < na) {
+        const FhGqa &a = st.gqa;
+        fh_gqa_merge(a, st.part, splits, b, st.act + b * a.vdim);
+        if (b == na - 1)
+            for (int i = a.heads * a.vdim + lane; i < st.kpl; i += 64) st.act[i] = 0.f;
+        return;
+    }
+    const FhRecurrent &r = st.r;
+    const int g = b - na, inner = r.heads * r.vdim, gl = inner / r.norm_groups;
+    const float *o = st.o + g * gl, *gate = st.proj + r.col_g + g * gl;
+    float ss = 0.f;
+    for (int i = lane; i < gl; i += 64) ss = fmaf(o[i], o[i], ss);
+    const float inv = 1.0f / sqrtf(fh_wave_sum(ss) / (float)gl + r.eps);
+    for (int i = lane; i < gl; i += 64) {
+        float v = o[i] * inv;
+        if (r.norm) v *= r.norm[r.norm_len == inner ? g * gl + i : i % r.norm_len];
+        st.act[st.kpl + g * gl + i] = v * fh_silu_f(gate[i]) * r.out_scale;
+    }
+}
+
+fh_status fh_step_mix_out(fh_device *dev, const FhMixStep &st, const fh_kvcache *cache) {
+    FH_REQUIRE(!st.rec || !st.r.gate_first, "this step gates behind the norm");
+    const int blocks = (st.attn ? st.gqa.heads : 0) + (st.rec ? st.r.norm_groups : 0);
+    k_step_mix_out<<<dim3((unsigned)blocks), 64, 0, dev->stream>>>(st, st.attn ? fh_gqa_splits(cache) : 1);
     FH_HIP(hipGetLastError());
     return FH_OK;
 }

@@ -25,7 +25,7 @@ def _hybrid(device: Device, path: str, dtype: str, ctx: int) -> Decoder:
     return HybridModel.open(device, path, dtype=dtype, ctx=ctx)
 
 
-ARCHITECTURES: Dict[str, Callable[[Device, str, str, int], Decoder]] = {"llama": _llama, "Fidasun": _hybrid}
+ARCHITECTURES: Dict[str, Callable[[Device, str, str, int], Decoder]] = {"llama": _llama, "Fidasun": _hybrid, "Zovovik": _hybrid}
 
 
 def architecture(path: str) -> str:
