@@ -1,5 +1,6 @@
 """Decoders whose configuration lists their layers one by one (csrc/fh_hybrid.hip): latent attention, gated delta rule and
-state space mixers, each with an optional mixture-of-experts feed-forward.  Weights are bf16 in a safetensors file beside
+state space mixers with an optional mixture-of-experts feed-forward (Fidasun); retention, and grouped-query attention beside
+time mixing, with an optional dense feed-forward (Zovovik).  Weights are bf16 in a safetensors file beside
 `config.json`."""
 from __future__ import annotations
 
@@ -51,7 +52,7 @@ class HybridModel(Decoder):
         """Random weights, generated tensor by tensor; `keep(name, values)` receives each as f32."""
         m = HybridModel(device, cfg, **kw)
         for name, n, k in synth.hybrid_tensor_specs(cfg):
-            bits = synth.hybrid_random_tensor(name, n, k, seed)
+            bits = synth.hybrid_random_tensor(name, n, k, seed, cfg["architecture"] == "Fidasun")
             m.load_tensor(name, synth.W_BF16, n, k, bits)
             if keep is not None:
                 keep(name, synth.from_bf16_bits(bits).reshape((n, k) if k else (n,)))

@@ -139,10 +139,14 @@ def llama_random_tensor(name: str, ty: int, n: int, k: int, seed: int, sigma: fl
 
 # ---------------------------------------------------------------------------------------------
 # Layer-list decoders (kalosm_amd.hybrid): tensor names and shapes from a configuration, random bf16 weights.
-def hybrid_tensor_specs(cfg: dict):
-    """[(name, n, k)]; k is 0 for vectors."""
+def hybrid_tensor_specs(cfg: dict, decay_rank: int = 0):
+    """[(name, n, k)]; k is 0 for vectors.  The low rank of the channel decays is no configuration value (0: a sixteenth of the
+    width, at most 64)."""
     D, V = cfg["width"], cfg["vocab"]
+    rank = decay_rank or min(64, max(1, D // 16))
     specs = [("embed", V, D), ("final.norm", D, 0), ("head", V, D)]
+    if cfg["architecture"] == "Zovovik":
+        specs.append(("pos", cfg["max_positions"], D))
     for i, layer in enumerate(cfg["layers"]):
         p, c = f"l{i}.", layer["mixer"]
         specs.append((p + "norm1", D, 0))
@@ -152,6 +156,19 @@ def hybrid_tensor_specs(cfg: dict):
             inner = H * dv
             specs += [(m + "q", H * (dn + dr), D), (m + "dkv", R + dr, D), (m + "dkv.norm", R, 0), (m + "uk", H * dn, R),
                       (m + "uv", H * dv, R), (m + "sink", H, 0)]
+        elif layer["type"] == "parallel":
+            a, r = c["left"], c["right"]
+            inner = a["heads"] * a["vdim"]
+            specs += [(m + "left.q", a["heads"] * a["dim"], D), (m + "left.k", a["kv_heads"] * a["dim"], D),
+                      (m + "left.v", a["kv_heads"] * a["vdim"], D), (m + "left.q.norm", a["dim"], 0), (m + "left.k.norm", a["dim"], 0),
+                      (m + "left.sink", a["heads"], 0), (m + "left.o", D, inner)]
+            m, inner = m + "right.", r["heads"] * r["dim"]
+            specs += [(m + "mu." + n, D, 0) for n in "rkvgw"] + [(m + n, inner, D) for n in "rkvg"]
+            specs += [(m + "w1", rank, D), (m + "w2", inner, rank), (m + "w0", inner, 0), (m + "u", r["heads"], r["dim"]),
+                      (m + "norm", inner, 0)]
+        elif layer["type"] == "retention":
+            inner = c["heads"] * c["vdim"]
+            specs += [(m + "q", c["heads"] * c["dim"], D), (m + "k", c["heads"] * c["dim"], D), (m + "v", inner, D), (m + "g", inner, D)]
         elif layer["type"] == "delta":
             H, nq, taps = c["heads"], c["kv_heads"] * c["dim"], c["conv"]
             inner = H * c["vdim"]
@@ -165,7 +182,9 @@ def hybrid_tensor_specs(cfg: dict):
                       (m + "dt_bias", H, 0), (m + "A_log", H, 0), (m + "D", H, 0), (m + "norm", inner, 0)]
         specs.append((m + "o", D, inner))
         mlp = layer.get("mlp")
-        if mlp:
+        if mlp and cfg["architecture"] == "Zovovik":
+            specs += [(p + "norm2", D, 0), (p + "mlp.up", mlp["ff"], D), (p + "mlp.down", D, mlp["ff"])]
+        elif mlp:
             f = p + "mlp."
             parts = [(f"e{e}", mlp["expert"]["ff"]) for e in range(mlp["router"]["experts"])]
             if mlp.get("shared"):
@@ -176,17 +195,25 @@ def hybrid_tensor_specs(cfg: dict):
     return specs
 
 
-def hybrid_random_tensor(name: str, n: int, k: int, seed: int) -> np.ndarray:
+def hybrid_random_tensor(name: str, n: int, k: int, seed: int, one_plus: bool = True) -> np.ndarray:
     """Deterministic bf16 bit patterns: rows of matrices with a norm near one, decays and step sizes spread over useful
-    ranges, norm weights away from their neutral value."""
+    ranges, norm weights away from their neutral value (`one_plus`: those of layers are distances from one)."""
     rng = np.random.default_rng(_name_seed(name, seed))
     last = name.rsplit(".", 1)[-1]
     if last == "A_log":
         x = rng.uniform(-3.0, 1.0, n)
     elif last == "dt_bias":
         x = rng.uniform(-3.0, 0.5, n)
-    elif last in ("norm1",) or name == "final.norm":
-        x = 0.2 * rng.standard_normal(n)
+    elif last in ("norm1", "norm2") or name == "final.norm":
+        x = (0.0 if one_plus else 1.0) + 0.2 * rng.standard_normal(n)
+    elif last == "w0":
+        x = rng.uniform(-6.0, 1.0, n)
+    elif last == "u":
+        x = 0.7 * rng.standard_normal((n, k))
+    elif ".mu." in name:
+        x = rng.uniform(0.0, 1.0, n)
+    elif name == "pos":
+        x = 0.3 * rng.standard_normal((n, k), np.float32)
     elif last in ("norm", "D"):
         x = 1.0 + 0.2 * rng.standard_normal(n)
     elif last in ("sink", "b") and k == 0:

@@ -38,6 +38,29 @@ def moe(experts=5, top=3, ff=56, shared=72, scale=1.7):
     return m
 
 
+def attention(heads=6, kv_heads=3, dim=20, vdim=12, window=19, keep=5, dims=14, base=5000.0, scale=0.31):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "rot": {"base": base, "dims": dims},
+            "mask": {"size": window, "keep_first": keep}}
+
+
+def pair(left=None, right=None, scales=(0.7, 1.6)):
+    return {"type": "parallel", "mixer": {"left": left or attention(), "right": right or {"heads": 5, "dim": 24},
+                                          "left_scale": scales[0], "right_scale": scales[1]}}
+
+
+def retention(heads=3, dim=28, vdim=40, dims=20, base=900.0, decay=None):
+    return {"type": "retention", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "rot": {"base": base, "dims": dims},
+                                           "decay": decay or [1.0 - 0.5 ** (2 + 3 * i) for i in range(heads)]}}
+
+
+def dense(ff=90):
+    return {"kind": "dense", "ff": ff}
+
+
+def config_apart(layers, width=150, vocab=110, eps=3e-6, positions=700):
+    return {"architecture": "Zovovik", "width": width, "vocab": vocab, "max_positions": positions, "norm": {"eps": eps}, "layers": layers}
+
+
 def config(layers, width=200, vocab=130, eps=1e-5):
     return {"architecture": "Fidasun", "width": width, "vocab": vocab, "norm": {"eps": eps}, "layers": layers}
 
@@ -61,6 +84,19 @@ CONFIGS = {
     "large": config([with_mlp(latent(heads=2, dim=128, rot_dim=64, vdim=128, kv_rank=512, window=70), moe(4, 2, 112, 80)),
                      with_mlp(delta(4, 2, 128, 128, 4), moe(4, 2, 112, 80)), with_mlp(mamba2(4, 64, 128, 2, 2, 4), None),
                      with_mlp(delta(2, 1, 200, 72, 4), None)], width=256, vocab=200),
+    # sublayers normed at their end: sizes that divide nothing, every order of mixers, layers without a feed-forward
+    "apart": config_apart([with_mlp(retention(), dense()), with_mlp(pair(), dense(77)), with_mlp(retention(1, 10, 9, 4), None),
+                           with_mlp(pair(attention(4, 1, 9, 30, 40, 3, 4, scale=0.5), {"heads": 2, "dim": 40}, (1.3, 0.4)), None)]),
+    "apart_ones": config_apart([with_mlp(pair(attention(1, 1, 2, 1, 1, 1, 2), {"heads": 1, "dim": 2}, (1.0, 1.0)), dense(1)),
+                                with_mlp(retention(1, 2, 1, 2, decay=[0.5]), dense(3))], width=64, vocab=40, eps=1e-3),
+    # a window nothing falls out of, no kept tokens
+    "apart_full": config_apart([with_mlp(pair(attention(4, 4, 16, 48, 5000, 0, 16), {"heads": 3, "dim": 16}), dense(128)),
+                                with_mlp(pair(attention(5, 5, 48, 16, 3, 0, 10), {"heads": 1, "dim": 100}), dense(64))], width=128, vocab=96),
+    # head sizes of large models
+    "apart_large": config_apart([with_mlp(pair(attention(8, 1, 128, 128, 70, 9, 96, scale=0.08), {"heads": 2, "dim": 128}), dense(320)),
+                                 with_mlp(pair(attention(2, 1, 200, 250, 33, 40, 200, scale=0.07), {"heads": 1, "dim": 200}), dense(112)),
+                                 with_mlp(retention(2, 256, 128, 256, decay=[0.999, 0.9]), None),
+                                 with_mlp(retention(3, 128, 72, 64), dense(200))], width=256, vocab=200),
     # values wider than one block of the attention kernel, latent rows beyond 640
     "wide": config([with_mlp(latent(heads=3, dim=96, rot_dim=32, vdim=160, kv_rank=640, window=37), None)], width=128, vocab=64),
 }
@@ -70,7 +106,7 @@ def weights(cfg, seed=0):
     """{name: f32 array} of bf16 values."""
     out = {}
     for name, n, k in synth.hybrid_tensor_specs(cfg):
-        out[name] = synth.from_bf16_bits(synth.hybrid_random_tensor(name, n, k, seed)).reshape((n, k) if k else (n,))
+        out[name] = synth.from_bf16_bits(synth.hybrid_random_tensor(name, n, k, seed, cfg["architecture"] == "Fidasun")).reshape((n, k) if k else (n,))
     return out
 
 
@@ -124,6 +160,23 @@ def matching_latent(cfg, w, layer, gain, pairs):
     uk[:, np.arange(dn), np.arange(dn)] = 1.0
     w[p + "uk"] = round_bf16(uk.reshape(H * dn, R))
     w[p + "uv"] = round_bf16(w[p + "uv"] * 2.0)
+    return w
+
+
+def matching_attention(cfg, w, layer, gain, pairs):
+    """The same for grouped-query attention beside time mixing: queries are `gain` times unit keys of their partners; rotated
+    dimensions, positions and the other mixer stay out of it."""
+    c, p = cfg["layers"][layer]["mixer"]["left"], f"l{layer}.mix.left."
+    d, dims, D = c["dim"], c["rot"]["dims"], cfg["width"]
+    A = np.random.default_rng(5).standard_normal((d, D)) / np.sqrt(D)
+    A[:dims] = 0.0
+    w["pos"][:] = 0.0
+    for x, y in pairs:
+        w["embed"][y] = np.roll(w["embed"][x], 1)
+    w[p + "q"] = round_bf16(np.tile(np.roll(A, -1, axis=1), (c["heads"], 1)))
+    w[p + "k"] = round_bf16(np.tile(A, (c["kv_heads"], 1)))
+    w[p + "q.norm"][:] = gain
+    w[p + "k.norm"][:] = 1.0
     return w
 
 

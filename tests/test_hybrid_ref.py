@@ -172,3 +172,88 @@ def test_unknown_architectures_are_refused(tmp_path):
     assert registry.architecture(str(tmp_path)) == "Nothing"
     with pytest.raises(ValueError, match="unknown architecture"):
         registry.load(None, str(tmp_path))
+
+
+# ------------------------------------------------------------------ sublayers normed at their end
+def test_rotated_halves_are_complex_products():
+    f, _ = R.yarn_frequencies(50.0, 6)
+    x = rng.standard_normal((5, 9))
+    y = R.rotated_halves(x, np.arange(5), f)
+    z = (x[:, :3] + 1j * x[:, 3:6]) * np.exp(1j * np.arange(5)[:, None] * f)
+    assert np.allclose(y[:, :3], z.real, atol=1e-6) and np.allclose(y[:, 3:6], z.imag, atol=1e-6)
+    assert np.array_equal(y[:, 6:], x[:, 6:])
+
+
+def test_kept_window_by_counting():
+    v = R.kept_window(12, 3, 2)
+    for i in range(12):
+        assert set(np.flatnonzero(v[i])) == {j for j in range(i + 1) if j > i - 3 or j in (0, 1)}
+    assert np.array_equal(R.kept_window(6, 6, 0), np.tri(6, dtype=bool))
+
+
+def test_grouped_attention_head_by_head():
+    cfg = G.config_apart([G.with_mlp(G.pair(G.attention(window=4, keep=2)), None)])
+    c, D = cfg["layers"][0]["mixer"]["left"], cfg["width"]
+    w = {k[len("l0.mix.left."):]: v.astype(np.float64) for k, v in G.weights(cfg).items() if k.startswith("l0.mix.left.")}
+    h = rng.standard_normal((10, D))
+    got = R.grouped_attention(h, w, c, 1e-4)
+    H, d, dv, rep = c["heads"], c["dim"], c["vdim"], c["heads"] // c["kv_heads"]
+    f = np.array([c["rot"]["base"] ** (-2.0 * i / c["rot"]["dims"]) for i in range(c["rot"]["dims"] // 2)])
+
+    def turned(x, p, weight):
+        x = x / np.sqrt((x @ x) / d + 1e-4) * weight
+        z = (x[0:2 * len(f):2] + 1j * x[1:2 * len(f):2]) * np.exp(1j * np.float64(p) * f)
+        return np.concatenate([np.stack([z.real, z.imag], 1).reshape(-1), x[2 * len(f):]])
+
+    out = np.zeros((10, H * dv))
+    for i in range(10):
+        for n in range(H):
+            g = n // rep
+            q = turned((w["q"] @ h[i])[n * d:(n + 1) * d], i, w["q.norm"])
+            den, num = np.exp(w["sink"][n]), np.zeros(dv)
+            for j in range(i + 1):
+                if i - j < 4 or j < 2:
+                    e = np.exp(q @ turned((w["k"] @ h[j])[g * d:(g + 1) * d], j, w["k.norm"]) * c["scale"])
+                    den, num = den + e, num + e * (w["v"] @ h[j])[g * dv:(g + 1) * dv]
+            out[i, n * dv:(n + 1) * dv] = num / den
+    assert np.allclose(got, out @ w["o"].T, atol=1e-5)
+
+
+def test_fixed_decay_is_a_masked_product():
+    q, k, v = (rng.standard_normal((9, n)) for n in (4, 4, 3))
+    t = np.arange(9)
+    m = np.where(t[:, None] >= t[None, :], 0.8 ** (t[:, None] - t[None, :]).astype(float), 0.0)
+    assert np.allclose(R.fixed_decay(q, k, v, 0.8), (q @ k.T * m) @ v)
+
+
+def test_channel_decay_term_by_term():
+    r, k, g = rng.standard_normal((7, 4)), rng.standard_normal((7, 4)), rng.uniform(0.1, 1.0, (7, 4))
+    v, u = rng.standard_normal((7, 3)), rng.standard_normal(4)
+    want = np.zeros((7, 3))
+    for t in range(7):
+        want[t] += (r[t] * u * k[t]).sum() * v[t]
+        for s in range(t):  # forgotten at every token between the two
+            want[t] += (r[t] * k[s] * np.prod(g[s + 1:t], axis=0)).sum() * v[s]
+    assert np.allclose(R.channel_decay(r, k, v, g, u), want)
+    same = R.channel_decay(r, k, v, np.full((7, 4), 0.5), np.ones(4))
+    assert np.allclose(same[1:] - (r * k).sum(1)[1:, None] * v[1:], R.fixed_decay(r[1:], k[:-1], v[:-1], 0.5))
+
+
+def test_shift_reads_zeros_ahead_of_the_first_token():
+    h, mu = rng.standard_normal((4, 5)), rng.uniform(0, 1, 5)
+    y = R.shifted(h, mu)
+    assert np.allclose(y[0], h[0] * (1 - mu)) and np.allclose(y[2], h[2] * (1 - mu) + h[1] * mu)
+
+
+def test_output_norm_layers_add_unit_vectors():
+    """Whatever the scale of a sublayer's matrices, what joins the residual stream has the norm weight's root mean square."""
+    cfg = G.config_apart([G.with_mlp(G.retention(), G.dense())], eps=1e-12)
+    w = G.weights(cfg)
+    w["l0.norm1"][:], w["l0.norm2"][:] = 3.0, 2.0
+    toks = rng.integers(0, cfg["vocab"], 6)
+    bare, layers = R.forward(dict(cfg, layers=[dict(cfg["layers"][0], mlp=None)]), w, toks)
+    x0 = w["embed"][toks] + w["pos"][:6]
+    assert np.allclose(np.sqrt(np.mean((layers[0] - x0) ** 2, axis=1)), 3.0, rtol=1e-6)
+    w["l0.mlp.up"] *= 7.0
+    full, both = R.forward(cfg, w, toks)
+    assert np.allclose(np.sqrt(np.mean((both[0] - layers[0]) ** 2, axis=1)), 2.0, rtol=1e-6)
