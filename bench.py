@@ -466,7 +466,8 @@ def main() -> int:
                     help="skip the launch-floor calibration (an empty kernel and plain streaming reads of the matrices' sizes)")
     ap.add_argument("--hybrid", action="store_true",
                     help="instead of the default workload: prefill and decode of layer-list decoders beside the Llama decoder")
-    ap.add_argument("--hybrid-only", default="", help="one size of --hybrid (w2048, w4096)")
+    ap.add_argument("--zovovik", action="store_true", help="as --hybrid, with the Zovovik design beside the two")
+    ap.add_argument("--hybrid-only", default="", help="one size of --hybrid / --zovovik (w2048, w4096)")
     ap.add_argument("--calib-copy", action="store_true", help="append 4 device copies of 256 MiB (counter calibration)")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -479,12 +480,12 @@ def main() -> int:
 
     dev = Device.gpu(0)
     info = dev.info()
-    if args.hybrid:
+    if args.hybrid or args.zovovik:
         from kalosm_amd import bench_hybrid
 
         dev.set_option("step_eager", int(args.no_graph))
         print(json.dumps({"metric": "prefill and decode of layer-list decoders beside the Llama decoder", "n_gpus": 1,
-                          "data": "synthetic", "device": info["name"], "hybrid": bench_hybrid.run(dev, only=args.hybrid_only)}))
+                          "data": "synthetic", "device": info["name"], "hybrid": bench_hybrid.run(dev, only=args.hybrid_only, zovovik=args.zovovik)}))
         return 0
     m = args.m
     ty = synth.Q4_K

@@ -1,5 +1,6 @@
 """Prefill and decode throughput of layer-list decoders at layer sizes of real models (random weights), beside the Llama
-decoder at equal width, depth and active feed-forward length (`bench.py --hybrid`)."""
+decoder at equal width, depth and active feed-forward length (`bench.py --hybrid`: Fidasun; `bench.py --zovovik`: Zovovik,
+beside Fidasun as well)."""
 from __future__ import annotations
 
 import statistics
@@ -29,6 +30,19 @@ def config(width: int, heads: int, experts: int, top: int, ff: int, window: int,
             "layers": [dict(l, mlp=mlp) for l in (latent, delta, latent, mamba)]}
 
 
+def zovovik_config(width: int, heads: int, ff: int, window: int, vocab: int = 32768) -> dict:
+    """Four layers: attention beside time mixing, retention, and the same again, all with a dense feed-forward."""
+    left = {"heads": heads, "kv_heads": heads // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "rot": {"base": 500000.0, "dims": 128},
+            "mask": {"size": window, "keep_first": 64}}
+    pair = {"type": "parallel", "mixer": {"left": left, "right": {"heads": width // 64, "dim": 64}, "left_scale": 1.0, "right_scale": 1.0}}
+    ret = {"type": "retention", "mixer": {"heads": width // 256, "dim": 256, "vdim": 256, "rot": {"base": 10000.0, "dims": 256},
+                                          "decay": [1.0 - 2.0 ** (-5 - 0.5 * i) for i in range(width // 256)]}}
+    return {"architecture": "Zovovik", "width": width, "vocab": vocab, "max_positions": 8192, "norm": {"eps": 1e-6},
+            "layers": [dict(l, mlp={"kind": "dense", "ff": ff}) for l in (pair, ret, pair, ret)]}
+
+
+ZOVOVIK = {"w2048": dict(width=2048, heads=16, ff=8192, window=1024), "w4096": dict(width=4096, heads=32, ff=14336, window=4096)}
+
 SIZES = {"w2048": dict(width=2048, heads=16, experts=64, top=6, ff=1024, window=1024, groups=2),
          "w4096": dict(width=4096, heads=32, experts=32, top=4, ff=2048, window=4096, groups=8)}
 
@@ -42,7 +56,7 @@ def matrix_flops(c: dict, tokens: int) -> float:
     """Multiply-adds x 2 of the weight matrices of a prompt (routed experts: the chosen ones), without the head."""
     f = 0.0
     for name, n, k in synth.hybrid_tensor_specs(c):
-        if not k or name in ("embed", "head") or name.endswith("conv"):
+        if not k or name in ("embed", "head", "pos") or name.endswith("conv") or name.endswith(".u"):
             continue
         part = name.split(".")
         if len(part) > 2 and part[1] == "mlp" and part[2].startswith("e") and part[2][1:].isdigit():
@@ -62,7 +76,7 @@ def _model(dev, c: dict) -> HybridModel:
             part = name.split(".")
             key = (part[-1], n, k) if len(part) == 4 and part[1] == "mlp" else name
             if key not in cache:
-                bits = synth.hybrid_random_tensor(name, n, k, 1)
+                bits = synth.hybrid_random_tensor(name, n, k, 1, c["architecture"] == "Fidasun")
                 if key == name:
                     yield name, n, k, bits
                     continue
@@ -85,7 +99,7 @@ def _measure(m, prompt, steps: int, repeats: int):
     return statistics.median(pre[1:]), statistics.median(dec[1:])
 
 
-def run(dev, prompts=(512, 2048), steps: int = 64, repeats: int = 5, only: str = "") -> dict:
+def run(dev, prompts=(512, 2048), steps: int = 64, repeats: int = 5, only: str = "", zovovik: bool = False) -> dict:
     out = {}
     for name, s in SIZES.items():
         if only and name != only:
@@ -95,8 +109,13 @@ def run(dev, prompts=(512, 2048), steps: int = 64, repeats: int = 5, only: str =
         rng = np.random.default_rng(1)
         res = {"config": s, "layers": [l["type"] for l in c["layers"]], "llama": {k: lc[k] for k in ("n_heads", "n_kv_heads", "ffn")},
                "dtype": {"Fidasun": "bf16 weights", "llama": "Q4_K_M weights"}, "runs": []}
-        models = {"Fidasun": _model(dev, c),
-                  "llama": Model.random_init(dev, lc, seed=1, sigma=1e-4)}
+        models, configs = {"Fidasun": _model(dev, c)}, {"Fidasun": c}
+        if zovovik:
+            configs["Zovovik"] = zovovik_config(**ZOVOVIK[name])
+            models["Zovovik"] = _model(dev, configs["Zovovik"])
+            res["dtype"]["Zovovik"], res["zovovik"] = "bf16 weights", ZOVOVIK[name]
+            res["zovovik_layers"] = [l["type"] for l in configs["Zovovik"]["layers"]]
+        models["llama"] = Model.random_init(dev, lc, seed=1, sigma=1e-4)
         for n in prompts:
             prompt = rng.integers(0, c["vocab"], n)
             for kind, m in models.items():
@@ -105,8 +124,8 @@ def run(dev, prompts=(512, 2048), steps: int = 64, repeats: int = 5, only: str =
                 r = {"model": kind, "prompt": n, "prefill_ms": round(pre * 1e3, 3), "prefill_tok_per_s": round(n / pre, 1),
                      "decode_ms": round(dec, 4), "decode_tok_per_s": round(1e3 / dec, 1), "weight_bytes_per_token": wb,
                      "decode_frac_hbm_peak": round(wb / (dec * 1e-3) / HBM_PEAK, 4)}
-                if kind == "Fidasun":
-                    fl = matrix_flops(c, n)
+                if kind in configs:
+                    fl = matrix_flops(configs[kind], n)
                 else:
                     D, H, K, F = lc["d_model"], lc["n_heads"] * 128, lc["n_kv_heads"] * 128, lc["ffn"]
                     fl = 2.0 * n * lc["n_layers"] * (D * (H + 2 * K) + H * D + 3 * D * F)
