@@ -130,6 +130,7 @@ fh_status fh_token_shift(fh_device *dev, int dtype, const FhShift &m, const floa
 
 // Decode: x' = x + y / rms(y) * w (y NULL: x), then up to FH_MV_MAX matrices on mixtures of x' (mu NULL: x' itself).  One
 // workgroup stores x' (x_out, not x) and, with a state, the row of this position.
+// With a gate: x' = x / rms(x) * w * silu(gate) * scale, the norm over `groups` equal groups of x (w NULL: without).
 enum { FH_MV_ACT_NONE = 0, FH_MV_ACT_RELU2 = 1, FH_MV_ACT_TANH = 2, FH_MV_MAX = 6 };
 struct FhMvMix { const uint16_t *w; const float *mu; float *y; int n, act; };
 struct FhMvAdd {
@@ -138,6 +139,9 @@ struct FhMvAdd {
     float *x_out = nullptr;
     float *state = nullptr;       // [2][k]
     const int *pos_dev = nullptr;
+    const float *gate = nullptr;
+    int groups = 0, w_len = 0;
+    float scale = 1.f;
 };
 fh_status fh_matvec_mix(fh_device *dev, const FhMvAdd &in, int k, const FhMvMix *segs, int n_segs);
 

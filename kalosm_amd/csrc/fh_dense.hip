@@ -435,18 +435,37 @@ template <typename T>
 __global__ __launch_bounds__(256) void k_add_normed(const float *__restrict__ x, const float *__restrict__ y, int k,
                                                     const float *__restrict__ w, float eps, float *__restrict__ x_out,
                                                     T *__restrict__ act, int kp) {
+    constexpr int R = 16; // values of a thread that are requested at once; longer rows are read twice
     __shared__ float red[4];
     const int64_t row = (int64_t)blockIdx.x * k;
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < k; i += 256) ss = fmaf(y[row + i], y[row + i], ss);
+    float xv[R], yv[R], wv[R], ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < R; j++) {
+        const int i = threadIdx.x + 256 * j;
+        const bool ok = i < k;
+        yv[j] = ok ? y[row + i] : 0.f;
+        xv[j] = ok ? x[row + i] : 0.f;
+        wv[j] = ok ? w[i] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < R; j++) ss = fmaf(yv[j], yv[j], ss);
+    for (int i = threadIdx.x + 256 * R; i < k; i += 256) ss = fmaf(y[row + i], y[row + i], ss);
     ss = fh_wave_sum(ss);
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
     __syncthreads();
     const float inv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)k + eps);
-    for (int i = threadIdx.x; i < kp; i += 256) {
+    T *ar = act + (int64_t)blockIdx.x * kp;
+#pragma unroll
+    for (int j = 0; j < R; j++) {
+        const int i = threadIdx.x + 256 * j;
+        const float v = xv[j] + yv[j] * inv * wv[j];
+        if (i < k) x_out[row + i] = v;
+        if (act && i < kp) ar[i] = fh_to<T>(v); // zeros from k on
+    }
+    for (int i = threadIdx.x + 256 * R; i < kp; i += 256) {
         float v = 0.f;
         if (i < k) x_out[row + i] = v = x[row + i] + y[row + i] * inv * w[i];
-        if (act) act[(int64_t)blockIdx.x * kp + i] = fh_to<T>(v);
+        if (act) ar[i] = fh_to<T>(v);
     }
 }
 
@@ -549,71 +568,160 @@ fh_status fh_low_rank_tanh(fh_device *dev, const float *x, int kp, int rows, con
     return FH_OK;
 }
 
-// As k_matvec_norm, with a workgroup of eight wavefronts: the input is worked out once per workgroup into the LDS.
+// A workgroup of eight wavefronts works its input out once, into the LDS; one wavefront per ROWS weight rows, a lane takes
+// eight consecutive weights (16 bytes) of every 512.  The first AHEAD pieces of 512 are requested before the input, later ones
+// while earlier ones are multiplied.
 struct MvMixes { FhMvMix s[FH_MV_MAX]; int tiles[FH_MV_MAX]; int n; };
 
-template <int ROWS>
-__global__ __launch_bounds__(512) void k_matvec_mix(FhMvAdd in, int k, int kp, MvMixes segs) {
-    extern __shared__ __attribute__((aligned(16))) float xs[]; // [kp]
-    __shared__ float red[8];
+__device__ __forceinline__ float mv_sum8(const float *red) {
+    return ((red[0] + red[1]) + (red[2] + red[3])) + ((red[4] + red[5]) + (red[6] + red[7]));
+}
+
+// x' into the LDS, mixed with the token before it where the matrix wants that.
+__device__ __forceinline__ void mv_input(const FhMvAdd &in, const float *mu, int k, int kp, float *xs, float *red) {
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-    int tile = blockIdx.x, si = 0;
-    while (si + 1 < segs.n && tile >= segs.tiles[si]) tile -= segs.tiles[si++];
-    const FhMvMix seg = segs.s[si];
-    const int row0 = (tile * 8 + wave) * ROWS;
-    const uint16_t *wr[ROWS];
+    const int pos = in.state ? *in.pos_dev : 0;
+    const float *before = in.state + ((pos - 1) & 1) * k;
+    float *here = in.state + (pos & 1) * k;
+    const bool one = blockIdx.x == 0, shift = mu && pos > 0;
+    if (!(k & 3) && k <= 4096) { // everything is requested at once
+        float4 x[2], y[2], w[2], m[2], b[2];
+        const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+        float ss = 0.f;
 #pragma unroll
-    for (int r = 0; r < ROWS; r++) wr[r] = seg.w + (int64_t)(row0 + r < seg.n ? row0 + r : seg.n - 1) * kp + lane * 8;
-    uint4 cur[ROWS]; // the first weights are requested before the input is worked out
-    const bool in0 = lane * 8 < kp;
+        for (int j = 0; j < 2; j++) {
+            const int i = (tid + 512 * j) * 4;
+            const bool ok = i < k;
+            x[j] = ok ? *(const float4 *)(in.x + i) : zero;
+            y[j] = ok && in.y ? *(const float4 *)(in.y + i) : zero;
+            w[j] = ok && in.y ? *(const float4 *)(in.w + i) : zero;
+            m[j] = ok && mu ? *(const float4 *)(mu + i) : zero;
+            b[j] = ok && shift ? *(const float4 *)(before + i) : zero;
+        }
+        float inv = 0.f;
+        if (in.y) {
 #pragma unroll
-    for (int r = 0; r < ROWS; r++) cur[r] = in0 ? *(const uint4 *)wr[r] : uint4{0, 0, 0, 0};
+            for (int j = 0; j < 2; j++) ss = fmaf(y[j].x, y[j].x, fmaf(y[j].y, y[j].y, fmaf(y[j].z, y[j].z, fmaf(y[j].w, y[j].w, ss))));
+            ss = fh_wave_sum(ss);
+            if (lane == 0) red[wave] = ss;
+            __syncthreads();
+            inv = 1.0f / sqrtf(mv_sum8(red) / (float)k + in.eps);
+        }
+#pragma unroll
+        for (int j = 0; j < 2; j++) {
+            const int i = (tid + 512 * j) * 4;
+            if (i >= kp) break;
+            float4 v = x[j];
+            if (in.y) v = make_float4(v.x + y[j].x * inv * w[j].x, v.y + y[j].y * inv * w[j].y, v.z + y[j].z * inv * w[j].z, v.w + y[j].w * inv * w[j].w);
+            if (one && i < k) {
+                if (in.x_out) *(float4 *)(in.x_out + i) = v;
+                if (in.state) *(float4 *)(here + i) = v;
+            }
+            if (mu)
+                v = make_float4(fmaf(b[j].x - v.x, m[j].x, v.x), fmaf(b[j].y - v.y, m[j].y, v.y), fmaf(b[j].z - v.z, m[j].z, v.z),
+                                fmaf(b[j].w - v.w, m[j].w, v.w));
+            *(float4 *)(xs + i) = v;
+        }
+        return;
+    }
     float inv = 0.f;
     if (in.y) {
         float ss = 0.f;
+#pragma unroll 4
         for (int i = tid; i < k; i += 512) ss = fmaf(in.y[i], in.y[i], ss);
         ss = fh_wave_sum(ss);
         if (lane == 0) red[wave] = ss;
         __syncthreads();
-        inv = 1.0f / sqrtf((((red[0] + red[1]) + (red[2] + red[3])) + ((red[4] + red[5]) + (red[6] + red[7]))) / (float)k + in.eps);
+        inv = 1.0f / sqrtf(mv_sum8(red) / (float)k + in.eps);
+    } else if (!(k & 3) && !in.x_out && !in.state && !mu) { // a plain copy
+#pragma unroll 4
+        for (int i = tid * 4; i < kp; i += 2048) *(float4 *)(xs + i) = i < k ? *(const float4 *)(in.x + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+        return;
     }
-    const int pos = in.state ? *in.pos_dev : 0;
-    const float *before = in.state + ((pos - 1) & 1) * k;
-    float *here = in.state + (pos & 1) * k;
     for (int i = tid; i < kp; i += 512) {
         float v = 0.f;
         if (i < k) {
             v = in.x[i];
             if (in.y) v += in.y[i] * inv * in.w[i];
-            if (blockIdx.x == 0) {
+            if (one) {
                 if (in.x_out) in.x_out[i] = v;
                 if (in.state) here[i] = v;
             }
-            if (seg.mu) v = fmaf((pos > 0 ? before[i] : 0.f) - v, seg.mu[i], v);
+            if (mu) v = fmaf((shift ? before[i] : 0.f) - v, mu[i], v);
         }
         xs[i] = v;
     }
+}
+
+// Normed group by group and gated.
+__device__ __forceinline__ void mv_gated(const FhMvAdd &in, int k, int kp, float *xs, float *ginv) {
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, gl = k / in.groups;
+#pragma unroll 4
+    for (int i = tid; i < kp; i += 512) xs[i] = i < k ? in.x[i] : 0.f;
+    __syncthreads();
+    for (int g = wave; g < in.groups; g += 8) {
+        float ss = 0.f;
+        for (int i = lane; i < gl; i += 64) ss = fmaf(xs[g * gl + i], xs[g * gl + i], ss);
+        ss = fh_wave_sum(ss);
+        if (lane == 0) ginv[g] = 1.0f / sqrtf(ss / (float)gl + in.eps) * in.scale;
+    }
+    __syncthreads();
+#pragma unroll 4
+    for (int i = tid; i < k; i += 512) {
+        float v = xs[i] * ginv[i / gl];
+        if (in.w) v *= in.w[in.w_len == k ? i : i % in.w_len];
+        xs[i] = v * fh_silu_f(in.gate[i]);
+    }
+}
+
+template <int ROWS, bool GATED>
+__global__ __launch_bounds__(512) void k_matvec_mix(FhMvAdd in, int k, int kp, MvMixes segs) {
+    constexpr int AHEAD = ROWS == 4 ? 3 : 8 / ROWS;
+    extern __shared__ __attribute__((aligned(16))) float xs[]; // [kp | groups]
+    __shared__ float red[8];
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    int tile = blockIdx.x, si = 0;
+    while (si + 1 < segs.n && tile >= segs.tiles[si]) tile -= segs.tiles[si++];
+    const FhMvMix seg = segs.s[si];
+    const int row0 = (tile * 8 + wave) * ROWS, pieces = (kp + 511) / 512;
+    const uint16_t *wr[ROWS];
+#pragma unroll
+    for (int r = 0; r < ROWS; r++) wr[r] = seg.w + (int64_t)(row0 + r < seg.n ? row0 + r : seg.n - 1) * kp + lane * 8;
+    uint4 u[AHEAD][ROWS];
+    auto fetch = [&](int i, uint4 *v) {
+        const bool ok = i * 512 + lane * 8 < kp;
+#pragma unroll
+        for (int r = 0; r < ROWS; r++) v[r] = ok ? *(const uint4 *)(wr[r] + i * 512) : uint4{0, 0, 0, 0};
+    };
+#pragma unroll
+    for (int i = 0; i < AHEAD; i++) fetch(i, u[i]);
+    if (GATED) mv_gated(in, k, kp, xs, xs + kp);
+    else mv_input(in, seg.mu, k, kp, xs, red);
     __syncthreads();
     float acc[ROWS];
 #pragma unroll
     for (int r = 0; r < ROWS; r++) acc[r] = 0.f;
-    for (int c = lane * 8; c < kp; c += 512) {
-        uint4 nxt[ROWS];
-        const bool more = c + 512 < kp;
+    for (int p = 0; p < pieces; p += AHEAD) {
 #pragma unroll
-        for (int r = 0; r < ROWS; r++) nxt[r] = more ? *(const uint4 *)(wr[r] + (c - lane * 8) + 512) : uint4{0, 0, 0, 0};
-        const float4 a = *(const float4 *)(xs + c), b = *(const float4 *)(xs + c + 4);
+        for (int i = 0; i < AHEAD; i++) {
+            uint4 cur[ROWS];
 #pragma unroll
-        for (int r = 0; r < ROWS; r++) {
-            acc[r] = fmaf(fh_bf_lo(cur[r].x), a.x, acc[r]);
-            acc[r] = fmaf(fh_bf_hi(cur[r].x), a.y, acc[r]);
-            acc[r] = fmaf(fh_bf_lo(cur[r].y), a.z, acc[r]);
-            acc[r] = fmaf(fh_bf_hi(cur[r].y), a.w, acc[r]);
-            acc[r] = fmaf(fh_bf_lo(cur[r].z), b.x, acc[r]);
-            acc[r] = fmaf(fh_bf_hi(cur[r].z), b.y, acc[r]);
-            acc[r] = fmaf(fh_bf_lo(cur[r].w), b.z, acc[r]);
-            acc[r] = fmaf(fh_bf_hi(cur[r].w), b.w, acc[r]);
-            cur[r] = nxt[r];
+            for (int r = 0; r < ROWS; r++) cur[r] = u[i][r];
+            fetch(p + i + AHEAD, u[i]);
+            const int c = (p + i) * 512 + lane * 8;
+            if (c >= kp) continue;
+            const float4 a = *(const float4 *)(xs + c), b = *(const float4 *)(xs + c + 4);
+#pragma unroll
+            for (int r = 0; r < ROWS; r++) {
+                acc[r] = fmaf(fh_bf_lo(cur[r].x), a.x, acc[r]);
+                acc[r] = fmaf(fh_bf_hi(cur[r].x), a.y, acc[r]);
+                acc[r] = fmaf(fh_bf_lo(cur[r].y), a.z, acc[r]);
+                acc[r] = fmaf(fh_bf_hi(cur[r].y), a.w, acc[r]);
+                acc[r] = fmaf(fh_bf_lo(cur[r].z), b.x, acc[r]);
+                acc[r] = fmaf(fh_bf_hi(cur[r].z), b.y, acc[r]);
+                acc[r] = fmaf(fh_bf_lo(cur[r].w), b.z, acc[r]);
+                acc[r] = fmaf(fh_bf_hi(cur[r].w), b.w, acc[r]);
+            }
         }
     }
 #pragma unroll
@@ -629,9 +737,20 @@ __global__ __launch_bounds__(512) void k_matvec_mix(FhMvAdd in, int k, int kp, M
             }
 }
 
+template <int ROWS, bool GATED>
+static fh_status matvec_mix_go(fh_device *dev, const FhMvAdd &in, int k, int kp, const MvMixes &ms, int tiles) {
+    const size_t lds = (size_t)(kp + (GATED ? in.groups : 0)) * 4;
+    FH_REQUIRE(lds <= 150 * 1024, "k = %d too long for the matvec", k);
+    if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, (const void *)k_matvec_mix<ROWS, GATED>, lds));
+    k_matvec_mix<ROWS, GATED><<<dim3((unsigned)tiles), 512, lds, dev->stream>>>(in, k, kp, ms);
+    FH_HIP(hipGetLastError());
+    return FH_OK;
+}
+
 fh_status fh_matvec_mix(fh_device *dev, const FhMvAdd &in, int k, const FhMvMix *segs, int n_segs) {
     FH_REQUIRE(n_segs >= 1 && n_segs <= FH_MV_MAX, "1 to %d matrices per launch", FH_MV_MAX);
     FH_REQUIRE(in.x && in.x != in.x_out && (!in.y || in.w) && (!in.state || in.pos_dev), "bad input of a decode product");
+    FH_REQUIRE(!in.gate || (!in.y && !in.state && in.groups > 0 && k % in.groups == 0), "bad gated input of a decode product");
     const int kp = (int)fh_pad64(k);
     MvMixes ms{};
     int64_t total = 0;
@@ -644,16 +763,11 @@ fh_status fh_matvec_mix(fh_device *dev, const FhMvAdd &in, int k, const FhMvMix 
         ms.tiles[i] = (segs[i].n + 8 * rows - 1) / (8 * rows);
         tiles += ms.tiles[i];
     }
-    const size_t lds = (size_t)kp * 4;
-    FH_REQUIRE(lds <= 120 * 1024, "k = %d too long for the matvec", k);
-    const void *fn = rows == 4 ? (const void *)k_matvec_mix<4> : rows == 2 ? (const void *)k_matvec_mix<2> : (const void *)k_matvec_mix<1>;
-    if (lds > 48 * 1024) FH_TRY(fh_kernel_lds(dev, fn, lds));
-    const dim3 grid((unsigned)tiles);
-    if (rows == 4) k_matvec_mix<4><<<grid, 512, lds, dev->stream>>>(in, k, kp, ms);
-    else if (rows == 2) k_matvec_mix<2><<<grid, 512, lds, dev->stream>>>(in, k, kp, ms);
-    else k_matvec_mix<1><<<grid, 512, lds, dev->stream>>>(in, k, kp, ms);
-    FH_HIP(hipGetLastError());
-    return FH_OK;
+    if (in.gate)
+        return rows == 4 ? matvec_mix_go<4, true>(dev, in, k, kp, ms, tiles) : rows == 2 ? matvec_mix_go<2, true>(dev, in, k, kp, ms, tiles)
+                                                                                        : matvec_mix_go<1, true>(dev, in, k, kp, ms, tiles);
+    return rows == 4 ? matvec_mix_go<4, false>(dev, in, k, kp, ms, tiles) : rows == 2 ? matvec_mix_go<2, false>(dev, in, k, kp, ms, tiles)
+                                                                                     : matvec_mix_go<1, false>(dev, in, k, kp, ms, tiles);
 }
 
 // ------------------------------------------------------------------------------ fh_qmatmul on bf16 rows

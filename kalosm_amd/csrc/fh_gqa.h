@@ -51,22 +51,53 @@ static inline size_t fh_gqa_lds(const FhGqa &a) {
 
 #ifdef __HIPCC__
 #include "fh_recurrent.h"
-// RMS norm (w NULL: none) and rotation of one head of `dim` values by one wavefront: raw -> dst, through `tmp` [dim] (LDS).
-__device__ __forceinline__ void fh_head_rotate(const FhGqa &a, const float *raw, const float *w, const float *ct, const float *st,
-                                               float mul, float *tmp, float *dst, int pad) {
+// One head of at most 256 values in a wavefront's registers: value, norm weight, and the cosine and sine of its pair.  The
+// request and the work are apart, so that several heads' requests can be on their way at once.
+struct FhHead { float x[4], w[4], c[4], s[4]; };
+__device__ __forceinline__ void fh_head_load(const FhGqa &a, const float *raw, const float *w, const float *ct, const float *st, FhHead &h) {
     const int lane = threadIdx.x & 63;
-    float inv = 1.f;
-    if (w) {
-        float ss = 0.f;
-        for (int i = lane; i < a.dim; i += 64) ss = fmaf(raw[i], raw[i], ss);
-        inv = 1.0f / sqrtf(fh_wave_sum(ss) / (float)a.dim + a.eps);
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+        const int i = lane + 64 * j, p = a.halves ? i < a.pairs ? i : i - a.pairs : i >> 1;
+        const bool ok = i < a.dim, turn = ok && i < 2 * a.pairs;
+        h.x[j] = ok ? raw[i] : 0.f;
+        h.w[j] = ok && w ? w[i] : 1.f;
+        h.c[j] = turn ? ct[p] : 1.f;
+        h.s[j] = turn ? st[p] : 0.f;
     }
-    for (int i = lane; i < a.dim; i += 64) tmp[i] = w ? raw[i] * inv * w[i] : raw[i];
+}
+// RMS norm (norm 0: none) and rotation: dst [pad] times mul, through `tmp` [dim] (LDS).
+__device__ __forceinline__ void fh_head_rotate(const FhGqa &a, FhHead &h, int norm, float mul, float *tmp, float *dst, int pad) {
+    const int lane = threadIdx.x & 63;
+    if (norm) {
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < 4; j++) ss = fmaf(h.x[j], h.x[j], ss);
+        const float inv = 1.0f / sqrtf(fh_wave_sum(ss) / (float)a.dim + a.eps);
+#pragma unroll
+        for (int j = 0; j < 4; j++) h.x[j] *= inv * h.w[j];
+    }
+#pragma unroll
+    for (int j = 0; j < 4; j++)
+        if (lane + 64 * j < a.dim) tmp[lane + 64 * j] = h.x[j];
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-    for (int i = lane; i < pad; i += 64)
-        dst[i] = i < a.dim ? fh_rotated([&](int j) { return tmp[j]; }, i, a.pairs, a.halves, ct, st) * mul : 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+        const int i = lane + 64 * j;
+        if (i >= pad) break;
+        float v = 0.f;
+        if (i < a.dim) {
+            v = h.x[j];
+            if (i < 2 * a.pairs) {
+                const bool second = a.halves ? i >= a.pairs : i & 1;
+                const float o = tmp[a.halves ? second ? i - a.pairs : i + a.pairs : i ^ 1];
+                v = v * h.c[j] + (second ? o : -o) * h.s[j];
+            }
+        }
+        dst[i] = v * mul;
+    }
 }
 
 // Workgroup b of fh_gqa_blocks: up to FH_GQA_HEADS query heads of one key head against one part of the cache.  The 16 lanes
@@ -97,18 +128,19 @@ __device__ __forceinline__ void fh_gqa_step(const FhGqa &a, const float *proj, T
     };
     if (k0 + rg < k1) fetch(k0 + rg); // requested before the query is worked on; this position's row is replaced below
     const float *ct = a.cos_t + (int64_t)pos * a.pairs, *st = a.sin_t + (int64_t)pos * a.pairs;
-    if (wave < nh) {
-        const float *raw = proj + a.col_q + (h0 + wave) * a.dim;
-        fh_head_rotate(a, raw, a.q_norm, ct, st, a.scale * LOG2E, od + wave * a.dnp, sq + wave * a.dnp, a.dnp);
+    FhHead hq, hk;
+    float hv = 0.f;
+    if (wave < nh) fh_head_load(a, proj + a.col_q + (h0 + wave) * a.dim, a.q_norm, ct, st, hq);
+    if (own) {
+        if (wave == 0) fh_head_load(a, proj + a.col_k + kh * a.dim, a.k_norm, ct, st, hk);
+        if (tid < a.vdim) hv = proj[a.col_v + kh * a.vdim + tid];
     }
+    if (wave < nh) fh_head_rotate(a, hq, a.q_norm != nullptr, a.scale * LOG2E, od + wave * a.dnp, sq + wave * a.dnp, a.dnp);
+    if (own && wave == 0) fh_head_rotate(a, hk, a.k_norm != nullptr, 1.f, od, sk, a.dnp);
     __syncthreads();
     if (own) {
-        if (wave == 0) fh_head_rotate(a, proj + a.col_k + kh * a.dim, a.k_norm, ct, st, 1.f, od, sk, a.dnp);
-        else
-            for (int i = tid - 64; i < a.dvp; i += 192) sv[i] = i < a.vdim ? proj[a.col_v + kh * a.vdim + i] : 0.f;
-        __syncthreads();
         for (int i = tid; i < a.dnp; i += 256) sk[i] = fh_up(fh_to<T>(sk[i])); // as the cache holds it
-        for (int i = tid; i < a.dvp; i += 256) sv[i] = fh_up(fh_to<T>(sv[i]));
+        for (int i = tid; i < a.dvp; i += 256) sv[i] = fh_up(fh_to<T>(hv)); // dvp is at most 256
         if (hg == 0) {
             T *dst = ring + (int64_t)mine * row;
             for (int i = tid; i < a.dnp; i += 256) dst[kh * a.dnp + i] = fh_to<T>(sk[i]);

@@ -12,7 +12,10 @@ __global__ __launch_bounds__(256) void k_gqa_rows(FhGqa a, const float *__restri
     if (job < a.heads + a.kv_heads) {
         const bool key = job >= a.heads;
         const int h = key ? job - a.heads : job, pad = key ? a.dnp : dq;
-        fh_head_rotate(a, p + (key ? a.col_k : a.col_q) + h * a.dim, key ? a.k_norm : a.q_norm, ct, st, 1.f, tmp[wave], dst[wave], pad);
+        const float *norm = key ? a.k_norm : a.q_norm;
+        FhHead x;
+        fh_head_load(a, p + (key ? a.col_k : a.col_q) + h * a.dim, norm, ct, st, x);
+        fh_head_rotate(a, x, norm != nullptr, 1.f, tmp[wave], dst[wave], pad);
         T *o = key ? kn + ((int64_t)(old + t) * a.kv_heads + h) * a.dnp : q + ((int64_t)t * a.heads + h) * dq;
         for (int i = lane; i < pad; i += 64) o[i] = fh_to<T>(dst[wave][i]); // a lane reads back what it wrote
     } else if (job < a.heads + 2 * a.kv_heads) {

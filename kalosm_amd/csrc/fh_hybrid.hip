@@ -863,14 +863,22 @@ fh_status Hybrid::step_apart(Layer &l) {
         FH_TRY(fh_matvec_mix(dev, in, d_model, &seg, 1));
     }
     FH_TRY(fh_step_mixers(dev, dtype, st, l.cache));
-    FH_TRY(fh_step_mix_out(dev, st, l.cache));
     auto plain = [&](const float *v, int k, const fh_qmatrix *q) {
         FhMvAdd a;
         a.x = v;
         const FhMvMix seg{(const uint16_t *)q->data, nullptr, mix, d_model, FH_MV_ACT_NONE};
         return fh_matvec_mix(dev, a, k, &seg, 1);
     };
-    FH_TRY(plain(qa, l.inner, l.wo));
+    if (l.kind == MIX_PAIR) {
+        FH_TRY(fh_step_mix_out(dev, st, l.cache));
+        FH_TRY(plain(qa, l.inner, l.wo));
+    } else { // norm and gate on the way into the output projection
+        FhMvAdd a;
+        a.x = o, a.eps = eps, a.gate = proj + l.rec.col_g, a.groups = l.rec.norm_groups, a.w = l.rec.norm, a.w_len = l.rec.norm_len;
+        a.scale = l.rec.out_scale;
+        const FhMvMix seg{(const uint16_t *)l.wo->data, nullptr, mix, d_model, FH_MV_ACT_NONE};
+        FH_TRY(fh_matvec_mix(dev, a, l.inner, &seg, 1));
+    }
     pend = l.norm;
     if (!l.ff) return FH_OK;
     const FhMvMix up{(const uint16_t *)l.up->data, nullptr, act1, l.ff, FH_MV_ACT_RELU2};

@@ -35,20 +35,24 @@ __global__ __launch_bounds__(256) void k_rec_prep(FhRecurrent r, const float *__
     }
 }
 
-// Retention: rotated queries and keys, values as they are, constant decays.  One workgroup per token.
+// Retention: rotated queries and keys, values as they are, constant decays.  grid (s, groups of four jobs): one wavefront per
+// head of q, of k, of v.
 __global__ __launch_bounds__(256) void k_rec_rotate(FhRecurrent r, const float *__restrict__ proj, int64_t ldp, int pos, FhRecWork w, int dp) {
-    const int t = blockIdx.x, tid = threadIdx.x, inner = r.heads * r.vdim;
+    const int t = blockIdx.x, lane = threadIdx.x & 63, job = (int)blockIdx.y * 4 + (threadIdx.x >> 6), part = job / r.heads, h = job % r.heads;
     const float *row = proj + (int64_t)t * ldp;
-    const float *ct = r.cos_t + (int64_t)(pos + t) * r.pairs, *st = r.sin_t + (int64_t)(pos + t) * r.pairs;
-    for (int i = tid; i < 2 * r.heads * dp; i += 256) {
-        const int h = i / dp % r.heads, c = i % dp;
-        const bool key = i >= r.heads * dp;
-        const float *x = row + (key ? r.col_k : r.col_q) + h * r.dim;
-        const float v = c < r.dim ? fh_rotated([&](int j) { return x[j]; }, c, r.pairs, r.halves, ct, st) * (key ? r.k_scale : r.q_scale) : 0.f;
-        (key ? w.k : w.q)[((int64_t)t * r.heads + h) * dp + c] = v;
+    if (part >= 3) return;
+    if (part == 2) {
+        float *dst = w.v + (int64_t)t * r.heads * r.vdim + h * r.vdim;
+        for (int i = lane; i < r.vdim; i += 64) dst[i] = row[r.col_v + h * r.vdim + i];
+        if (lane == 0) w.la[(int64_t)t * r.heads + h] = r.log_decay[h], w.beta[(int64_t)t * r.heads + h] = 1.f;
+        return;
     }
-    for (int i = tid; i < inner; i += 256) w.v[(int64_t)t * inner + i] = row[r.col_v + i];
-    for (int h = tid; h < r.heads; h += 256) w.la[(int64_t)t * r.heads + h] = r.log_decay[h], w.beta[(int64_t)t * r.heads + h] = 1.f;
+    const float *ct = r.cos_t + (int64_t)(pos + t) * r.pairs, *st = r.sin_t + (int64_t)(pos + t) * r.pairs;
+    const float *x = row + (part ? r.col_k : r.col_q) + h * r.dim, mul = part ? r.k_scale : r.q_scale;
+    float *dst = (part ? w.k : w.q) + ((int64_t)t * r.heads + h) * dp;
+#pragma unroll 4
+    for (int i = lane; i < dp; i += 64)
+        dst[i] = i < r.dim ? fh_rotated([&](int j) { return x[j]; }, i, r.pairs, r.halves, ct, st) * mul : 0.f;
 }
 
 // Projections of the portion's last `taps` tokens into the ring, after every reader of its old rows.
@@ -332,7 +336,9 @@ __global__ __launch_bounds__(256) void k_rec_chunk_prep(FhRecurrent r, FhRecWork
 }
 
 // Channel decay: one workgroup per (chunk, head).  Sums of la start anew in every block of 16 tokens, so that a fast decay
-// ahead of a block takes no digits from the sums inside it; longer ones are put together from those.
+// ahead of a block takes no digits from the sums inside it; longer ones are put together from those.  They are base-2
+// logarithms: no exponent is positive, so that v_exp_f32 does as it is (results below 2^-126 count as zero).
+__device__ __forceinline__ float rec_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
 template <int DP>
 __global__ __launch_bounds__(256) void k_rec_channel_prep(FhRecurrent r, FhRecRows in, RecChunks c, int s) {
     constexpr int LD = DP + 4;
@@ -347,7 +353,7 @@ __global__ __launch_bounds__(256) void k_rec_channel_prep(FhRecurrent r, FhRecRo
         const int64_t o = (int64_t)(t0 + t) * nq + h * r.dim + x;
         sk[t * LD + x] = ok ? in.k[o] : 0.f;
         sq[t * LD + x] = ok ? in.q[o] : 0.f;
-        sc[(t / 16 * 17 + t % 16 + 1) * LD + x] = ok ? fh_rec_la(in.z[o] + r.w0[h * r.dim + x]) : 0.f; // nothing is forgotten past the end
+        sc[(t / 16 * 17 + t % 16 + 1) * LD + x] = ok ? fh_rec_la(in.z[o] + r.w0[h * r.dim + x]) * 1.4426950408889634f : 0.f; // nothing is forgotten past the end
     }
     for (int x = tid; x < DP; x += 256) ub[x] = x < r.dim ? r.bonus[h * r.dim + x] : 0.f;
     __syncthreads();
@@ -374,14 +380,14 @@ __global__ __launch_bounds__(256) void k_rec_channel_prep(FhRecurrent r, FhRecRo
         for (int x = 0; x < DP / 16; x++) {
             const int o = 16 * x + 4 * g, t = 16 * wave + li;
             const float4 cq = *(const float4 *)(sc + (17 * wave + li) * LD + o), q = *(const float4 *)(sq + t * LD + o);
-            const float4 qa = make_float4(q.x * expf(cq.x), q.y * expf(cq.y), q.z * expf(cq.z), q.w * expf(cq.w));
+            const float4 qa = make_float4(q.x * rec_exp2(cq.x), q.y * rec_exp2(cq.y), q.z * rec_exp2(cq.z), q.w * rec_exp2(cq.w));
 #pragma unroll
             for (int b = 0; b < 3; b++) {
                 if (b >= wave) break;
                 const float4 k = *(const float4 *)(sk + (16 * b + li) * LD + o);
                 float f[4];
 #pragma unroll
-                for (int e = 0; e < 4; e++) f[e] = expf(rest(b, li + 1, o + e) + blocks(b + 1, wave, o + e));
+                for (int e = 0; e < 4; e++) f[e] = rec_exp2(rest(b, li + 1, o + e) + blocks(b + 1, wave, o + e));
                 off[b] = mma4(qa, make_float4(k.x * f[0], k.y * f[1], k.z * f[2], k.w * f[3]), off[b]);
             }
         }
@@ -402,7 +408,7 @@ __global__ __launch_bounds__(256) void k_rec_channel_prep(FhRecurrent r, FhRecRo
                 if (u == t) f = *(const float4 *)(ub + x);
                 else {
                     const float4 ct = *(const float4 *)(sc + (17 * wave + 4 * g + e) * LD + x), cu = *(const float4 *)(sc + (17 * wave + li + 1) * LD + x);
-                    f = make_float4(expf(ct.x - cu.x), expf(ct.y - cu.y), expf(ct.z - cu.z), expf(ct.w - cu.w));
+                    f = make_float4(rec_exp2(ct.x - cu.x), rec_exp2(ct.y - cu.y), rec_exp2(ct.z - cu.z), rec_exp2(ct.w - cu.w));
                 }
                 a = fmaf(q.x * k.x, f.x, fmaf(q.y * k.y, f.y, fmaf(q.z * k.z, f.z, fmaf(q.w * k.w, f.w, a))));
             }
@@ -410,13 +416,13 @@ __global__ __launch_bounds__(256) void k_rec_channel_prep(FhRecurrent r, FhRecRo
     }
     for (int i = tid; i < 64 * DP; i += 256) {
         const int t = i / DP, x = i % DP;
-        c.q[(hc * 64 + t) * DP + x] = sq[t * LD + x] * expf(blocks(0, t / 16, x) + sc[(t / 16 * 17 + t % 16) * LD + x]);
+        c.q[(hc * 64 + t) * DP + x] = sq[t * LD + x] * rec_exp2(blocks(0, t / 16, x) + sc[(t / 16 * 17 + t % 16) * LD + x]);
     }
     for (int i = tid; i < DP * 64; i += 256) {
         const int t = i & 63, x = i >> 6;
-        c.kt[hc * DP * 64 + i] = sk[t * LD + x] * expf(rest(t / 16, t % 16 + 1, x) + blocks(t / 16 + 1, 4, x));
+        c.kt[hc * DP * 64 + i] = sk[t * LD + x] * rec_exp2(rest(t / 16, t % 16 + 1, x) + blocks(t / 16 + 1, 4, x));
     }
-    for (int x = tid; x < DP; x += 256) c.f[hc * DP + x] = expf(blocks(0, 4, x));
+    for (int x = tid; x < DP; x += 256) c.f[hc * DP + x] = rec_exp2(blocks(0, 4, x));
 }
 
 // grid (blocks of 16 value columns, heads), four wavefronts.  Wavefront w works out rows 16 w .. + 15 of U and O and rows
@@ -627,7 +633,7 @@ fh_status fh_recurrent_prefill(fh_device *dev, int dtype, const FhRecurrent &r, 
                                int64_t ldp, int s, int pos, const FhRecWork &w, void *y, int kp) {
     hipStream_t str = dev->stream;
     const int dp = fh_rec_dp(r);
-    if (r.kind == FH_REC_RETENTION) k_rec_rotate<<<dim3((unsigned)s), 256, 0, str>>>(r, proj, ldp, pos, w, dp);
+    if (r.kind == FH_REC_RETENTION) k_rec_rotate<<<dim3((unsigned)s, (unsigned)((3 * r.heads + 3) / 4)), 256, 0, str>>>(r, proj, ldp, pos, w, dp);
     else {
         const int nq = r.kv_heads * r.dim, channels = fh_rec_channels(r);
         const size_t lds = (size_t)2 * nq * 4;

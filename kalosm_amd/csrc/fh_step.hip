@@ -351,20 +351,34 @@ __device__ __forceinline__ void linear_step(const FhMixStep &st, int pos, int b,
     float o = 0.f;
     if (r.kind == FH_REC_CHANNEL) {
         float *g = lds, *t1 = lds + 256; // [d], [rp]
+        // every request goes out before the first wait
+        uint4 w2[RPT];
+        float kk[RPT], qq[RPT], uu[RPT], w0[RPT];
+#pragma unroll
+        for (int i = 0; i < RPT; i++) { // the 16 lanes of a DPP row share a channel: 16 i + tid / 16
+            const int c = 16 * i + (tid >> 4);
+            const bool ok = c < d, in = i0 + i < d;
+            w2[i] = ok && rg * 8 < r.rp ? *(const uint4 *)(r.w2 + (int64_t)(h * d + c) * r.rp + rg * 8) : uint4{0, 0, 0, 0};
+            w0[i] = ok ? r.w0[h * d + c] : 0.f;
+            kk[i] = in ? k[i0 + i] : 0.f, qq[i] = in ? q[i0 + i] : 0.f, uu[i] = in ? r.bonus[h * d + i0 + i] : 0.f;
+        }
         for (int i = tid; i < r.rp; i += 256) t1[i] = i < r.rank ? st.proj[r.col_a + i] : 0.f;
         __syncthreads();
-        for (int c = tid >> 4; c < d; c += 16) {
-            float z = 0.f;
-            for (int i = rg * 8; i < r.rp; i += 128) z = dot8(*(const uint4 *)(r.w2 + (int64_t)(h * d + c) * r.rp + i), t1 + i, z);
+#pragma unroll
+        for (int i = 0; i < RPT; i++) {
+            const int c = 16 * i + (tid >> 4);
+            float z = rg * 8 < r.rp ? dot8(w2[i], t1 + rg * 8, 0.f) : 0.f;
+            if (c < d)
+                for (int x = rg * 8 + 128; x < r.rp; x += 128) z = dot8(*(const uint4 *)(r.w2 + (int64_t)(h * d + c) * r.rp + x), t1 + x, z);
             z = fh_row16_sum(z);
-            if (rg == 0) g[c] = expf(fh_rec_la(z + r.w0[h * d + c]));
+            if (rg == 0 && c < d) g[c] = expf(fh_rec_la(z + w0[i]));
         }
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < RPT; i++)
             if (i0 + i < d) {
-                const float kv = k[i0 + i] * v;
-                o = fmaf(fmaf(r.bonus[h * d + i0 + i], kv, S[i]), q[i0 + i], o);
+                const float kv = kk[i] * v;
+                o = fmaf(fmaf(uu[i], kv, S[i]), qq[i], o);
                 S[i] = fmaf(S[i], g[i0 + i], kv);
             }
     } else {
