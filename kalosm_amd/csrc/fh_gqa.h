@@ -118,15 +118,18 @@ __device__ __forceinline__ void fh_gqa_step(const FhGqa &a, const float *proj, T
     const bool own = mine >= k0 && mine < k1;
     float *sq = lds, *sk = sq + HB * a.dnp, *sv = sk + a.dnp, *od = sv + a.dvp;
     const T *kp_ = ring + kh * a.dnp, *vp_ = ring + a.kv_heads * a.dnp + kh * a.dvp;
-    FhPiece<T> nx[NP], ny[NP];
-    auto fetch = [&](int k) {
+    constexpr int U = NP == 1 ? 4 : 2; // rows of a lane group on their way
+    FhPiece<T> nx[U][NP], ny[U][NP];
+    auto fetch = [&](int k, FhPiece<T> *x, FhPiece<T> *y) {
+        const bool in = k < k1;
 #pragma unroll
         for (int i = 0; i < NP; i++) {
-            nx[i] = l16 + 16 * i < nk ? fh_ld_piece(kp_ + (int64_t)k * row + (l16 + 16 * i) * 8) : fh_zero_piece<T>();
-            ny[i] = l16 + 16 * i < nv ? fh_ld_piece(vp_ + (int64_t)k * row + (l16 + 16 * i) * 8) : fh_zero_piece<T>();
+            x[i] = in && l16 + 16 * i < nk ? fh_ld_piece(kp_ + (int64_t)k * row + (l16 + 16 * i) * 8) : fh_zero_piece<T>();
+            y[i] = in && l16 + 16 * i < nv ? fh_ld_piece(vp_ + (int64_t)k * row + (l16 + 16 * i) * 8) : fh_zero_piece<T>();
         }
     };
-    if (k0 + rg < k1) fetch(k0 + rg); // requested before the query is worked on; this position's row is replaced below
+#pragma unroll
+    for (int u = 0; u < U; u++) fetch(k0 + rg + 16 * u, nx[u], ny[u]); // before the query is worked on; this position's row is replaced below
     const float *ct = a.cos_t + (int64_t)pos * a.pairs, *st = a.sin_t + (int64_t)pos * a.pairs;
     FhHead hq, hk;
     float hv = 0.f;
@@ -160,36 +163,41 @@ __device__ __forceinline__ void fh_gqa_step(const FhGqa &a, const float *proj, T
                 o[i][j][e] = 0.f;
             }
     }
-    for (int k = k0 + rg; k < k1; k += 16) {
-        float c[NP][8], v[NP][8];
+    for (int kb = k0 + rg; kb < k1; kb += 16 * U) {
 #pragma unroll
-        for (int j = 0; j < NP; j++)
-#pragma unroll
-            for (int e = 0; e < 8; e++) c[j][e] = fh_up(nx[j].v[e]), v[j][e] = fh_up(ny[j].v[e]);
-        if (k + 16 < k1) fetch(k + 16);
-        if (k == mine)
+        for (int u = 0; u < U; u++) {
+            const int k = kb + 16 * u;
+            float c[NP][8], v[NP][8];
 #pragma unroll
             for (int j = 0; j < NP; j++)
 #pragma unroll
-                for (int e = 0; e < 8; e++) {
-                    c[j][e] = l16 + 16 * j < nk ? sk[(l16 + 16 * j) * 8 + e] : 0.f;
-                    v[j][e] = l16 + 16 * j < nv ? sv[(l16 + 16 * j) * 8 + e] : 0.f;
-                }
+                for (int e = 0; e < 8; e++) c[j][e] = fh_up(nx[u][j].v[e]), v[j][e] = fh_up(ny[u][j].v[e]);
+            fetch(k + 16 * U, nx[u], ny[u]);
+            if (k >= k1) continue; // the same for the 16 lanes of a row
+            if (k == mine)
 #pragma unroll
-        for (int i = 0; i < HB; i++) {
-            float d = 0.f;
+                for (int j = 0; j < NP; j++)
 #pragma unroll
-            for (int j = 0; j < NP; j++)
+                    for (int e = 0; e < 8; e++) {
+                        c[j][e] = l16 + 16 * j < nk ? sk[(l16 + 16 * j) * 8 + e] : 0.f;
+                        v[j][e] = l16 + 16 * j < nv ? sv[(l16 + 16 * j) * 8 + e] : 0.f;
+                    }
 #pragma unroll
-                for (int e = 0; e < 8; e++) d = fmaf(q[i][j][e], c[j][e], d);
-            d = fh_row16_sum(d);
-            const float mn = fmaxf(m[i], d), r = exp2f(m[i] - mn), w = exp2f(d - mn);
-            l[i] = l[i] * r + w;
-            m[i] = mn;
+            for (int i = 0; i < HB; i++) {
+                float d = 0.f;
 #pragma unroll
-            for (int j = 0; j < NP; j++)
+                for (int j = 0; j < NP; j++)
 #pragma unroll
-                for (int e = 0; e < 8; e++) o[i][j][e] = fmaf(w, v[j][e], o[i][j][e] * r);
+                    for (int e = 0; e < 8; e++) d = fmaf(q[i][j][e], c[j][e], d);
+                d = fh_row16_sum(d);
+                const float mn = fmaxf(m[i], d), r = exp2f(m[i] - mn), w = exp2f(d - mn);
+                l[i] = l[i] * r + w;
+                m[i] = mn;
+#pragma unroll
+                for (int j = 0; j < NP; j++)
+#pragma unroll
+                    for (int e = 0; e < 8; e++) o[i][j][e] = fmaf(w, v[j][e], o[i][j][e] * r);
+            }
         }
     }
     // the four row groups of a wavefront, then the four wavefronts through the LDS

@@ -347,13 +347,24 @@ __global__ __launch_bounds__(256) void k_rec_channel_prep(FhRecurrent r, FhRecRo
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, li = lane & 15, g = lane >> 4;
     const int ch = blockIdx.x, h = blockIdx.y, t0 = ch * 64, nq = r.heads * r.dim;
     const int64_t hc = (int64_t)ch * r.heads + h;
-    for (int i = tid; i < 64 * DP; i += 256) {
-        const int t = i / DP, x = i % DP;
-        const bool ok = t0 + t < s && x < r.dim;
-        const int64_t o = (int64_t)(t0 + t) * nq + h * r.dim + x;
-        sk[t * LD + x] = ok ? in.k[o] : 0.f;
-        sq[t * LD + x] = ok ? in.q[o] : 0.f;
-        sc[(t / 16 * 17 + t % 16 + 1) * LD + x] = ok ? fh_rec_la(in.z[o] + r.w0[h * r.dim + x]) * 1.4426950408889634f : 0.f; // nothing is forgotten past the end
+    constexpr int B = 8; // requests of a thread and array on their way; places outside read a valid address
+    for (int i0 = tid; i0 < 64 * DP; i0 += 256 * B) {
+        float k[B], q[B], z[B];
+#pragma unroll
+        for (int j = 0; j < B; j++) {
+            const int i = i0 + 256 * j, t = t0 + i / DP, x = i % DP;
+            const int64_t o = (int64_t)(t < s ? t : s - 1) * nq + h * r.dim + (x < r.dim ? x : r.dim - 1);
+            k[j] = in.k[o], q[j] = in.q[o], z[j] = in.z[o];
+        }
+#pragma unroll
+        for (int j = 0; j < B; j++) {
+            const int i = i0 + 256 * j, t = i / DP, x = i % DP;
+            const bool ok = t0 + t < s && x < r.dim;
+            sk[t * LD + x] = ok ? k[j] : 0.f;
+            sq[t * LD + x] = ok ? q[j] : 0.f;
+            // nothing is forgotten past the end
+            sc[(t / 16 * 17 + t % 16 + 1) * LD + x] = ok ? fh_rec_la(z[j] + r.w0[h * r.dim + x]) * 1.4426950408889634f : 0.f;
+        }
     }
     for (int x = tid; x < DP; x += 256) ub[x] = x < r.dim ? r.bonus[h * r.dim + x] : 0.f;
     __syncthreads();
