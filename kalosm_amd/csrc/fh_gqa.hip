@@ -2,10 +2,10 @@
 #include "fh_gqa.h"
 
 // grid (s, groups of four heads): one wavefront per head - queries first, then keys, then values.
-template <typename T>
+template <typename T, int J>
 __global__ __launch_bounds__(256) void k_gqa_rows(FhGqa a, const float *__restrict__ proj, int64_t ldp, int old, int pos, int dq,
                                                   T *__restrict__ q, T *__restrict__ kn, T *__restrict__ vr) {
-    __shared__ float tmp[4][256], dst[4][256];
+    __shared__ float tmp[4][64 * J], dst[4][64 * J];
     const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63, job = (int)blockIdx.y * 4 + wave;
     const float *p = proj + (int64_t)t * ldp;
     const float *ct = a.cos_t + (int64_t)(pos + t) * a.pairs, *st = a.sin_t + (int64_t)(pos + t) * a.pairs;
@@ -13,9 +13,9 @@ __global__ __launch_bounds__(256) void k_gqa_rows(FhGqa a, const float *__restri
         const bool key = job >= a.heads;
         const int h = key ? job - a.heads : job, pad = key ? a.dnp : dq;
         const float *norm = key ? a.k_norm : a.q_norm;
-        FhHead x;
-        fh_head_load(a, p + (key ? a.col_k : a.col_q) + h * a.dim, norm, ct, st, x);
-        fh_head_rotate(a, x, norm != nullptr, 1.f, tmp[wave], dst[wave], pad);
+        FhHead<J> x;
+        fh_head_load<J>(a, p + (key ? a.col_k : a.col_q) + h * a.dim, norm, ct, st, x);
+        fh_head_rotate<J>(a, x, norm != nullptr, 1.f, tmp[wave], dst[wave]);
         T *o = key ? kn + ((int64_t)(old + t) * a.kv_heads + h) * a.dnp : q + ((int64_t)t * a.heads + h) * dq;
         for (int i = lane; i < pad; i += 64) o[i] = fh_to<T>(dst[wave][i]); // a lane reads back what it wrote
     } else if (job < a.heads + 2 * a.kv_heads) {
@@ -68,7 +68,9 @@ static fh_status gqa_prefill_t(fh_device *dev, int dtype, const FhGqa &a, fh_kvc
     FH_REQUIRE(dq && w.ldt >= keys, "attention over %d query dimensions (at most 256)", a.dim);
     FH_REQUIRE(pos + s <= cache->capacity || cache->capacity == cache->max_len, "cache of %d rows has not grown to %d", cache->capacity, pos + s);
     T *q = (T *)w.q, *kn = (T *)w.kn, *vr = (T *)w.vr, *ring = (T *)cache->k;
-    k_gqa_rows<T><<<dim3((unsigned)s, (unsigned)((a.heads + 2 * a.kv_heads + 3) / 4)), 256, 0, str>>>(a, proj, ldp, old, pos, dq, q, kn, vr);
+    const dim3 rows((unsigned)s, (unsigned)((a.heads + 2 * a.kv_heads + 3) / 4));
+    if (dq <= 128) k_gqa_rows<T, 2><<<rows, 256, 0, str>>>(a, proj, ldp, old, pos, dq, q, kn, vr);
+    else k_gqa_rows<T, 4><<<rows, 256, 0, str>>>(a, proj, ldp, old, pos, dq, q, kn, vr);
     if (old > 0) k_gqa_old<T><<<dim3((unsigned)old), 256, 0, str>>>(a, ring, cache->capacity, kept, lo - kept, kn, vr);
     k_gqa_append<T><<<dim3((unsigned)s), 256, 0, str>>>(a, kn, vr, old, pos, s, ring, cache->capacity);
     k_gqa_values<T><<<dim3((unsigned)((keys + 63) / 64), (unsigned)((a.kv_heads * a.dvp + 63) / 64)), 256, 0, str>>>(a, vr, keys, (T *)w.vt, w.ldt);

@@ -335,6 +335,19 @@ fh_status fh_step_out(fh_device *dev, const FhStep &st) {
 }
 
 // ------------------------------------------------------------------------------ mixers of sublayers normed at their end
+// RPT consecutive values from i0 on, those past d repeat the last one.
+template <int RPT>
+__device__ __forceinline__ void rec_load(float *v, const float *p, int i0, int d, bool full) {
+    constexpr int N = RPT < 4 ? RPT : 4;
+    if (full) {
+#pragma unroll
+        for (int i = 0; i < RPT; i += N) __builtin_memcpy(v + i, p + i0 + i, N * 4);
+    } else {
+#pragma unroll
+        for (int i = 0; i < RPT; i++) v[i] = p[i0 + i < d ? i0 + i : d - 1];
+    }
+}
+
 // One step of a recurrence without a short convolution: workgroup b takes 16 columns of one head's state.
 template <int RPT>
 __device__ __forceinline__ void linear_step(const FhMixStep &st, int pos, int b, float *lds) {
@@ -344,8 +357,10 @@ __device__ __forceinline__ void linear_step(const FhMixStep &st, int pos, int b,
     const bool live = col < r.vdim;
     float *sp = st.state.s + ((int64_t)h * r.vdim + (live ? col : r.vdim - 1)) * d;
     float S[RPT];
+    const bool full = d == 16 * RPT; // whole rows in float4s
+    rec_load<RPT>(S, sp, i0, d, full);
 #pragma unroll
-    for (int i = 0; i < RPT; i++) S[i] = pos > 0 && i0 + i < d ? sp[i0 + i] : 0.f;
+    for (int i = 0; i < RPT; i++) S[i] = pos > 0 ? S[i] : 0.f;
     const float *q = st.proj + r.col_q + h * d, *k = st.proj + r.col_k + h * d;
     const float v = st.proj[r.col_v + h * r.vdim + (live ? col : r.vdim - 1)];
     float o = 0.f;
@@ -357,11 +372,16 @@ __device__ __forceinline__ void linear_step(const FhMixStep &st, int pos, int b,
 #pragma unroll
         for (int i = 0; i < RPT; i++) { // the 16 lanes of a DPP row share a channel: 16 i + tid / 16
             const int c = 16 * i + (tid >> 4);
-            const bool ok = c < d, in = i0 + i < d;
-            w2[i] = ok && rg * 8 < r.rp ? *(const uint4 *)(r.w2 + (int64_t)(h * d + c) * r.rp + rg * 8) : uint4{0, 0, 0, 0};
-            w0[i] = ok ? r.w0[h * d + c] : 0.f;
-            kk[i] = in ? k[i0 + i] : 0.f, qq[i] = in ? q[i0 + i] : 0.f, uu[i] = in ? r.bonus[h * d + i0 + i] : 0.f;
+            const int64_t cc = h * d + (c < d ? c : d - 1);
+            w2[i] = *(const uint4 *)(r.w2 + cc * r.rp + (rg * 8 < r.rp ? rg * 8 : 0));
+            w0[i] = r.w0[cc];
         }
+        rec_load<RPT>(kk, k, i0, d, full);
+        rec_load<RPT>(qq, q, i0, d, full);
+        rec_load<RPT>(uu, r.bonus + h * d, i0, d, full);
+#pragma unroll
+        for (int i = 0; i < RPT; i++) // rows past the end read nothing out
+            if (i0 + i >= d) kk[i] = 0.f, qq[i] = 0.f;
         for (int i = tid; i < r.rp; i += 256) t1[i] = i < r.rank ? st.proj[r.col_a + i] : 0.f;
         __syncthreads();
 #pragma unroll
@@ -375,32 +395,39 @@ __device__ __forceinline__ void linear_step(const FhMixStep &st, int pos, int b,
         }
         __syncthreads();
 #pragma unroll
-        for (int i = 0; i < RPT; i++)
-            if (i0 + i < d) {
-                const float kv = kk[i] * v;
-                o = fmaf(fmaf(uu[i], kv, S[i]), qq[i], o);
-                S[i] = fmaf(S[i], g[i0 + i], kv);
-            }
+        for (int i = 0; i < RPT; i++) {
+            const float kv = kk[i] * v;
+            o = fmaf(fmaf(uu[i], kv, S[i]), qq[i], o);
+            S[i] = fmaf(S[i], g[i0 + i], kv);
+        }
     } else {
         const float g = expf(r.log_decay[h]), *ct = r.cos_t + (int64_t)pos * r.pairs, *sn = r.sin_t + (int64_t)pos * r.pairs;
-        float *qk = lds; // [2 d]
-        for (int i = tid; i < 2 * d; i += 256) {
-            const float *x = i < d ? q : k;
-            qk[i] = fh_rotated([&](int j) { return x[j]; }, i < d ? i : i - d, r.pairs, r.halves, ct, sn) * (i < d ? r.q_scale : r.k_scale);
+        float *qk = lds; // [2][16 RPT], zeros from d on
+        for (int i = tid; i < 32 * RPT; i += 256) {
+            const bool key = i >= 16 * RPT;
+            const int c0 = i % (16 * RPT), c = c0 < d ? c0 : d - 1, p = r.halves ? c < r.pairs ? c : c - r.pairs : c >> 1;
+            const bool second = r.halves ? c >= r.pairs : c & 1, turn = c < 2 * r.pairs;
+            const float *x = key ? k : q;
+            const float y = x[c], z = x[!turn ? c : !r.halves ? c ^ 1 : second ? c - r.pairs : c + r.pairs];
+            const float co = ct[turn ? p : 0], si = sn[turn ? p : 0];
+            qk[i] = c0 < d ? (turn ? y * co + (second ? z * si : -z * si) : y) * (key ? r.k_scale : r.q_scale) : 0.f;
         }
         __syncthreads();
 #pragma unroll
-        for (int i = 0; i < RPT; i++)
-            if (i0 + i < d) {
-                S[i] = fmaf(qk[d + i0 + i], v, S[i] * g);
-                o = fmaf(S[i], qk[i0 + i], o);
-            }
+        for (int i = 0; i < RPT; i++) {
+            S[i] = fmaf(qk[16 * RPT + i0 + i], v, S[i] * g);
+            o = fmaf(S[i], qk[i0 + i], o);
+        }
     }
     o = fh_row16_sum(o);
+    if (!live) return;
+    if (full)
 #pragma unroll
-    for (int i = 0; i < RPT; i++)
-        if (live && i0 + i < d) sp[i0 + i] = S[i];
-    if (rg == 0 && live) st.o[h * r.vdim + col] = o;
+        for (int i = 0; i < RPT; i += RPT < 4 ? RPT : 4) __builtin_memcpy(sp + i0 + i, S + i, (RPT < 4 ? RPT : 4) * 4);
+    else
+        for (int i = 0; i < RPT; i++)
+            if (i0 + i < d) sp[i0 + i] = S[i];
+    if (rg == 0) st.o[h * r.vdim + col] = o;
 }
 
 template <typename T, int NP, int RPT>
@@ -416,7 +443,7 @@ static fh_status step_mixers_t(fh_device *dev, const FhMixStep &st, fh_kvcache *
     const int splits = st.attn ? fh_gqa_splits(cache) : 1, n_attn = st.attn ? fh_gqa_blocks(st.gqa, splits) : 0;
     const int n_rec = st.rec ? st.r.heads * ((st.r.vdim + 15) / 16) : 0, rpt = st.rec ? (st.r.dim + 15) / 16 : 1;
     size_t lds = st.attn ? fh_gqa_lds(st.gqa) : 0;
-    const size_t need = !st.rec ? 0 : (size_t)(st.r.kind == FH_REC_CHANNEL ? 256 + st.r.rp : 2 * st.r.dim) * 4;
+    const size_t need = !st.rec ? 0 : (size_t)(st.r.kind == FH_REC_CHANNEL ? 256 + st.r.rp : 512) * 4;
     lds = lds > need ? lds : need;
     FH_REQUIRE(lds <= 60 * 1024 && rpt <= 16, "mixers too wide for a decode step (%zu bytes of LDS)", lds);
     const dim3 grid((unsigned)(n_attn + n_rec));
