@@ -487,9 +487,10 @@ fh_status fh_llama_load_gguf(fh_llama *m, const fh_gguf *g);
 /* ---------------------------------------------------------------- any decoder
  * The handle all decoder families share.  fh_llama_decoder gives that of a Llama decoder (owned by the fh_llama);
  * fh_decoder_create / _open make one for a model that comes as a configuration text and a safetensors file, by the
- * configuration's "architecture" (registered: "Fidasun", whose configuration lists its layers).  dtype: FH_F32
- * (everything in 32 bits) or FH_DECODER_BF16 (operands of the matrix products in bf16; sums, scores, norms, routers,
- * recurrent states and the residual stream in 32 bits). */
+ * configuration's "architecture" (registered: "Fidasun" and "Zovovik", whose configurations list their layers).
+ * The context is ctx, or the configuration's "max_positions" where that is less.  dtype: FH_F32 (everything in 32
+ * bits) or FH_DECODER_BF16 (operands of the matrix products in bf16; sums, scores, norms, routers, recurrent states
+ * and the residual stream in 32 bits). */
 enum { FH_DECODER_BF16 = 2 };
 fh_status fh_llama_decoder(fh_llama *m, fh_decoder **out);
 fh_status fh_decoder_create(fh_device *dev, const char *config_json, int32_t dtype, int32_t ctx, fh_decoder **out);
